@@ -468,7 +468,10 @@ class ModelRunner:
 
     def memory_report(self) -> dict:
         if self.hybrid:
-            kv = sum(t.numel() * t.element_size() for c in self.kv for t in c.values())
+            def size(c) -> int:  # a side-by-side run's cache nests its two mixers
+                return sum(size(t) if isinstance(t, dict) else t.numel() * t.element_size() for t in c.values())
+
+            kv = sum(size(c) for c in self.kv)
         else:
             kv = (self.k_cache.numel() + self.v_cache.numel()) * self.k_cache.element_size()
         return {"kv_cache_bytes": kv, "kv_blocks": self.num_blocks, "block_size": BLOCK_SIZE,

@@ -175,11 +175,14 @@ class DenseSpec:
 class LayerSpec:
     """One decoder layer of a :class:`HybridConfig`: a token mixer (``kind`` names an entry of
     models/hybrid.py MIXERS, ``mixer`` holds that mixer's sizes and constants as sorted
-    (key, value) pairs so the spec stays hashable) and an optional feed-forward."""
+    (key, value) pairs so the spec stays hashable) and an optional feed-forward.  ``weights_of``: the
+    layer has no tensors of its own, it runs with that layer's (an equal spec) and a cache or state of
+    its own."""
 
     kind: str
     mixer: tuple
     mlp: Optional[object] = None  # MoESpec, DenseSpec or None
+    weights_of: Optional[int] = None
 
     @property
     def m(self) -> dict:
@@ -227,6 +230,20 @@ class HybridConfig:
     def traits(self) -> dict:
         return DESIGN_TRAITS[self.arch]
 
+    def owner(self, i: int) -> int:
+        """The layer whose tensors layer ``i`` uses: itself, or what its ``weights_of`` leads to."""
+        seen = []
+        while self.layers[i].weights_of is not None:
+            seen.append(i)
+            j = self.layers[i].weights_of
+            if not 0 <= j < len(self.layers) or j in seen:
+                raise ValueError(f"layer {seen[0]}: weights_of {j} leads to no layer with tensors of its own")
+            a, b = self.layers[i], self.layers[j]
+            if (a.kind, a.mixer, a.mlp) != (b.kind, b.mixer, b.mlp):
+                raise ValueError(f"layer {i}: weights_of {j}, but the two layers' entries differ")
+            i = j
+        return i
+
     def runs(self) -> list:
         """Execution order as (layer index, pass number or -1, first layer of its pass)."""
         n = len(self.layers)
@@ -255,8 +272,10 @@ class HybridConfig:
 #   ffn            the feed-forward family: "swiglu_topk" (gated experts, biased router, softmax over
 #                  the chosen logits, sigmoid-gated shared expert), "plain_softmax" (ungated
 #                  experts with erf-GELU, softmax over all logits and the chosen probabilities
-#                  used as they are, ungated shared expert, dense layers with xIELU) or "gated_gelu"
-#                  (dense layers down(gelu_tanh(gate h) * up h))
+#                  used as they are, ungated shared expert, dense layers with xIELU), "gated_gelu"
+#                  (dense layers down(gelu_tanh(gate h) * up h)), "relu_glu_grouped" (dense layers
+#                  down(relu(gate h) * up h), clamped gated experts with a group-limited sigmoid
+#                  router) or "relu_sq" (dense layers down(relu(up h)^2))
 #   max_position   positions a model accepts when its config.json does not say
 # and, where present (absent = the first value):
 #   scalar_norm    False / True: a block or final norm's weight is one number for all coordinates
@@ -269,6 +288,12 @@ class HybridConfig:
 #                  softmax denominator) / False
 #   norm           "rms" / "layer": block and final norms are RMSNorms, or layer norms with a weight
 #                  and no bias ((x - mean) / sqrt(variance + eps) * w)
+#   norm_bias      False / True: the layer norms also have a bias (the norm's name with ``.b``)
+#   post_norm      False / True: every sublayer's result passes a norm of its own before it joins the
+#                  stream: x += norm1b(mixer(norm1(x))), then x += norm2b(ff(norm2(x)))
+#   pair_norm      None / a number: a side-by-side layer's two results are each RMS-normed over the width
+#                  (weights ``mix.left.out`` / ``mix.right.out``) and their sum is multiplied by the number;
+#                  such layers have no left_scale / right_scale
 #   composite      config ``type`` -> {"left": (MIXERS entry, options), "right": (MIXERS entry, options)}:
 #                  a layer of that type runs two mixers side by side on the same normed input (their
 #                  constants under ``mixer.left`` / ``mixer.right``, tensors under ``mix.left.`` /
@@ -293,6 +318,13 @@ DESIGN_TRAITS = {
                             left=("rotary_attention", dict(rotary="pairs", qk_norm="before", values="keys", temp=False,
                                                            gate=False)),
                             right=("gated_linear", {}))}),
+    "dopivik": dict(block="sequential", one_plus_norm=False, learned_pos=False, token_shift=False,
+                    depth_average=False, ffn="relu_sq", max_position=1 << 17, norm="layer", norm_bias=True,
+                    post_norm=True, pair_norm=0.5,
+                    composite={
+                        "parallel": dict(
+                            left=("rotary_attention", dict(rotary="half", mask="chunk", temp=False, gate=True)),
+                            right=("gated_delta", dict(decay="head", gate="silu")))}),
 }
 
 
@@ -311,7 +343,8 @@ def hybrid_config_from_dict(c: dict, name: Optional[str] = None) -> HybridConfig
     ``width``, ``max_positions``, ``norm.eps``, ``logit_scale``, ``logit_softcap``, ``residual_mult``,
     ``embedding.scale``, ``token_side.dim``, ``loop`` {start, stop, times} and
     ``layers`` [{type, mixer {...}, mlp {kind: moe, expert.ff, expert.limit, router.experts, router.top,
-    router.scale, router.groups {count, keep}, shared.ff} | {kind: dense, ff} | null}].  Nested mixer keys are flattened with dots (``mask.size``)."""
+    router.scale, router.groups {count, keep}, shared.ff} | {kind: dense, ff} | null, weights_of: layer or
+    absent}].  Nested mixer keys are flattened with dots (``mask.size``)."""
     arch = str(c["architecture"]).lower()
     if arch not in DESIGN_TRAITS:
         raise ValueError(f"unknown architecture {c['architecture']!r} (known: {sorted(DESIGN_TRAITS)})")
@@ -333,7 +366,9 @@ def hybrid_config_from_dict(c: dict, name: Optional[str] = None) -> HybridConfig
                 moe = DenseSpec(ff=int(ml["ff"]))
             else:
                 raise ValueError(f"unsupported feed-forward kind {kind!r}")
-        layers.append(LayerSpec(kind=spec["type"], mixer=tuple(sorted(_flat(spec.get("mixer") or {}))), mlp=moe))
+        wo = spec.get("weights_of")
+        layers.append(LayerSpec(kind=spec["type"], mixer=tuple(sorted(_flat(spec.get("mixer") or {}))), mlp=moe,
+                                weights_of=None if wo is None else int(wo)))
     lp = c.get("loop")
     loop = (int(lp["start"]), int(lp["stop"]), int(lp["times"])) if lp else None
     if loop and not (0 <= loop[0] < loop[1] <= len(layers) and loop[2] >= 1):
@@ -377,6 +412,8 @@ def hybrid_config_to_dict(c: HybridConfig) -> dict:
             if s.mlp.route_scale != 1.0:
                 ml["router"]["scale"] = s.mlp.route_scale
         layers.append({"type": s.kind, "mixer": nest(s.mixer), "mlp": ml})
+        if s.weights_of is not None:
+            layers[-1]["weights_of"] = s.weights_of
     d = {"architecture": c.arch.capitalize(), "vocab": c.vocab_size, "width": c.d_model, "layers": layers,
          "max_positions": c.max_position, "norm": {"eps": c.norm_eps}, "logit_scale": c.logit_scale,
          "bos_id": c.bos_id, "eos_ids": list(c.eos_ids)}
@@ -482,3 +519,32 @@ LEVOVIK_TINY = _reg(HybridConfig(
                             dict(heads=2, kv_heads=2, dim=24, vdim=8, conv=4), 0.8, 0.5),
                       MoESpec(6, 3, 24, limit=2.0, groups=2, keep_groups=1, route_scale=2.5))),
     max_position=1 << 17, norm_eps=1e-5, logit_scale=0.6, embed_scale=9.0, side_dim=12, bos_id=1, eos_ids=(2,)))
+
+
+def _mamba1(inner, state, conv, dt_rank):
+    return LayerSpec("mamba1", tuple(sorted({"inner": inner, "state": state, "conv": conv, "dt_rank": dt_rank}.items())))
+
+
+def _wkv(heads, dim, w_rank=16):
+    return LayerSpec("wkv", tuple(sorted({"heads": heads, "dim": dim, "w_rank": w_rank}.items())))
+
+
+def _chunk_pair(left: dict, right: dict) -> LayerSpec:
+    return LayerSpec("parallel", tuple(sorted(_flat({"left": left, "right": right}))))
+
+
+# Small Dopivik-design model for CPU tests and GPU smoke runs (random weights): selective scan, wkv and
+# attention beside the delta rule, the last three layers sharing the tensors of earlier ones.
+_DOPIVIK_LAYERS = (
+    _with_mlp(_mamba1(112, 12, 4, 10), DenseSpec(144)),
+    _with_mlp(_chunk_pair(dict(heads=4, kv_heads=2, dim=16, vdim=24, scale=0.25, softcap=15.0, mask=dict(size=40),
+                               rot=dict(dims=8, base=10000.0)),
+                          dict(heads=4, kv_heads=2, dim=24, vdim=16, conv=3)), DenseSpec(96)),
+    _with_mlp(_wkv(3, 16, 8), None),
+    _with_mlp(_chunk_pair(dict(heads=2, kv_heads=2, dim=32, vdim=16, scale=0.2, softcap=30.0, mask=dict(size=24),
+                               rot=dict(dims=32, base=5000.0)),
+                          dict(heads=2, kv_heads=2, dim=16, vdim=40, conv=4)), None))
+DOPIVIK_TINY = _reg(HybridConfig(
+    name="dopivik-tiny", arch="dopivik", vocab_size=336, d_model=80,
+    layers=_DOPIVIK_LAYERS + tuple(dataclasses.replace(_DOPIVIK_LAYERS[j], weights_of=j) for j in (2, 0, 1)),
+    max_position=4096, norm_eps=1e-5, embed_scale=4.0, bos_id=1, eos_ids=(2,)))

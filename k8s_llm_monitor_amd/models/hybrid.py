@@ -1,11 +1,19 @@
 """Layer-list decoders: every layer names its token mixer (windowed attention with a softmax
-sink, the Mamba-2 recurrence, latent attention, rotary grouped-query attention or fixed-decay
-linear attention) and an optional feed-forward; a span of layers may run several times with shared
-weights.  ``Dunesun``, ``Kisutar`` and ``Bitonex`` are the designs served; mixers are registered by
+sink, the Mamba-1 and Mamba-2 recurrences, latent attention, rotary grouped-query attention, linear
+attention with fixed or learned decays, the gated delta rule, wkv time mixing, or two of these side by
+side) and an optional feed-forward; a span of layers may run several times with shared
+weights, and a layer may use another layer's tensors (``weights_of``).  ``Dunesun``, ``Kisutar``,
+``Bitonex``, ``Levovik`` and ``Dopivik`` are the designs served; mixers are registered by
 name (``MIXERS``) and feed-forward families by the design's ``ffn`` trait (``_ffn_for``), with their
 sizes and constants read from the layer's spec, so another layer-list design can reuse them in
 another order.  What a design fixes (block form, norm form, positions, token shift, depth average,
 gated residual, rotation layout) is models/config.DESIGN_TRAITS.
+
+Dopivik, per layer (sequential block with norms on both sides of a sublayer): ``x += norm1b(mixer(
+norm1(x)))``, then ``x += norm2b(ff(norm2(x)))``, all layer norms with a bias; the norm behind a sublayer,
+the sum into the fp32 stream and the next sublayer's norm are one launch (ops.hybrid.join_norm).  Its
+mixers: the selective scan (Mamba-1), wkv time mixing, and chunked softmax attention with capped scores
+beside the delta rule with one decay per head.
 
 Bitonex, per layer (sequential block): ``x += m * mixer(h) * sigmoid(R1 h + b1)`` with
 ``h = norm1(x)``, then the same with the feed-forward, ``norm2``, ``R2`` and ``b2`` (gated
@@ -356,7 +364,11 @@ class RotaryAttention:
       ``k.norm`` [dim], then turned) / "after" (turned, then divided by its root mean square, no weight);
     * ``sink`` False / True: a learned logit per query head (``sink``) joins the softmax denominator;
     * ``values`` "own" (``v`` projection) / "keys" (the values are the keys as projected, before norm
-      and turn; no ``v`` tensor, vdim = dim).
+      and turn; no ``v`` tensor, vdim = dim);
+    * ``mask`` "window" / "chunk" (a position sees the earlier ones of its own chunk of ``mask.size``
+      positions, counted from position 0).
+
+    ``softcap`` (absent: none): scores become ``softcap * tanh(score / softcap)``.
 
     ``tail``: extra rows for the input projection (see LatentAttention).  ``forward(..., proj=)``: the
     input projection computed by the caller (this mixer's columns of a wider GEMM)."""
@@ -374,6 +386,7 @@ class RotaryAttention:
             raise ValueError(f"{prefix}: heads {self.H} not a multiple of kv_heads {self.G}")
         self.scale = float(m.get("scale", 1.0 / math.sqrt(self.dk)))
         self.window = int(m.get("mask.size", 0) or 0)
+        self.chunked, self.cap = o.get("mask", "window") == "chunk", float(m.get("softcap", 0.0) or 0.0)
         self.base, self.rdims = float(m.get("rot.base", 10000.0)), int(m.get("rot.dims", self.dk))
         if self.rdims % 2 or not 0 <= self.rdims <= self.dk:
             raise ValueError(f"{prefix}: rot.dims {self.rdims} must be even and at most dim {self.dk}")
@@ -421,16 +434,16 @@ class RotaryAttention:
         hops.rotary_cache(proj, H, G, dk, dv, meta.positions, self.freq, self.pairs, self.temp, kc, vc, meta.slot_mapping,
                           norm=self.norm, qw=self.qn, kw=self.kn, eps=self.eps, v_from_k=self.v_from_k)
         args = (H, G, dk, dv, self.scale, self.window, self.sink)
+        kw = dict(sinks=self.sinks, chunked=self.chunked, cap=self.cap)
         if not meta.is_prefill:
-            o = hops.window_attention_decode(proj, kc, vc, meta.block_tables, meta.seq_lens, *args, vec=bool(self.fast),
-                                             sinks=self.sinks)
+            o = hops.window_attention_decode(proj, kc, vc, meta.block_tables, meta.seq_lens, *args, vec=bool(self.fast), **kw)
         else:
             nd = meta.num_decode
             o = hops.window_attention_prefill(proj[nd:], kc, vc, meta.cu_seqlens, meta.ctx_start, meta.block_tables,
-                                              *args, mfma=self.fast, sinks=self.sinks)
+                                              *args, mfma=self.fast, **kw)
             if nd:
                 od = hops.window_attention_decode(proj[:nd], kc, vc, meta.dec_block_tables, meta.dec_seq_lens, *args,
-                                                  vec=bool(self.fast), sinks=self.sinks)
+                                                  vec=bool(self.fast), **kw)
                 o = torch.cat([od, o])
         if self.has_gate:
             o = hops.sigmoid_gate(o, proj, self.g_col)
@@ -517,7 +530,11 @@ class GatedDeltaMixer:
     ``S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q``.  Each head's o is RMS-normed
     over vdim (weight ``norm`` [vdim], shared by the heads) and multiplied by ``sigmoid(W_g2 (W_g1 h))``,
     then projected.  State per sequence slot: S (fp32) and the last taps - 1 convolution inputs.
-    Everything behind the convolution is fp32 (ops.hybrid.decay_scan)."""
+    Everything behind the convolution is fp32 (ops.hybrid.decay_scan).  What a design fixes comes as
+    ``opts`` (absent: the first value):
+
+    * ``decay`` "channel" / "head": one decay per head, ``exp(-exp(A_log[h]) softplus(W_a h + dt_bias[h]))``;
+    * ``gate`` "low_rank" (the above) / "silu": the output gate is ``silu(W_g h)``."""
 
     kind = "gated_delta"
     stateful = True
@@ -533,18 +550,27 @@ class GatedDeltaMixer:
         H, Gk, dk, dv = self.H, self.Gk, self.dk, self.dv
         s = 1.0 / math.sqrt(d)
         self.C = 2 * Gk * dk + H * dv  # convolved channels [q | k | v]
-        wa1, self.wa2 = _low_rank(p, prefix, "a1", "a2", H * dk, d, int(m.get("a_rank", 16)))
-        wg1, self.wg2 = _low_rank(p, prefix, "g1", "g2", H * dv, d, int(m.get("g_rank", 16)))
-        self.ra, self.rg = wa1.shape[0], wg1.shape[0]
-        # rows [q | k | v | beta | a1 | g1]: everything that reads the mixer's input, one launch
+        o = opts or {}
+        self.per_head, self.low_rank_gate = o.get("decay", "channel") == "head", o.get("gate", "low_rank") == "low_rank"
+        self.wa2 = self.wg2 = None
+        if self.per_head:
+            wa = p.get(prefix + "a", (H, d), s)
+        else:
+            wa, self.wa2 = _low_rank(p, prefix, "a1", "a2", H * dk, d, int(m.get("a_rank", 16)))
+        if self.low_rank_gate:
+            wg, self.wg2 = _low_rank(p, prefix, "g1", "g2", H * dv, d, int(m.get("g_rank", 16)))
+        else:
+            wg = p.get(prefix + "g", (H * dv, d), s)
+        self.ra, self.rg = wa.shape[0], wg.shape[0]
+        # rows [q | k | v | beta | a | g] (a, g: low-rank or whole): everything that reads the mixer's input, one launch
         self.w_in = torch.cat([p.get(prefix + "q", (Gk * dk, d), s), p.get(prefix + "k", (Gk * dk, d), s),
-                               p.get(prefix + "v", (H * dv, d), s), p.get(prefix + "b", (H, d), s), wa1, wg1]).contiguous()
+                               p.get(prefix + "v", (H * dv, d), s), p.get(prefix + "b", (H, d), s), wa, wg]).contiguous()
         self.b_col, self.a_col, self.g_col = self.C, self.C + H, self.C + H + self.ra
         self.conv_w = torch.cat([p.get(prefix + "q.conv", (Gk * dk, self.taps), 0.4, small=True),
                                  p.get(prefix + "k.conv", (Gk * dk, self.taps), 0.4, small=True),
                                  p.get(prefix + "v.conv", (H * dv, self.taps), 0.4, small=True)]).contiguous()
         self.a_log = p.get(prefix + "A_log", (H,), 0.5, -0.5, small=True)
-        self.dt_bias = p.get(prefix + "dt_bias", (H * dk,), 0.5, -1.0, small=True)
+        self.dt_bias = p.get(prefix + "dt_bias", (H if self.per_head else H * dk,), 0.5, -1.0, small=True)
         self.norm_w = p.get(prefix + "norm", (dv,), 0.1, 1.0, small=True)
         self.norm_all = self.norm_w.repeat(H).contiguous()  # the norm kernel reads one weight per column
         self.wo = p.get(prefix + "o", (d, H * dv), 1.0 / math.sqrt(H * dv))
@@ -562,19 +588,24 @@ class GatedDeltaMixer:
             proj = F.linear(h, self.w_in)
         seg = (meta.seg_cu, meta.seg_ctx, meta.seg_slot)
         qkv = hops.conv_silu(proj, 0, self.C, self.conv_w, None, cache["conv"], *seg)
-        z = F.linear(proj[:, self.a_col:self.a_col + self.ra], self.wa2)
-        gate = F.linear(proj[:, self.g_col:self.g_col + self.rg], self.wg2)
+        z, z_col = (proj, self.a_col) if self.per_head else (F.linear(proj[:, self.a_col:self.a_col + self.ra], self.wa2), 0)
         o = hops.decay_scan(qkv, 0, Gk * dk, 2 * Gk * dk, z, self.dt_bias, cache["state"], *seg, H, Gk, dk, dv,
-                            dk ** -0.5, a_log=self.a_log, beta=proj, beta_col=self.b_col, unit=True)
-        g = hops.gated_group_norm(o, gate, 0, self.norm_all, self.eps, H, h.dtype, after=True)
+                            dk ** -0.5, a_log=self.a_log, beta=proj, beta_col=self.b_col, unit=True, z_col=z_col)
+        if self.low_rank_gate:
+            gate = F.linear(proj[:, self.g_col:self.g_col + self.rg], self.wg2)
+            g = hops.gated_group_norm(o, gate, 0, self.norm_all, self.eps, H, h.dtype, after=True)
+        else:
+            g = hops.gated_group_norm(o, proj, self.g_col, self.norm_all, self.eps, H, h.dtype, after=True, gate="silu")
         return F.linear(g, self.wo)
 
     def export(self, p: str) -> dict:
         n = self.Gk * self.dk
         w, cw = self.w_in, self.conv_w
-        return {p + "q": w[:n], p + "k": w[n:2 * n], p + "v": w[2 * n:self.C], p + "b": w[self.b_col:self.a_col],
-                p + "a1": w[self.a_col:self.g_col], p + "g1": w[self.g_col:self.g_col + self.rg], p + "a2": self.wa2,
-                p + "g2": self.wg2, p + "q.conv": cw[:n], p + "k.conv": cw[n:2 * n], p + "v.conv": cw[2 * n:],
+        a, g = w[self.a_col:self.g_col], w[self.g_col:self.g_col + self.rg]
+        return {**({p + "a": a} if self.per_head else {p + "a1": a, p + "a2": self.wa2}),
+                **({p + "g1": g, p + "g2": self.wg2} if self.low_rank_gate else {p + "g": g}),
+                p + "q": w[:n], p + "k": w[n:2 * n], p + "v": w[2 * n:self.C], p + "b": w[self.b_col:self.a_col],
+                p + "q.conv": cw[:n], p + "k.conv": cw[n:2 * n], p + "v.conv": cw[2 * n:],
                 p + "A_log": self.a_log, p + "dt_bias": self.dt_bias, p + "norm": self.norm_w, p + "o": self.wo}
 
 
@@ -630,13 +661,124 @@ class GatedLinearMixer:
                 p + "norm": self.norm_w, p + "o": self.wo}
 
 
+class Mamba1Mixer:
+    """The selective scan: in-projection [x | z], a short causal convolution (with bias) + SiLU over x,
+    ``[dt | B | C] = W_x x``, step sizes ``softplus(W_dt dt + dt.b)`` per channel, decays ``exp(dt A)`` with
+    ``A = -exp(A_log)`` per channel and state, the fp32 recurrence with its skip term ``D x`` and output gate
+    ``silu(z)`` (ops.hybrid.selective_scan), and the out-projection.  State per sequence slot: [inner,
+    state] fp32 and the last taps - 1 convolution inputs."""
+
+    kind = "mamba1"
+    stateful = True
+
+    def __init__(self, spec: LayerSpec, d: int, eps: float, p: _Params, prefix: str, traits: Optional[dict] = None,
+                 tail: Optional[torch.Tensor] = None, opts: Optional[dict] = None):
+        m = spec.m
+        self.inner, self.N, self.taps, self.rank = int(m["inner"]), int(m["state"]), int(m["conv"]), int(m["dt_rank"])
+        if min(self.inner, self.N, self.taps, self.rank) < 1:
+            raise ValueError(f"{prefix}: inner / state / conv / dt_rank must be positive")
+        C, N, r = self.inner, self.N, self.rank
+        self.w_in = p.get(prefix + "in", (2 * C, d), 1.0 / math.sqrt(d))
+        self.conv_w = p.get(prefix + "conv", (C, self.taps), 0.4, small=True)
+        self.conv_b = p.get(prefix + "conv.b", (C,), 0.1, small=True)
+        self.w_x = p.get(prefix + "x", (r + 2 * N, C), 1.0 / math.sqrt(C))
+        self.w_dt = p.get(prefix + "dt", (C, r), 1.0 / math.sqrt(r))
+        self.dt_bias = p.get(prefix + "dt.b", (C,), 0.5, -2.0, small=True)
+        self.a_log = p.get(prefix + "A_log", (C, N), 0.5, 0.5, small=True)
+        self.d_skip = p.get(prefix + "D", (C,), 0.3, 1.0, small=True)
+        self.wo = p.get(prefix + "o", (d, C), 1.0 / math.sqrt(C))
+
+    def new_cache(self, num_blocks: int, num_slots: int, dtype, device) -> dict:
+        return {"conv": torch.zeros(num_slots, max(1, self.taps - 1), self.inner, dtype=dtype, device=device),
+                "state": torch.zeros(num_slots, self.inner, self.N, dtype=torch.float32, device=device)}
+
+    def cache_bytes(self, esize: int) -> tuple:
+        return 0, (self.taps - 1) * self.inner * esize + self.inner * self.N * 4
+
+    def forward(self, h: torch.Tensor, meta: AttnMeta, cache: dict) -> torch.Tensor:
+        C, N, r = self.inner, self.N, self.rank
+        seg = (meta.seg_cu, meta.seg_ctx, meta.seg_slot)
+        proj = F.linear(h, self.w_in)
+        x = hops.conv_silu(proj, 0, C, self.conv_w, self.conv_b, cache["conv"], *seg)
+        q = F.linear(x, self.w_x)
+        dt = F.linear(q[:, :r], self.w_dt)
+        y = hops.selective_scan(x, q, r, r + N, dt, self.dt_bias, self.a_log, self.d_skip, proj, C, cache["state"], *seg)
+        return F.linear(y, self.wo)
+
+    def export(self, p: str) -> dict:
+        return {p + "in": self.w_in, p + "conv": self.conv_w, p + "conv.b": self.conv_b, p + "x": self.w_x, p + "dt": self.w_dt,
+                p + "dt.b": self.dt_bias, p + "A_log": self.a_log, p + "D": self.d_skip, p + "o": self.wo}
+
+
+class WkvMixer:
+    """RWKV-style time mixing.  With h' the previous token's h (zeros for a sequence's first), each of r,
+    k, v, g, w reads its own mix ``h + (h' - h) * mu.<name>``; ``r, k, v`` ([heads, dim]) and the gate
+    ``silu(W_g mix_g)`` are projections, the decays per head and key channel ``exp(-exp(W_w2 tanh(W_w1 mix_w) +
+    w0))``.  Per head ``o_t = (S + diag(u) k_t v_t^T)^T r_t``, then ``S <- diag(w_t) S + k_t v_t^T``
+    (ops.hybrid.decay_scan with a bonus).  Each head's o is divided by its root mean square; the heads
+    together are multiplied by ``norm`` [heads * dim] and the gate, then projected.  State per sequence
+    slot: S (fp32) and the last h (fp32).  The mixes are formed in fp32 from the fp32 norm output
+    (``h_fp32``) and rounded once; r, k, v, g run as one batched GEMM."""
+
+    kind = "wkv"
+    stateful = True
+    h_fp32 = True
+
+    def __init__(self, spec: LayerSpec, d: int, eps: float, p: _Params, prefix: str, traits: Optional[dict] = None,
+                 tail: Optional[torch.Tensor] = None, opts: Optional[dict] = None):
+        m = spec.m
+        self.H, self.dk = int(m["heads"]), int(m["dim"])
+        self.eps = eps
+        H, dk = self.H, self.dk
+        n, s = H * dk, 1.0 / math.sqrt(d)
+        self.n, self.d = n, d
+        self.mu = torch.stack([p.get(prefix + "mu." + k, (d,), 0.25, 0.5, small=True) for k in "rkvgw"]).contiguous()
+        # [4, d, n]: the right operand of the batched product, contiguous as it is read
+        self.w_rkvg = torch.stack([p.get(prefix + k, (n, d), s).t() for k in "rkvg"]).contiguous()
+        self.w1, self.w2 = _low_rank(p, prefix, "w1", "w2", n, d, int(m.get("w_rank", 32)))
+        self.w0 = p.get(prefix + "w0", (n,), 1.0, -1.5, small=True)
+        self.u = p.get(prefix + "u", (H, dk), 0.5, 0.3, small=True)
+        self.norm_w = p.get(prefix + "norm", (n,), 0.1, 1.0, small=True)
+        self.wo = p.get(prefix + "o", (d, n), 1.0 / math.sqrt(n))
+
+    def new_cache(self, num_blocks: int, num_slots: int, dtype, device) -> dict:
+        return {"prev": torch.zeros(num_slots, self.d, dtype=torch.float32, device=device),
+                "state": torch.zeros(num_slots, self.H, self.dk, self.dk, dtype=torch.float32, device=device)}
+
+    def cache_bytes(self, esize: int) -> tuple:
+        return 0, 4 * (self.d + self.H * self.dk * self.dk)
+
+    def forward(self, h: torch.Tensor, meta: AttnMeta, cache: dict) -> torch.Tensor:
+        T, n, H, dk = h.shape[0], self.n, self.H, self.dk
+        seg = (meta.seg_cu, meta.seg_ctx, meta.seg_slot)
+        dtype = self.wo.dtype
+        mix = hops.token_mix(h, self.mu, cache["prev"], *seg, dtype)
+        rkvg = torch.empty(T, 4 * n, dtype=dtype, device=h.device)
+        torch.bmm(mix[:, :4].transpose(0, 1), self.w_rkvg, out=rkvg.view(T, 4, n).transpose(0, 1))
+        z = F.linear(hops.activation(F.linear(mix[:, 4], self.w1), "tanh"), self.w2)
+        o = hops.decay_scan(rkvg, 0, n, 2 * n, z, self.w0, cache["state"], *seg, H, H, dk, dk, 1.0, decay="exp_exp", bonus=self.u)
+        g = hops.gated_group_norm(o, rkvg, 3 * n, self.norm_w, self.eps, H, dtype, after=True, gate="silu")
+        return F.linear(g, self.wo)
+
+    def export(self, p: str) -> dict:
+        out = {p + "mu." + k: self.mu[i] for i, k in enumerate("rkvgw")}
+        out.update({p + k: self.w_rkvg[i].t() for i, k in enumerate("rkvg")})
+        out.update({p + "w1": self.w1, p + "w2": self.w2, p + "w0": self.w0, p + "u": self.u, p + "norm": self.norm_w,
+                    p + "o": self.wo})
+        return out
+
+
 class SideBySide:
     """Two mixers on the same normed input, added with fixed weights: ``left_scale * left(h) +
     right_scale * right(h)``.  Which two, and what the design fixes for each, is the design's
     ``composite`` trait for the layer's ``type``; their constants sit under ``mixer.left`` /
     ``mixer.right`` and their tensors under ``mix.left.`` / ``mix.right.``.  Both input projections run
     as ONE GEMM (each mixer then reads its own columns); forward returns the two results with their
-    weights, and the sum happens in fp32 in the launch of the next norm (ops.hybrid.sum_norm)."""
+    weights, and the sum happens in fp32 in the launch of the next norm (ops.hybrid.sum_norm).
+
+    Designs with ``pair_norm``: the results are RMS-normed over the width each (weights ``left.out`` /
+    ``right.out``, in ``out_w``) and their sum is multiplied by that number; forward returns the two
+    results, and norms and sum happen in the launch of the norm behind the sublayer (ops.hybrid.join_norm)."""
 
     kind = "side_by_side"
 
@@ -651,13 +793,22 @@ class SideBySide:
             kind, o = comp[side]
             self.subs.append(MIXERS[kind](spec.sub(side, kind), d, eps, p, f"{prefix}{side}.", traits=traits, opts=o))
         self.scales = (float(m.get("left_scale", 1.0)), float(m.get("right_scale", 1.0)))
+        self.mix = (traits or {}).get("pair_norm")
+        self.out_w = None if self.mix is None else tuple(p.get(f"{prefix}{side}.out", (d,), 0.1, 1.0, small=True)
+                                                         for side in ("left", "right"))
         self.stateful = any(getattr(x, "stateful", False) for x in self.subs)
-        self.n_left = nl = self.subs[0].w_in.shape[0]
-        n = nl + self.subs[1].w_in.shape[0]
-        # rows padded with zeros to a multiple of 8: the kernels' 16-byte accesses need aligned row strides
-        pad = [torch.zeros(-n % 8, d, dtype=self.subs[0].w_in.dtype, device=self.subs[0].w_in.device)] if n % 8 else []
-        self.w_in = torch.cat([x.w_in for x in self.subs] + pad).contiguous()
-        self.subs[0].w_in, self.subs[1].w_in = self.w_in[:nl], self.w_in[nl:n]
+        # each mixer's rows padded with zeros to a multiple of 8: the kernels' 16-byte accesses need aligned
+        # row strides and first columns
+        parts, self.cols = [], []
+        for x in self.subs:
+            w, o = x.w_in, sum(t.shape[0] for t in parts)
+            self.cols.append((o, o + w.shape[0]))
+            parts.append(w)
+            if w.shape[0] % 8:
+                parts.append(torch.zeros(-w.shape[0] % 8, d, dtype=w.dtype, device=w.device))
+        self.w_in = torch.cat(parts).contiguous()
+        for x, (a, b) in zip(self.subs, self.cols):
+            x.w_in = self.w_in[a:b]
 
     @property
     def fast(self) -> int:
@@ -679,17 +830,23 @@ class SideBySide:
 
     def forward(self, h: torch.Tensor, meta: AttnMeta, cache: dict) -> tuple:
         proj = F.linear(h, self.w_in)
-        yl = self.subs[0].forward(h, meta, cache["left"], proj=proj[:, :self.n_left])
-        yr = self.subs[1].forward(h, meta, cache["right"], proj=proj[:, self.n_left:self.n_left + self.subs[1].w_in.shape[0]])
+        yl, yr = (x.forward(h, meta, cache[side], proj=proj[:, a:b])
+                  for x, side, (a, b) in zip(self.subs, ("left", "right"), self.cols))
+        if self.out_w is not None:
+            return yl, yr
         return (yl, self.scales[0]), (yr, self.scales[1])
 
     def export(self, p: str) -> dict:
-        return {**self.subs[0].export(p + "left."), **self.subs[1].export(p + "right.")}
+        out = {**self.subs[0].export(p + "left."), **self.subs[1].export(p + "right.")}
+        if self.out_w is not None:
+            out.update({p + "left.out": self.out_w[0], p + "right.out": self.out_w[1]})
+        return out
 
 
 MIXERS = {WindowAttention.kind: WindowAttention, Mamba2Mixer.kind: Mamba2Mixer, LatentAttention.kind: LatentAttention,
           RotaryAttention.kind: RotaryAttention, LightningMixer.kind: LightningMixer,
-          GatedDeltaMixer.kind: GatedDeltaMixer, GatedLinearMixer.kind: GatedLinearMixer, SideBySide.kind: SideBySide}
+          GatedDeltaMixer.kind: GatedDeltaMixer, GatedLinearMixer.kind: GatedLinearMixer, Mamba1Mixer.kind: Mamba1Mixer,
+          WkvMixer.kind: WkvMixer, SideBySide.kind: SideBySide}
 
 
 class RoutedFFN:
@@ -745,6 +902,18 @@ class DenseFFN:
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         return F.linear(hops.activation(F.linear(h, self.w_up), "xielu", self.a_pos, self.a_neg), self.w_down)
+
+
+class UngatedDenseFFN:
+    """``down(act(up h))`` with an activation that has no constants (ops.hybrid.activation)."""
+
+    def __init__(self, spec: DenseSpec, d: int, p: _Params, prefix: str, act: str):
+        self.ff, self.act = spec.ff, act
+        self.w_up = p.get(prefix + "up", (self.ff, d), 1.0 / math.sqrt(d))
+        self.w_down = p.get(prefix + "down", (d, self.ff), 1.0 / math.sqrt(self.ff))
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        return F.linear(hops.activation(F.linear(h, self.w_up), self.act), self.w_down)
 
 
 class GatedDenseFFN:
@@ -842,6 +1011,8 @@ def _ffn_for(family: str, spec, d: int, p: _Params, prefix: str, tail: Optional[
     if family == "relu_glu_grouped":
         return GatedDenseFFN(spec, d, p, prefix, tail, act="relu") if isinstance(spec, DenseSpec) else \
             GroupRoutedFFN(spec, d, p, prefix)
+    if family == "relu_sq" and isinstance(spec, DenseSpec):
+        return UngatedDenseFFN(spec, d, p, prefix, "relu_sq")
     if family == "plain_softmax":
         return DenseFFN(spec, d, p, prefix) if isinstance(spec, DenseSpec) else PlainRoutedFFN(spec, d, p, prefix)
     raise ValueError(f"{prefix}: no {type(spec).__name__} feed-forward in the {family!r} family")
@@ -884,6 +1055,13 @@ class HybridLM:
         if self.summed and (self.shifted or self.depth_avg or self.gated or not self.sequential):
             raise ValueError(f"{cfg.name}: layer norm, side-by-side mixers and per-layer token input are built for "
                              "plain sequential blocks")
+        self.post_norm = bool(tr.get("post_norm"))
+        if self.post_norm and (not self.center or not tr.get("norm_bias") or not self.sequential or cfg.loop or self.side_dim
+                               or self.shifted or self.depth_avg or self.gated):
+            raise ValueError(f"{cfg.name}: norms behind the sublayers are built for plain sequential blocks on layer "
+                             "norms with a bias, without looped layers")
+        if not self.post_norm and (tr.get("norm_bias") or tr.get("pair_norm") is not None):
+            raise ValueError(f"{cfg.name}: norm biases and normed mixer pairs are built for blocks with norms behind the sublayers")
         nm = 1.0 if not self.one_plus else 0.0  # plain norm weights sit around one
         self.embed = p.get("embed", (V, d), 0.5)
         self.pos = p.get("pos", (cfg.max_position, d), 0.1) if tr["learned_pos"] else None
@@ -902,10 +1080,22 @@ class HybridLM:
             w = p.get(name, nshape, 0.1, nm, small=True)
             return w.reshape(1).expand(d).contiguous() if self.scalar_norm else w
 
+        self.post1, self.post2, self.bias1, self.bias2 = [], [], [], []  # (w, b) behind a sublayer; biases of norm1 / norm2
+
+        def norm_b(name):
+            return p.get(name + ".b", (d,), 0.1, small=True)
+
         def rgate(name):
             return p.get(name, (d, d), 1.0 / math.sqrt(d)), p.get(name + ".b", (d,), 0.5, small=True)
 
+        per_layer = (self.norms, self.norms2, self.mixers, self.ffns, self.shifts, self.dwa, self.rg1, self.rg2, self.post1,
+                     self.post2, self.bias1, self.bias2, *((self.side_gate, self.side_proj, self.side_norm) if sd else ()))
+        owners = [cfg.owner(i) for i in range(len(cfg.layers))]
         for i, spec in enumerate(cfg.layers):
+            if owners[i] != i:
+                for lst in per_layer:
+                    lst.append(None)
+                continue
             kind = names.get(spec.kind, spec.kind)
             if kind not in MIXERS:
                 raise ValueError(f"layer {i}: unknown mixer {spec.kind!r} (known: {sorted(MIXERS)})")
@@ -919,6 +1109,11 @@ class HybridLM:
             self.rg1.append(self._gate_for(self.mixers[-1], g1))
             self.rg2.append(self._gate_for(self.ffns[-1], g2))
             self.norms2.append(norm_w(f"l{i}.norm2") if self.sequential and spec.mlp is not None else None)
+            post, two = self.post_norm, spec.mlp is not None
+            self.bias1.append(norm_b(f"l{i}.norm1") if post else None)
+            self.post1.append((norm_w(f"l{i}.norm1b"), norm_b(f"l{i}.norm1b")) if post else None)
+            self.bias2.append(norm_b(f"l{i}.norm2") if post and two else None)
+            self.post2.append((norm_w(f"l{i}.norm2b"), norm_b(f"l{i}.norm2b")) if post and two else None)
             if sd:
                 self.side_gate.append(p.get(f"l{i}.side.gate", (sd, d), 1.0 / math.sqrt(d)))
                 self.side_proj.append(p.get(f"l{i}.side.proj", (d, sd), 1.0 / math.sqrt(sd)))
@@ -927,7 +1122,12 @@ class HybridLM:
             # depth-average coefficients: random init leans on the newest result so the stream stays sane
             self.dwa.append(p.get(f"l{i}.dwa", (i + 2,), 0.3 / (i + 2), 1.0 / (i + 2), small=True)
                             if self.depth_avg else None)
+        for i, j in enumerate(owners):  # a layer that uses another's tensors shares its objects
+            if j != i:
+                for lst in per_layer:
+                    lst[i] = lst[j]
         self.final_norm = norm_w("final.norm")
+        self.final_bias = norm_b("final.norm") if self.post_norm else None
         self.head = p.get("head", (V, d), 1.0 / math.sqrt(d))
         self.runs = cfg.runs()
         # the run whose pages a run reads: its own, or the latest earlier run of the layer it names
@@ -996,6 +1196,9 @@ class HybridLM:
     def _tensors(self) -> list:
         ts = [self.embed, self.final_norm, self.head] + self.norms + self.side_gate + self.side_proj + self.side_norm
         ts += [t for t in [self.pos, self.loop_step, self.side_embed] + self.norms2 + self.shifts + self.dwa if t is not None]
+        ts += [t for t in self.bias1 + self.bias2 + [self.final_bias] if t is not None]
+        ts += [t for pair in self.post1 + self.post2 if pair is not None for t in pair]
+        ts += [t for m in self.mixers for t in (getattr(m, "out_w", None) or ())]
         ts += [t for g in self.rg1 + self.rg2 if g is not None for t in g.values() if t is not None]
         subs = [x for m in self.mixers for x in getattr(m, "subs", ())]
         for o in self.mixers + subs + [f for f in self.ffns if f is not None]:
@@ -1054,6 +1257,8 @@ class HybridLM:
                                scale=c.embed_scale)
         if self.gated:
             return self._forward_gated(x, meta, caches)
+        if self.post_norm:
+            return self._forward_post_norm(x, meta, caches)
         if self.summed:
             return self._forward_summed(ids, x, meta, caches)
         pending: tuple = ()
@@ -1124,6 +1329,33 @@ class HybridLM:
         hf = hops.sum_norm(x, pend, normed, self.final_norm, eps, ctr, op, self.dtype)
         return self._logits(hf)
 
+    def _forward_post_norm(self, x: torch.Tensor, meta: AttnMeta, caches: list) -> torch.Tensor:
+        """Sequential blocks with a norm on both sides of every sublayer: a sublayer's result (or a pair of
+        results) stays pending until the launch of the next norm, which norms it, adds it to the stream
+        and norms the stream (ops.hybrid.join_norm)."""
+        eps = self.cfg.norm_eps
+        pend: tuple = ((), None, {})  # (results, the norm behind them, how a pair is combined)
+
+        def join(stream, pre, dtype):
+            return hops.join_norm(stream, pend[0], pend[1], pre, eps, dtype, **pend[2])
+
+        for r, (li, _, _) in enumerate(self.runs):
+            mx, ff = self.mixers[li], self.ffns[li]
+            h = join(x, (self.norms[li], self.bias1[li]), torch.float32 if getattr(mx, "h_fp32", False) else self.dtype)
+            y = mx.forward(h, meta, caches[self.kv_run[r]])
+            pend = (y, self.post1[li], dict(branch_w=mx.out_w, mix=mx.mix)) if isinstance(y, tuple) else ((y,), self.post1[li], {})
+            if ff is not None:
+                pend = ((ff.forward(join(x, (self.norms2[li], self.bias2[li]), self.dtype)),), self.post2[li], {})
+            if self.layer_probe is not None:
+                full = x.clone()
+                join(full, None, self.dtype)
+                self.layer_probe.append(full)
+        if meta.logits_idx is not None:
+            idx = meta.logits_idx
+            x = x.index_select(0, idx)
+            pend = (tuple(a.index_select(0, idx) for a in pend[0]), *pend[1:])
+        return self._logits(join(x, (self.final_norm, self.final_bias), self.dtype))
+
     def _logits(self, hf: torch.Tensor) -> torch.Tensor:
         c = self.cfg
         z = F.linear(hf, self.head).float()
@@ -1185,9 +1417,19 @@ def state_dict(model: HybridLM) -> dict:
         out["loop.step"] = model.loop_step
     if model.side_embed is not None:
         out["side.embed"] = model.side_embed
+    if model.final_bias is not None:
+        out["final.norm.b"] = model.final_bias
     for i, (n, m, f) in enumerate(zip(model.norms, model.mixers, model.ffns)):
+        if model.cfg.owner(i) != i:
+            continue
         p = f"l{i}."
         out[p + "norm1"] = one(n)
+        for key, t in (("norm1.b", model.bias1[i]), ("norm2.b", model.bias2[i])):
+            if t is not None:
+                out[p + key] = t
+        for key, pair in (("norm1b", model.post1[i]), ("norm2b", model.post2[i])):
+            if pair is not None:
+                out[p + key], out[p + key + ".b"] = pair
         if model.side_dim:
             out.update({p + "side.gate": model.side_gate[i], p + "side.proj": model.side_proj[i],
                         p + "side.norm": model.side_norm[i]})
@@ -1224,6 +1466,8 @@ def state_dict(model: HybridLM) -> dict:
                         p + "mix.norm": m.norm_w, p + "mix.o": m.wo})
         if isinstance(f, GatedDenseFFN):
             out.update({p + "mlp.gate": f.w_in[:f.ff], p + "mlp.up": f.w_in[f.ff:2 * f.ff], p + "mlp.down": f.w_down})
+        elif isinstance(f, UngatedDenseFFN):
+            out.update({p + "mlp.up": f.w_up, p + "mlp.down": f.w_down})
         elif isinstance(f, DenseFFN):
             out.update({p + "mlp.up": f.w_up, p + "mlp.down": f.w_down, p + "mlp.act": f.act})
         elif isinstance(f, GroupRoutedFFN):

@@ -19,9 +19,10 @@ int k8sllm_hy_rotary_norm_cache(void* qkv, long stride, long T, int Hq, int G, i
                                 float eps, const float* q_scale, void* k_cache, void* v_cache, const int* slots, int bs,
                                 int v_from_k, int f32, hipStream_t s);
 int k8sllm_hy_decay_scan(float* o, const void* qkv, long stride, int q_col, int k_col, int v_col, const void* z,
-                         long z_stride, const float* z_bias, const float* a_log, float inv_tau, const void* beta,
-                         long b_stride, float* state, const int* cu, const int* ctx, const int* slot, int S, int H, int Gk,
-                         int dk, int dv, float q_scale, int unit, int f32, float* ws, long T, hipStream_t s);
+                         long z_stride, const float* z_bias, const float* a_log, float inv_tau, int dkind, int per_head,
+                         const void* beta, long b_stride, const float* bonus, float* state, const int* cu,
+                         const int* ctx, const int* slot, int S, int H, int Gk, int dk, int dv, float q_scale, int unit,
+                         int f32, float* ws, long T, hipStream_t s);
 long k8sllm_hy_decay_scan_ws(long T, int H, int Gk, int dk);
 int k8sllm_hy_router_grouped(int* ids, float* wts, const void* h, long T, int d, const float* wr, int E, int K,
                              int groups, int keep, float scale, int f32, hipStream_t s);
@@ -47,11 +48,11 @@ int k8sllm_hy_qk_norm_cache(void* qkv, long stride, const float* qw, const float
                             int nk, int nv, void* k_cache, void* v_cache, const int* slots, int bs, int f32, hipStream_t s);
 int k8sllm_hy_window_prefill(void* out, const void* qkv, long q_stride, const void* k_cache, const void* v_cache,
                              const int* cu, const int* ctx, const int* block_tables, int bt_stride, int S, long T,
-                             int Hq, int G, int dk, int dv, int bs, float scale, int window, int sink,
+                             int Hq, int G, int dk, int dv, int bs, float scale, int window, int chunked, float cap, int sink,
                              const float* sinks, int f32, int mfma, hipStream_t s);
 int k8sllm_hy_window_decode(void* out, const void* qkv, long q_stride, const void* k_cache, const void* v_cache,
                             const int* block_tables, int bt_stride, const int* seq_lens, int B, int Hq, int G, int dk,
-                            int dv, int bs, float scale, int window, int sink, const float* sinks, int f32, int vec,
+                            int dv, int bs, float scale, int window, int chunked, float cap, int sink, const float* sinks, int f32, int vec,
                             hipStream_t s);
 int k8sllm_hy_conv_silu(void* out, const void* proj, long stride, int col0, int C, const float* cw, const float* cb,
                         int taps, void* state, const int* cu, const int* ctx, const int* slot, int S, long T, int f32,
@@ -60,6 +61,15 @@ int k8sllm_hy_ssm_scan(float* y, const void* xbc, const void* proj, long p_strid
                        const float* a_log, const float* d_skip, const float* decay, float* state, const int* cu,
                        const int* ctx, const int* slot, int S, long T, int nh, int P, int N, int G, int f32, int mode,
                        hipStream_t s);
+int k8sllm_hy_selective_scan(void* out, const void* xc, const void* q, long q_stride, int b_col, int c_col,
+                             const void* dt, long dt_stride, const float* dt_bias, const float* a_log, const float* d_skip,
+                             const void* z, long z_stride, float* state, const int* cu, const int* ctx, const int* slot,
+                             int S, long T, int C, int N, int f32, hipStream_t s);
+int k8sllm_hy_join_norm(void* out, float* residual, const void* y0, int t0, const void* y1, int t1, const float* w0,
+                        const float* w1, float mix, const float* pw, const float* pb, const float* nw, const float* nb,
+                        long rows, int d, float eps, int f32, hipStream_t s);
+int k8sllm_hy_token_mix(void* out, const float* h, const float* mu, int n, float* state, const int* cu, const int* ctx,
+                        const int* slot, int S, long rows, int d, int f32, hipStream_t s);
 int k8sllm_hy_linear_attn_chunk(float* y, const void* vkq, const float* decay, float* state, const int* cu,
                                 const int* ctx, const int* slot, int S, int H, int dk, int dv, int nt, hipStream_t s);
 int k8sllm_hy_router(int* ids, float* wts, float* gate, const void* h, long T, int d, const float* wr,
@@ -316,7 +326,7 @@ void qk_norm_cache(Tensor qkv, Tensor qw, Tensor kw, double eps, int64_t Hq, int
 
 void window_attention_prefill(Tensor out, Tensor qkv, Tensor k_cache, Tensor v_cache, Tensor cu, Tensor ctx,
                               Tensor block_tables, int64_t Hq, int64_t G, int64_t dk, int64_t dv, double scale,
-                              int64_t window, bool sink, OptT sinks, int64_t mfma) {
+                              int64_t window, bool sink, OptT sinks, int64_t mfma, bool chunked, double cap) {
   const int f = act(qkv, "qkv");
   same(out, f, "out");
   pages(k_cache, f, G * dk, "k_cache");
@@ -330,18 +340,18 @@ void window_attention_prefill(Tensor out, Tensor qkv, Tensor k_cache, Tensor v_c
   TORCH_CHECK(qkv.dim() == 2 && qkv.stride(1) == 1 && qkv.size(1) >= Hq * dk, "qkv rows");
   TORCH_CHECK(out.is_contiguous() && out.numel() == T * Hq * dv, "out [T, Hq*dv]");
   TORCH_CHECK(cu.numel() == S + 1 && block_tables.size(0) >= S, "cu [S+1], block_tables [S, W]");
-  TORCH_CHECK(window >= 0 && G >= 1 && Hq % G == 0, "heads / window");
+  TORCH_CHECK(window >= 0 && G >= 1 && Hq % G == 0 && cap >= 0, "heads / window / cap");
   check(k8sllm_hy_window_prefill(out.data_ptr(), qkv.data_ptr(), qkv.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
                                  cu.data_ptr<int>(), ctx.data_ptr<int>(), block_tables.data_ptr<int>(),
                                  (int)block_tables.stride(0), (int)S, T, (int)Hq, (int)G, (int)dk, (int)dv,
-                                 (int)k_cache.size(1), (float)scale, (int)window, sink, sink_ptr(sinks, Hq), f,
-                                 (int)mfma, cur()),
+                                 (int)k_cache.size(1), (float)scale, (int)window, chunked, (float)cap, sink,
+                                 sink_ptr(sinks, Hq), f, (int)mfma, cur()),
         "window_attention_prefill");
 }
 
 void window_attention_decode(Tensor out, Tensor qkv, Tensor k_cache, Tensor v_cache, Tensor block_tables,
                              Tensor seq_lens, int64_t Hq, int64_t G, int64_t dk, int64_t dv, double scale,
-                             int64_t window, bool sink, OptT sinks, bool vec) {
+                             int64_t window, bool sink, OptT sinks, bool vec, bool chunked, double cap) {
   const int f = act(qkv, "qkv");
   same(out, f, "out");
   pages(k_cache, f, G * dk, "k_cache");
@@ -354,11 +364,11 @@ void window_attention_decode(Tensor out, Tensor qkv, Tensor k_cache, Tensor v_ca
   TORCH_CHECK(qkv.dim() == 2 && qkv.stride(1) == 1 && qkv.size(1) >= Hq * dk, "qkv rows");
   TORCH_CHECK(out.is_contiguous() && out.numel() == B * Hq * dv, "out [B, Hq*dv]");
   TORCH_CHECK(seq_lens.numel() >= B && block_tables.size(0) >= B, "seq_lens [B], block_tables [B, W]");
-  TORCH_CHECK(window >= 0 && G >= 1 && Hq % G == 0, "heads / window");
+  TORCH_CHECK(window >= 0 && G >= 1 && Hq % G == 0 && cap >= 0, "heads / window / cap");
   check(k8sllm_hy_window_decode(out.data_ptr(), qkv.data_ptr(), qkv.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
                                 block_tables.data_ptr<int>(), (int)block_tables.stride(0), seq_lens.data_ptr<int>(),
                                 (int)B, (int)Hq, (int)G, (int)dk, (int)dv, (int)k_cache.size(1), (float)scale,
-                                (int)window, sink, sink_ptr(sinks, Hq), f, vec, cur()),
+                                (int)window, chunked, (float)cap, sink, sink_ptr(sinks, Hq), f, vec, cur()),
         "window_attention_decode");
 }
 
@@ -607,11 +617,14 @@ void rotary_norm_cache(Tensor qkv, int64_t Hq, int64_t G, int64_t dk, int64_t dv
         "rotary_norm_cache");
 }
 
-// The per-channel-decay recurrence (optionally with the delta rule: beta given); see decay_scan.hip
+// Linear attention with decays per head and key channel, or per head (z_bias [H]); plain, with the delta rule
+// (beta given) or with a bonus for the current token (bonus given); see decay_scan.hip.  dkind: how a decay
+// comes from its logit.  z_col: first column of the decay logits in z
 // ws: fp32 workspace of decay_scan_ws(T, ...) floats - given, the two-launch form for prompts runs
 void decay_scan(Tensor o, Tensor qkv, int64_t q_col, int64_t k_col, int64_t v_col, Tensor z, Tensor z_bias, OptT a_log,
                 double tau, OptT beta, int64_t beta_col, Tensor state, Tensor cu, Tensor ctx, Tensor slot, int64_t H,
-                int64_t Gk, int64_t dk, int64_t dv, double q_scale, bool unit, OptT ws) {
+                int64_t Gk, int64_t dk, int64_t dv, double q_scale, bool unit, OptT ws, int64_t z_col, int64_t dkind,
+                OptT bonus) {
   const int f = act(qkv, "qkv");
   same(z, f, "z");
   f32c(o, "o");
@@ -623,8 +636,19 @@ void decay_scan(Tensor o, Tensor qkv, int64_t q_col, int64_t k_col, int64_t v_co
   TORCH_CHECK(qkv.dim() == 2 && qkv.stride(1) == 1 && q_col >= 0 && k_col >= 0 && v_col >= 0 &&
                   q_col + Gk * dk <= qkv.size(1) && k_col + Gk * dk <= qkv.size(1) && v_col + H * dv <= qkv.size(1),
               "decay_scan: q / k / v columns");
-  TORCH_CHECK(z.dim() == 2 && z.stride(1) == 1 && z.size(0) == T && z.size(1) == H * dk && z_bias.numel() == H * dk,
-              "decay_scan: z [T, H*dk], z_bias [H*dk]");
+  const int64_t nz = z_bias.numel();
+  const bool per_head = nz == H && dk != 1;  // one key channel: both forms are the same numbers
+  TORCH_CHECK(nz == H * dk || nz == H, "decay_scan: z_bias [H*dk], or [H] for one decay per head");
+  TORCH_CHECK(z.dim() == 2 && z.stride(1) == 1 && z.size(0) == T && z_col >= 0 && z_col + nz <= z.size(1),
+              "decay_scan: z columns");
+  TORCH_CHECK(dkind >= 0 && dkind <= 2 && (dkind != 0 || a_log.has_value()), "decay_scan: decay kind");
+  const float* wp_bonus = nullptr;
+  if (bonus.has_value()) {
+    f32c(*bonus, "bonus");
+    TORCH_CHECK(bonus->numel() == H * dk && Gk == H && !beta.has_value(), "decay_scan: bonus [H, dk], a key head per head, no delta rule");
+    wp_bonus = bonus->data_ptr<float>();
+  }
+  TORCH_CHECK(!per_head || beta.has_value(), "decay_scan: one decay per head is built for the delta rule");
   TORCH_CHECK(o.numel() == T * H * dv, "decay_scan: o [T, H*dv]");
   TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == dv && state.size(3) == dk, "state [slots, H, dv, dk]");
   const float* ap = nullptr;
@@ -649,10 +673,92 @@ void decay_scan(Tensor o, Tensor qkv, int64_t q_col, int64_t k_col, int64_t v_co
     wp = ws->data_ptr<float>();
   }
   check(k8sllm_hy_decay_scan(o.data_ptr<float>(), qkv.data_ptr(), qkv.stride(0), (int)q_col, (int)k_col, (int)v_col,
-                             z.data_ptr(), z.stride(0), z_bias.data_ptr<float>(), ap, (float)(1.0 / tau), bp, bstride,
-                             state.data_ptr<float>(), cu.data_ptr<int>(), ctx.data_ptr<int>(), slot.data_ptr<int>(),
+                             (const char*)z.data_ptr() + z_col * z.element_size(), z.stride(0), z_bias.data_ptr<float>(), ap,
+                             (float)(1.0 / tau), (int)dkind, per_head, bp, bstride, wp_bonus, state.data_ptr<float>(), cu.data_ptr<int>(), ctx.data_ptr<int>(), slot.data_ptr<int>(),
                              (int)ctx.numel(), (int)H, (int)Gk, (int)dk, (int)dv, (float)q_scale, unit, f, wp, (long)T, cur()),
         "decay_scan");
+}
+
+// The selective state-space recurrence with a decay per channel and state; see selective_scan.hip.  q holds
+// the state inputs B and read-outs C from columns b_col, c_col on; proj's columns z_col .. are the output gate
+void selective_scan(Tensor out, Tensor xc, Tensor q, int64_t b_col, int64_t c_col, Tensor dt, Tensor dt_bias, Tensor a_log,
+                    Tensor d_skip, Tensor proj, int64_t z_col, Tensor state, Tensor cu, Tensor ctx, Tensor slot) {
+  const int f = act(xc, "xc");
+  same(out, f, "out");
+  same(q, f, "q");
+  same(dt, f, "dt");
+  same(proj, f, "proj");
+  f32c(dt_bias, "dt_bias");
+  f32c(a_log, "A_log");
+  f32c(d_skip, "D");
+  f32c(state, "state");
+  segs(cu, ctx, slot);
+  TORCH_CHECK(xc.dim() == 2 && xc.is_contiguous() && out.is_contiguous() && out.numel() == xc.numel(), "selective_scan: xc, out [T, C]");
+  const int64_t T = xc.size(0), C = xc.size(1);
+  TORCH_CHECK(a_log.dim() == 2 && a_log.size(0) == C && dt_bias.numel() == C && d_skip.numel() == C, "selective_scan: A_log [C, N], dt_bias, D [C]");
+  const int64_t N = a_log.size(1);
+  TORCH_CHECK(N >= 1 && N <= 256, "selective_scan: up to 256 states");
+  TORCH_CHECK(q.dim() == 2 && q.stride(1) == 1 && q.size(0) == T && b_col >= 0 && c_col >= 0 && b_col + N <= q.size(1) &&
+                  c_col + N <= q.size(1),
+              "selective_scan: B / C columns");
+  TORCH_CHECK(dt.dim() == 2 && dt.stride(1) == 1 && dt.size(0) == T && dt.size(1) == C, "selective_scan: dt [T, C]");
+  TORCH_CHECK(proj.dim() == 2 && proj.stride(1) == 1 && proj.size(0) == T && z_col >= 0 && z_col + C <= proj.size(1),
+              "selective_scan: gate columns");
+  TORCH_CHECK(state.dim() == 3 && state.size(1) == C && state.size(2) == N, "state [slots, C, N]");
+  check(k8sllm_hy_selective_scan(out.data_ptr(), xc.data_ptr(), q.data_ptr(), q.stride(0), (int)b_col, (int)c_col, dt.data_ptr(),
+                                 dt.stride(0), dt_bias.data_ptr<float>(), a_log.data_ptr<float>(), d_skip.data_ptr<float>(),
+                                 (const char*)proj.data_ptr() + z_col * proj.element_size(), proj.stride(0),
+                                 state.data_ptr<float>(), cu.data_ptr<int>(), ctx.data_ptr<int>(), slot.data_ptr<int>(),
+                                 (int)ctx.numel(), T, (int)C, (int)N, f, cur()),
+        "selective_scan");
+}
+
+// residual += LN(b) * pw + pb with the branch b = y0, or mix * (y0 / rms(y0) * w0 + y1 / rms(y1) * w1);
+// out = LN(residual) * nw + nb.  y0 absent: only the second norm; nw absent: only the first part
+void join_norm(OptT out, Tensor residual, OptT y0, OptT y1, OptT w0, OptT w1, double mix, OptT pw, OptT pb, OptT nw, OptT nb,
+               double eps) {
+  f32c(residual, "residual");
+  TORCH_CHECK(residual.dim() == 2, "residual [T, d]");
+  const int64_t rows = residual.size(0), d = residual.size(1);
+  TORCH_CHECK(d <= 8192, "join_norm: width up to 8192");
+  const int t0 = any_dt(y0, rows * d, "branch 0"), t1 = any_dt(y1, rows * d, "branch 1");
+  auto vec = [&](const OptT& t, const char* n) -> const float* {
+    if (!t.has_value()) return nullptr;
+    f32c(*t, n);
+    TORCH_CHECK(t->numel() == d, n, " must be [d]");
+    return t->data_ptr<float>();
+  };
+  const float *w0p = vec(w0, "branch weight 0"), *w1p = vec(w1, "branch weight 1"), *pwp = vec(pw, "post norm weight"),
+              *pbp = vec(pb, "post norm bias"), *nwp = vec(nw, "norm weight"), *nbp = vec(nb, "norm bias");
+  TORCH_CHECK((t0 != 0) == (pwp != nullptr && pbp != nullptr), "join_norm: a branch and its norm come together");
+  TORCH_CHECK(t1 == 0 || (t0 != 0 && w0p != nullptr && w1p != nullptr), "join_norm: two branches need their weights");
+  TORCH_CHECK(t1 != 0 || (w0p == nullptr && w1p == nullptr), "join_norm: branch weights without two branches");
+  TORCH_CHECK((nwp != nullptr) == out.has_value() && (nwp != nullptr) == (nbp != nullptr), "join_norm: out comes with the norm");
+  int f = 0;
+  if (out.has_value()) {
+    f = act(*out, "out");
+    TORCH_CHECK(out->is_contiguous() && out->numel() == rows * d, "join_norm: out shape");
+  }
+  check(k8sllm_hy_join_norm(out.has_value() ? out->data_ptr() : nullptr, residual.data_ptr<float>(), t0 ? y0->data_ptr() : nullptr, t0,
+                            t1 ? y1->data_ptr() : nullptr, t1, w0p, w1p, (float)mix, pwp, pbp, nwp, nbp, rows, (int)d,
+                            (float)eps, f, cur()),
+        "join_norm");
+}
+
+// out [T, n, d]: h[t] + (h[t-1] - h[t]) * mu[j], the row before a segment from the sequence's slot (fp32)
+void token_mix(Tensor out, Tensor h, Tensor mu, Tensor state, Tensor cu, Tensor ctx, Tensor slot) {
+  const int f = act(out, "out");
+  f32c(h, "h");
+  f32c(mu, "mu");
+  f32c(state, "token state");
+  segs(cu, ctx, slot);
+  TORCH_CHECK(h.dim() == 2 && mu.dim() == 2 && mu.size(1) == h.size(1), "token_mix: h [T, d], mu [n, d]");
+  const int64_t T = h.size(0), d = h.size(1), n = mu.size(0);
+  TORCH_CHECK(out.is_contiguous() && out.numel() == T * n * d && n >= 1 && n <= 8, "token_mix: out [T, n, d], n up to 8");
+  TORCH_CHECK(state.dim() == 2 && state.size(1) == d, "token state [slots, d]");
+  check(k8sllm_hy_token_mix(out.data_ptr(), h.data_ptr<float>(), mu.data_ptr<float>(), (int)n, state.data_ptr<float>(),
+                            cu.data_ptr<int>(), ctx.data_ptr<int>(), slot.data_ptr<int>(), (int)ctx.numel(), T, (int)d, f, cur()),
+        "token_mix");
 }
 
 void moe_router_grouped(Tensor ids, Tensor wts, Tensor h, Tensor wr, int64_t E, int64_t K, int64_t groups, int64_t keep,
@@ -771,7 +877,7 @@ void depth_mix(Tensor stack, int64_t n, OptT addend, Tensor coef) {
 void activation(Tensor out, Tensor x, int64_t kind, double a, double b) {
   const int f = act(x, "x");
   same(out, f, "out");
-  TORCH_CHECK(x.is_contiguous() && out.is_contiguous() && out.numel() == x.numel() && kind >= 0 && kind <= 3, "activation: shapes / kind");
+  TORCH_CHECK(x.is_contiguous() && out.is_contiguous() && out.numel() == x.numel() && ((kind >= 0 && kind <= 3) || kind == 6 || kind == 7), "activation: shapes / kind");
   check(k8sllm_hy_activation(out.data_ptr(), x.data_ptr(), x.numel(), (int)kind, (float)a, (float)b, f, cur()), "activation");
 }
 
@@ -902,5 +1008,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gated_lookup", &gated_lookup);
   m.def("rotary_norm_cache", &rotary_norm_cache);
   m.def("decay_scan", &decay_scan);
+  m.def("selective_scan", &selective_scan);
+  m.def("join_norm", &join_norm);
+  m.def("token_mix", &token_mix);
   m.def("moe_router_grouped", &moe_router_grouped);
 }

@@ -1,12 +1,15 @@
-// Linear attention with a decay per head and key channel, with or without the delta rule (any sizes up
-// to 256 key channels; state, decays, unit norms and every product fp32).
+// Linear attention with a decay per head and key channel - or one per head -, plain, with the delta rule or
+// with a bonus for the current token (any sizes up to 256 key channels; state, decays, unit norms and every
+// product fp32).
 //   decay_scan   per segment and head, token by token:
 //                    S <- diag(g_t) S
 //                    u  = beta_t (v_t - S^T k_t)      (delta rule)      |  u = v_t   (plain)
 //                    S <- S + k_t u^T;   o_t = S^T q_t
-//                with g_t = exp(-exp(a_log[h]) softplus(z_t + bias))  or  sigmoid(z_t + bias)^(1/tau), q and k
-//                optionally made unit vectors (x / sqrt(sum x^2 + 1e-6)), q times q_scale, beta_t = sigmoid of
-//                a projection column.  The state slot [H][dv][dk] (a value row's key channels contiguous) is
+//                or, with a bonus w [H][dk] (the read-out sees the state BEFORE this token's decay and write):
+//                    o_t = (S + diag(w) k_t v_t^T)^T q_t;   S <- diag(g_t) S + k_t v_t^T
+//                with g_t = exp(-exp(a_log[h]) softplus(z_t + bias)),  sigmoid(z_t + bias)^(1/tau)  or
+//                exp(-exp(z_t + bias)), q and k optionally made unit vectors (x / sqrt(sum x^2 + 1e-6)), q times
+//                q_scale, beta_t = sigmoid of a projection column.  The state slot [H][dv][dk] (a value row's key channels contiguous) is
 //                read at the segment's start (zero for a sequence that starts in this step), written at its end.
 // A segment is one sequence's rows of this step: cu[s] .. cu[s+1], ctx[s] tokens already in its state,
 // slot[s] its state slot (< 0: a padding row, output zero).
@@ -16,7 +19,8 @@
 // taken from the decayed state BEFORE the write: with S' = diag(g) S,
 //     o = S'^T q + u (k . q)
 // so the two sums over key channels that a token needs (S'^T k and S'^T q) are independent and their
-// lane reductions overlap; k . q does not depend on the state and is prepared with the tile.  The inputs
+// lane reductions overlap; k . q does not depend on the state and is prepared with the tile.  (Bonus: the
+// read-out takes S itself and v (k . diag(w) q) is added, the same shape.)  The inputs
 // of 16 tokens at a time are staged in LDS by the whole workgroup (q, k after the unit norm, the decays
 // after their exponentials, v, beta, k . q), so the token loop reads only LDS.
 //
@@ -30,24 +34,58 @@
 
 namespace k8sllm {
 
-template <int CH>
-__device__ __forceinline__ float lanes_sum(float v) {
-  if (CH >= 2) v += K8SLLM_DPP(v, 0xB1);
-  if (CH >= 4) v += K8SLLM_DPP(v, 0x4E);
-  if (CH >= 8) v += K8SLLM_DPP(v, 0x141);
-  if (CH >= 16) v += K8SLLM_DPP(v, 0x140);
-  if (CH >= 32) v = xor16_sum(v);
-  return v;
+// what a token writes and reads (MODE)
+constexpr int kPlain = 0, kDelta = 1, kBonus = 2;
+// how a decay comes from its logit x = z + bias (kind); A = exp(a_log[h])
+constexpr int kSoftplus = 0, kSigmoidRoot = 1, kExpExp = 2;
+__device__ __forceinline__ float decay_f(float x, int kind, float A, float inv_tau) {
+  if (kind == kSoftplus) return expf(-A * softplus_f(x));
+  if (kind == kSigmoidRoot) return expf(-softplus_f(-x) * inv_tau);
+  return expf(-expf(x));
 }
 
-__device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
+// One token of the recurrence for a lane's 8 key channels; returns the column's read-out (all lanes of the
+// column hold it).  gv: this token's decays (one number for all channels where HD).
+template <int CH, int MODE, bool HD>
+__device__ __forceinline__ float scan_token(float (&S)[8], const float* __restrict__ gp, float gh,
+                                            const float* __restrict__ kp, const float* __restrict__ qp, float v,
+                                            float bt, float kq) {
+  float gv[8];
+  if (HD) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) gv[i] = gh;
+  } else {
+    const float4 g0 = *reinterpret_cast<const float4*>(gp), g1 = *reinterpret_cast<const float4*>(gp + 4);
+    gv[0] = g0.x; gv[1] = g0.y; gv[2] = g0.z; gv[3] = g0.w;
+    gv[4] = g1.x; gv[5] = g1.y; gv[6] = g1.z; gv[7] = g1.w;
+  }
+  const float4 k0 = *reinterpret_cast<const float4*>(kp), k1 = *reinterpret_cast<const float4*>(kp + 4);
+  const float4 q0 = *reinterpret_cast<const float4*>(qp), q1 = *reinterpret_cast<const float4*>(qp + 4);
+  const float kv[8] = {k0.x, k0.y, k0.z, k0.w, k1.x, k1.y, k1.z, k1.w};
+  const float qv[8] = {q0.x, q0.y, q0.z, q0.w, q1.x, q1.y, q1.z, q1.w};
+  float pk = 0.f, pq = 0.f;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    if (MODE == kBonus) pq += S[i] * qv[i];
+    S[i] *= gv[i];
+    if (MODE == kDelta) pk += S[i] * kv[i];
+    if (MODE != kBonus) pq += S[i] * qv[i];
+  }
+  if (MODE == kDelta) pk = lanes_sum<CH>(pk);
+  pq = lanes_sum<CH>(pq);
+  const float u = MODE == kDelta ? bt * (v - pk) : v;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) S[i] += kv[i] * u;
+  return pq + u * kq;
+}
 
-template <typename T, int CH, bool DELTA>
+template <typename T, int CH, int MODE, bool HD>
 __global__ __launch_bounds__(256) void decay_scan_kernel(float* __restrict__ o, const T* __restrict__ qkv, long stride,
                                                          int q_col, int k_col, int v_col, const T* __restrict__ z,
                                                          long z_stride, const float* __restrict__ z_bias,
-                                                         const float* __restrict__ a_log, float inv_tau,
+                                                         const float* __restrict__ a_log, float inv_tau, int dkind,
                                                          const T* __restrict__ beta, long b_stride,
+                                                         const float* __restrict__ bonus,
                                                          float* __restrict__ state, const int* __restrict__ cu,
                                                          const int* __restrict__ ctx, const int* __restrict__ slot,
                                                          int H, int Gk, int dk, int dv, float q_scale, int unit) {
@@ -55,9 +93,9 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(float* __restrict__ o, 
   constexpr int ROW = 8 * CH + (CH / 8) * 4 + 4;  // channel n sits at n + 4 (n / 64): 64-float halves 4 banks apart
   __shared__ __attribute__((aligned(16))) float qs[TB][ROW];
   __shared__ __attribute__((aligned(16))) float ks[TB][ROW];
-  __shared__ __attribute__((aligned(16))) float gs[TB][ROW];
+  __shared__ __attribute__((aligned(16))) float gs[HD ? 1 : TB][HD ? 4 : ROW];  // not used with one decay per head
   __shared__ float vs[TB][PB];
-  __shared__ float bts[TB], kqs[TB];
+  __shared__ float bts[TB], kqs[TB], ghs[TB];
   const int s = blockIdx.x, h = blockIdx.y;
   const int sl = slot[s];
   const int t0 = cu[s], t1 = cu[s + 1];
@@ -78,7 +116,7 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(float* __restrict__ o, 
     for (int i = threadIdx.x; i < min(TB, t1 - t0) * ROW; i += 256) {
       (&qs[0][0])[i] = 0.f;
       (&ks[0][0])[i] = 0.f;
-      (&gs[0][0])[i] = 0.f;
+      if (!HD) (&gs[0][0])[i] = 0.f;
     }
   float S[8];
   float* sp = state + (((long)sl * H + h) * dv + p) * dk + n0;
@@ -105,15 +143,19 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(float* __restrict__ o, 
       const int off = n + (n >> 6) * 4;
       qs[tt][off] = ldf(row + q_col);
       ks[tt][off] = ldf(row + k_col);
-      const float zz = ldf(z + (long)(tb + tt) * z_stride + (long)h * dk + n) + z_bias[h * dk + n];
-      gs[tt][off] = a_log != nullptr ? expf(-A * softplus_f(zz)) : expf(-softplus_f(-zz) * inv_tau);
+      if (!HD) {
+        const float zz = ldf(z + (long)(tb + tt) * z_stride + (long)h * dk + n) + z_bias[h * dk + n];
+        gs[tt][off] = decay_f(zz, dkind, A, inv_tau);
+      }
     }
     for (int i = threadIdx.x; i < nt * PB; i += 256) {
       const int tt = i / PB, pp = i % PB;
       const int pg = blockIdx.z * PB + pp;
       vs[tt][pp] = pg < dv ? ldf(qkv + (long)(tb + tt) * stride + v_col + (long)h * dv + pg) : 0.f;
     }
-    if (DELTA && threadIdx.x < nt) bts[threadIdx.x] = sigmoid_f(ldf(beta + (long)(tb + threadIdx.x) * b_stride + h));
+    if (MODE == kDelta && threadIdx.x < nt) bts[threadIdx.x] = sigmoid_f(ldf(beta + (long)(tb + threadIdx.x) * b_stride + h));
+    if (HD && threadIdx.x >= 64 && threadIdx.x - 64 < nt)
+      ghs[threadIdx.x - 64] = decay_f(ldf(z + (long)(tb + threadIdx.x - 64) * z_stride + h) + z_bias[h], dkind, A, inv_tau);
     __syncthreads();
     {  // 16 threads per token: unit norms, the query scale and k . q
       const int tt = threadIdx.x >> 4, j = threadIdx.x & 15;
@@ -135,7 +177,7 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(float* __restrict__ o, 
         const float qv = qs[tt][off] * mq, kv = ks[tt][off] * mk;
         qs[tt][off] = qv;
         ks[tt][off] = kv;
-        kq += qv * kv;
+        kq += MODE == kBonus ? qv * kv * bonus[g * dk + n] : qv * kv;
       }
       kq = lanes_sum<16>(kq);
       if (j == 0) kqs[tt] = kq;
@@ -143,29 +185,9 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(float* __restrict__ o, 
     __syncthreads();
 #pragma unroll 2
     for (int tt = 0; tt < nt; ++tt) {
-      const float4 g0 = *reinterpret_cast<const float4*>(&gs[tt][boff]);
-      const float4 g1 = *reinterpret_cast<const float4*>(&gs[tt][boff + 4]);
-      const float4 k0 = *reinterpret_cast<const float4*>(&ks[tt][boff]);
-      const float4 k1 = *reinterpret_cast<const float4*>(&ks[tt][boff + 4]);
-      const float4 q0 = *reinterpret_cast<const float4*>(&qs[tt][boff]);
-      const float4 q1 = *reinterpret_cast<const float4*>(&qs[tt][boff + 4]);
-      const float gv[8] = {g0.x, g0.y, g0.z, g0.w, g1.x, g1.y, g1.z, g1.w};
-      const float kv[8] = {k0.x, k0.y, k0.z, k0.w, k1.x, k1.y, k1.z, k1.w};
-      const float qv[8] = {q0.x, q0.y, q0.z, q0.w, q1.x, q1.y, q1.z, q1.w};
-      float pk = 0.f, pq = 0.f;
-#pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        S[i] *= gv[i];
-        if (DELTA) pk += S[i] * kv[i];
-        pq += S[i] * qv[i];
-      }
-      if (DELTA) pk = lanes_sum<CH>(pk);
-      pq = lanes_sum<CH>(pq);
-      const float v = vs[tt][pl];
-      const float u = DELTA ? bts[tt] * (v - pk) : v;
-#pragma unroll
-      for (int i = 0; i < 8; ++i) S[i] += kv[i] * u;
-      if (live && chunk == 0) op[(long)tt * inner] = pq + u * kqs[tt];
+      const float r = scan_token<CH, MODE, HD>(S, &gs[HD ? 0 : tt][HD ? 0 : boff], HD ? ghs[tt] : 0.f, &ks[tt][boff],
+                                               &qs[tt][boff], vs[tt][pl], MODE == kDelta ? bts[tt] : 0.f, kqs[tt]);
+      if (live && chunk == 0) op[(long)tt * inner] = r;
     }
     op += (long)TB * inner;
   }
@@ -182,27 +204,30 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(float* __restrict__ o, 
 }
 
 // ---- the two-launch form for prompts
-// workspace rows (fp32): qn, kn [T][Gk][dk], gd [T][H][dk], kq [T][Gk], bt [T][H]
-template <typename T>
+// workspace rows (fp32): qn, kn [T][Gk][dk], gd [T][H][dk] (one decay per head: [T][H]), kq [T][Gk], bt [T][H]
+template <typename T, bool HD>
 __global__ __launch_bounds__(256) void decay_prep_kernel(float* __restrict__ qn, float* __restrict__ kn,
                                                          float* __restrict__ gd, float* __restrict__ kq,
                                                          float* __restrict__ bt, const T* __restrict__ qkv, long stride,
                                                          int q_col, int k_col, const T* __restrict__ z, long z_stride,
                                                          const float* __restrict__ z_bias,
-                                                         const float* __restrict__ a_log, float inv_tau,
-                                                         const T* __restrict__ beta, long b_stride, int H, int Gk,
+                                                         const float* __restrict__ a_log, float inv_tau, int dkind,
+                                                         const T* __restrict__ beta, long b_stride,
+                                                         const float* __restrict__ bonus, int H, int Gk,
                                                          int dk, float q_scale, int unit) {
   // one workgroup per token: the decays of all heads, beta, then a wave per query / key head
   const long t = blockIdx.x;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int nd = H * dk;
+  const int nd = HD ? H : H * dk;
   const T* zr = z + t * z_stride;
   float* gr = gd + t * nd;
-  if (a_log != nullptr) {
+  if (dkind == kSoftplus) {
     for (int e = threadIdx.x; e < nd; e += 256)
-      gr[e] = expf(-expf(a_log[e / dk]) * softplus_f(ldf(zr + e) + z_bias[e]));
+      gr[e] = decay_f(ldf(zr + e) + z_bias[e], kSoftplus, expf(a_log[HD ? e : e / dk]), 0.f);
+  } else if (dkind == kSigmoidRoot) {
+    for (int e = threadIdx.x; e < nd; e += 256) gr[e] = decay_f(ldf(zr + e) + z_bias[e], kSigmoidRoot, 0.f, inv_tau);
   } else {
-    for (int e = threadIdx.x; e < nd; e += 256) gr[e] = expf(-softplus_f(-(ldf(zr + e) + z_bias[e])) * inv_tau);
+    for (int e = threadIdx.x; e < nd; e += 256) gr[e] = decay_f(ldf(zr + e) + z_bias[e], kExpExp, 0.f, 0.f);
   }
   if (beta != nullptr)
     for (int h = threadIdx.x; h < H; h += 256) bt[t * H + h] = sigmoid_f(ldf(beta + t * b_stride + h));
@@ -225,14 +250,14 @@ __global__ __launch_bounds__(256) void decay_prep_kernel(float* __restrict__ qn,
       const float q = ldf(row + q_col + n) * mq, k = ldf(row + k_col + n) * mk;
       qn[(t * Gk + g) * dk + n] = q;
       kn[(t * Gk + g) * dk + n] = k;
-      dot += q * k;
+      dot += bonus != nullptr ? q * k * bonus[g * dk + n] : q * k;
     }
     dot = wave_sum(dot);
     if (lane == 0) kq[t * Gk + g] = dot;
   }
 }
 
-template <typename T, int CH, bool DELTA>
+template <typename T, int CH, int MODE, bool HD>
 __global__ __launch_bounds__(256) void decay_scan_staged_kernel(float* __restrict__ o, const T* __restrict__ qkv,
                                                                 long stride, int v_col, const float* __restrict__ qn,
                                                                 const float* __restrict__ kn,
@@ -249,9 +274,9 @@ __global__ __launch_bounds__(256) void decay_scan_staged_kernel(float* __restric
   constexpr int NV = (TB * PB + 255) / 256;       // values per thread
   __shared__ __attribute__((aligned(16))) float qs[TB][ROW];
   __shared__ __attribute__((aligned(16))) float ks[TB][ROW];
-  __shared__ __attribute__((aligned(16))) float gs[TB][ROW];
+  __shared__ __attribute__((aligned(16))) float gs[HD ? 1 : TB][HD ? 4 : ROW];  // not used with one decay per head
   __shared__ float vs[TB][PB];
-  __shared__ float bts[TB], kqs[TB];
+  __shared__ float bts[TB], kqs[TB], ghs[TB];
   const int s = blockIdx.x, h = blockIdx.y;
   const int sl = slot[s];
   const int t0 = cu[s], t1 = cu[s + 1];
@@ -283,7 +308,7 @@ __global__ __launch_bounds__(256) void decay_scan_staged_kernel(float* __restric
   const int boff = n0 + (n0 >> 6) * 4;
   const bool vec4 = (dk & 3) == 0;
   // the next tile's inputs, in registers while this tile's tokens are processed
-  float4 rq[NB], rk[NB], rg[NB];
+  float4 rq[NB], rk[NB], rg[HD ? 1 : NB];
   float rv[NV], rs = 0.f;
   auto fetch = [&](int tb) {
     const int nt = min(TB, t1 - tb);
@@ -291,20 +316,27 @@ __global__ __launch_bounds__(256) void decay_scan_staged_kernel(float* __restric
     for (int u = 0; u < NB; ++u) {
       const int i = threadIdx.x + 256 * u;
       const int tt = i / Q4, n = (i % Q4) * 4;
-      rq[u] = rk[u] = rg[u] = make_float4(0.f, 0.f, 0.f, 0.f);
+      rq[u] = rk[u] = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (!HD) rg[u] = make_float4(0.f, 0.f, 0.f, 0.f);
       if (tt < nt && n < dk) {
         const float* qp = qn + ((long)(tb + tt) * Gk + g) * dk + n;
         const float* kp = kn + ((long)(tb + tt) * Gk + g) * dk + n;
-        const float* gp = gd + ((long)(tb + tt) * H + h) * dk + n;
+        const float* gp = HD ? nullptr : gd + ((long)(tb + tt) * H + h) * dk + n;
         if (vec4) {
           rq[u] = *reinterpret_cast<const float4*>(qp);
           rk[u] = *reinterpret_cast<const float4*>(kp);
-          rg[u] = *reinterpret_cast<const float4*>(gp);
+          if (!HD) rg[u] = *reinterpret_cast<const float4*>(gp);
         } else {
-          rq[u].x = qp[0]; rk[u].x = kp[0]; rg[u].x = gp[0];
-          if (n + 1 < dk) { rq[u].y = qp[1]; rk[u].y = kp[1]; rg[u].y = gp[1]; }
-          if (n + 2 < dk) { rq[u].z = qp[2]; rk[u].z = kp[2]; rg[u].z = gp[2]; }
-          if (n + 3 < dk) { rq[u].w = qp[3]; rk[u].w = kp[3]; rg[u].w = gp[3]; }
+          rq[u].x = qp[0]; rk[u].x = kp[0];
+          if (n + 1 < dk) { rq[u].y = qp[1]; rk[u].y = kp[1]; }
+          if (n + 2 < dk) { rq[u].z = qp[2]; rk[u].z = kp[2]; }
+          if (n + 3 < dk) { rq[u].w = qp[3]; rk[u].w = kp[3]; }
+          if (!HD) {
+            rg[u].x = gp[0];
+            if (n + 1 < dk) rg[u].y = gp[1];
+            if (n + 2 < dk) rg[u].z = gp[2];
+            if (n + 3 < dk) rg[u].w = gp[3];
+          }
         }
       }
     }
@@ -315,7 +347,8 @@ __global__ __launch_bounds__(256) void decay_scan_staged_kernel(float* __restric
       rv[u] = (tt < nt && pg < dv) ? ldf(qkv + (long)(tb + tt) * stride + v_col + (long)h * dv + pg) : 0.f;
     }
     if (threadIdx.x < nt) rs = kq[(long)(tb + threadIdx.x) * Gk + g];
-    else if (DELTA && threadIdx.x >= TB && threadIdx.x - TB < nt) rs = bt[(long)(tb + threadIdx.x - TB) * H + h];
+    else if (MODE == kDelta && threadIdx.x >= TB && threadIdx.x - TB < nt) rs = bt[(long)(tb + threadIdx.x - TB) * H + h];
+    else if (HD && threadIdx.x >= 2 * TB && threadIdx.x - 2 * TB < nt) rs = gd[(long)(tb + threadIdx.x - 2 * TB) * H + h];
   };
   fetch(t0);
   float* op = o + (long)t0 * inner + (long)h * dv + p;  // this lane's output column, advanced per tile
@@ -330,7 +363,7 @@ __global__ __launch_bounds__(256) void decay_scan_staged_kernel(float* __restric
         const int off = tt * ROW + n + (n >> 6) * 4;
         *reinterpret_cast<float4*>(&qs[0][0] + off) = rq[u];
         *reinterpret_cast<float4*>(&ks[0][0] + off) = rk[u];
-        *reinterpret_cast<float4*>(&gs[0][0] + off) = rg[u];
+        if (!HD) *reinterpret_cast<float4*>(&gs[0][0] + off) = rg[u];
       }
     }
 #pragma unroll
@@ -339,34 +372,15 @@ __global__ __launch_bounds__(256) void decay_scan_staged_kernel(float* __restric
       if (i < TB * PB) (&vs[0][0])[i] = rv[u];
     }
     if (threadIdx.x < TB) kqs[threadIdx.x] = rs;
-    else if (DELTA && threadIdx.x < 2 * TB) bts[threadIdx.x - TB] = rs;
+    else if (MODE == kDelta && threadIdx.x < 2 * TB) bts[threadIdx.x - TB] = rs;
+    else if (HD && threadIdx.x >= 2 * TB && threadIdx.x < 3 * TB) ghs[threadIdx.x - 2 * TB] = rs;
     __syncthreads();
     if (tb + TB < t1) fetch(tb + TB);
 #pragma unroll 2
     for (int tt = 0; tt < nt; ++tt) {
-      const float4 g0 = *reinterpret_cast<const float4*>(&gs[tt][boff]);
-      const float4 g1 = *reinterpret_cast<const float4*>(&gs[tt][boff + 4]);
-      const float4 k0 = *reinterpret_cast<const float4*>(&ks[tt][boff]);
-      const float4 k1 = *reinterpret_cast<const float4*>(&ks[tt][boff + 4]);
-      const float4 q0 = *reinterpret_cast<const float4*>(&qs[tt][boff]);
-      const float4 q1 = *reinterpret_cast<const float4*>(&qs[tt][boff + 4]);
-      const float gv[8] = {g0.x, g0.y, g0.z, g0.w, g1.x, g1.y, g1.z, g1.w};
-      const float kv[8] = {k0.x, k0.y, k0.z, k0.w, k1.x, k1.y, k1.z, k1.w};
-      const float qv[8] = {q0.x, q0.y, q0.z, q0.w, q1.x, q1.y, q1.z, q1.w};
-      float pk = 0.f, pq = 0.f;
-#pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        S[i] *= gv[i];
-        if (DELTA) pk += S[i] * kv[i];
-        pq += S[i] * qv[i];
-      }
-      if (DELTA) pk = lanes_sum<CH>(pk);
-      pq = lanes_sum<CH>(pq);
-      const float v = vs[tt][pl];
-      const float u = DELTA ? bts[tt] * (v - pk) : v;
-#pragma unroll
-      for (int i = 0; i < 8; ++i) S[i] += kv[i] * u;
-      if (live && chunk == 0) op[(long)tt * inner] = pq + u * kqs[tt];
+      const float r = scan_token<CH, MODE, HD>(S, &gs[HD ? 0 : tt][HD ? 0 : boff], HD ? ghs[tt] : 0.f, &ks[tt][boff],
+                                               &qs[tt][boff], vs[tt][pl], MODE == kDelta ? bts[tt] : 0.f, kqs[tt]);
+      if (live && chunk == 0) op[(long)tt * inner] = r;
     }
     op += (long)TB * inner;
   }
@@ -386,51 +400,68 @@ __global__ __launch_bounds__(256) void decay_scan_staged_kernel(float* __restric
 
 using namespace k8sllm;
 
-template <typename T, bool DELTA>
-static int launch_decay_scan(float* o, const void* qkv, long stride, int q_col, int k_col, int v_col, const void* z,
-                             long z_stride, const float* z_bias, const float* a_log, float inv_tau, const void* beta,
-                             long b_stride, float* state, const int* cu, const int* ctx, const int* slot, int S, int H,
-                             int Gk, int dk, int dv, float q_scale, int unit, hipStream_t s) {
-#define K8SLLM_DS(CH)                                                                                                  \
-  hipLaunchKernelGGL((decay_scan_kernel<T, CH, DELTA>),                                                                \
-                     dim3((unsigned)S, (unsigned)H, (unsigned)((dv + 256 / CH - 1) / (256 / CH))), dim3(256), 0, s, o,  \
-                     (const T*)qkv, stride, q_col, k_col, v_col, (const T*)z, z_stride, z_bias, a_log, inv_tau,         \
-                     (const T*)beta, b_stride, state, cu, ctx, slot, H, Gk, dk, dv, q_scale, unit)
-  if (dk <= 16) K8SLLM_DS(2);
-  else if (dk <= 32) K8SLLM_DS(4);
-  else if (dk <= 64) K8SLLM_DS(8);
-  else if (dk <= 128) K8SLLM_DS(16);
-  else if (dk <= 256) K8SLLM_DS(32);
+// one step's arguments, as k8sllm_hy_decay_scan takes them
+struct ScanArgs {
+  float* o;
+  const void* qkv;
+  long stride;
+  int q_col, k_col, v_col;
+  const void* z;
+  long z_stride;
+  const float *z_bias, *a_log;
+  float inv_tau;
+  int dkind;
+  const void* beta;
+  long b_stride;
+  const float* bonus;
+  float* state;
+  const int *cu, *ctx, *slot;
+  int S, H, Gk, dk, dv;
+  float q_scale;
+  int unit;
+  float* ws;
+  long rows;
+};
+
+template <typename T, int CH, int MODE, bool HD>
+static void launch_scan_ch(const ScanArgs& a, hipStream_t s) {
+  const dim3 grid((unsigned)a.S, (unsigned)a.H, (unsigned)((a.dv + 256 / CH - 1) / (256 / CH)));
+  if (a.ws == nullptr) {
+    hipLaunchKernelGGL((decay_scan_kernel<T, CH, MODE, HD>), grid, dim3(256), 0, s, a.o, (const T*)a.qkv, a.stride, a.q_col,
+                       a.k_col, a.v_col, (const T*)a.z, a.z_stride, a.z_bias, a.a_log, a.inv_tau, a.dkind,
+                       (const T*)a.beta, a.b_stride, a.bonus, a.state, a.cu, a.ctx, a.slot, a.H, a.Gk, a.dk, a.dv,
+                       a.q_scale, a.unit);
+    return;
+  }
+  float* qn = a.ws;
+  float* kn = qn + a.rows * a.Gk * a.dk;
+  float* gd = kn + a.rows * a.Gk * a.dk;
+  float* kq = gd + a.rows * a.H * (HD ? 1 : a.dk);
+  float* bt = kq + a.rows * a.Gk;
+  hipLaunchKernelGGL((decay_prep_kernel<T, HD>), dim3((unsigned)a.rows), dim3(256), 0, s, qn, kn, gd, kq, bt,
+                     (const T*)a.qkv, a.stride, a.q_col, a.k_col, (const T*)a.z, a.z_stride, a.z_bias, a.a_log, a.inv_tau,
+                     a.dkind, (const T*)a.beta, a.b_stride, a.bonus, a.H, a.Gk, a.dk, a.q_scale, a.unit);
+  hipLaunchKernelGGL((decay_scan_staged_kernel<T, CH, MODE, HD>), grid, dim3(256), 0, s, a.o, (const T*)a.qkv, a.stride,
+                     a.v_col, qn, kn, gd, kq, bt, a.state, a.cu, a.ctx, a.slot, a.H, a.Gk, a.dk, a.dv);
+}
+
+template <typename T, int MODE, bool HD>
+static int launch_scan_mode(const ScanArgs& a, hipStream_t s) {
+  if (a.dk <= 16) launch_scan_ch<T, 2, MODE, HD>(a, s);
+  else if (a.dk <= 32) launch_scan_ch<T, 4, MODE, HD>(a, s);
+  else if (a.dk <= 64) launch_scan_ch<T, 8, MODE, HD>(a, s);
+  else if (a.dk <= 128) launch_scan_ch<T, 16, MODE, HD>(a, s);
+  else if (a.dk <= 256) launch_scan_ch<T, 32, MODE, HD>(a, s);
   else return -1;
-#undef K8SLLM_DS
   return (int)hipGetLastError();
 }
 
-template <typename T, bool DELTA>
-static int launch_decay_staged(float* o, const void* qkv, long stride, int q_col, int k_col, int v_col, const void* z,
-                               long z_stride, const float* z_bias, const float* a_log, float inv_tau, const void* beta,
-                               long b_stride, float* state, const int* cu, const int* ctx, const int* slot, int S, int H,
-                               int Gk, int dk, int dv, float q_scale, int unit, float* ws, long rows, hipStream_t s) {
-  float* qn = ws;
-  float* kn = qn + rows * Gk * dk;
-  float* gd = kn + rows * Gk * dk;
-  float* kq = gd + rows * H * dk;
-  float* bt = kq + rows * Gk;
-  hipLaunchKernelGGL(decay_prep_kernel<T>, dim3((unsigned)rows), dim3(256), 0, s, qn, kn, gd, kq, bt,
-                     (const T*)qkv, stride, q_col, k_col, (const T*)z, z_stride, z_bias, a_log, inv_tau, (const T*)beta,
-                     b_stride, H, Gk, dk, q_scale, unit);
-#define K8SLLM_DS(CH)                                                                                                  \
-  hipLaunchKernelGGL((decay_scan_staged_kernel<T, CH, DELTA>),                                                         \
-                     dim3((unsigned)S, (unsigned)H, (unsigned)((dv + 256 / CH - 1) / (256 / CH))), dim3(256), 0, s, o,  \
-                     (const T*)qkv, stride, v_col, qn, kn, gd, kq, bt, state, cu, ctx, slot, H, Gk, dk, dv)
-  if (dk <= 16) K8SLLM_DS(2);
-  else if (dk <= 32) K8SLLM_DS(4);
-  else if (dk <= 64) K8SLLM_DS(8);
-  else if (dk <= 128) K8SLLM_DS(16);
-  else if (dk <= 256) K8SLLM_DS(32);
-  else return -1;
-#undef K8SLLM_DS
-  return (int)hipGetLastError();
+template <typename T>
+static int launch_scan_t(const ScanArgs& a, int mode, int per_head, hipStream_t s) {
+  if (mode == kDelta) return per_head ? launch_scan_mode<T, kDelta, true>(a, s) : launch_scan_mode<T, kDelta, false>(a, s);
+  if (per_head) return -1;  // one decay per head is built for the delta rule
+  if (mode == kBonus) return launch_scan_mode<T, kBonus, false>(a, s);
+  return launch_scan_mode<T, kPlain, false>(a, s);
 }
 
 extern "C" {
@@ -438,28 +469,21 @@ extern "C" {
 // floats of workspace the two-launch form needs for T rows
 long k8sllm_hy_decay_scan_ws(long T, int H, int Gk, int dk) { return T * ((long)2 * Gk * dk + (long)H * dk + Gk + H); }
 
-// beta == nullptr: no delta rule.  a_log == nullptr: decays sigmoid(z + bias)^(inv_tau).  ws != nullptr: the
-// two-launch form for prompts, with k8sllm_hy_decay_scan_ws(T, ...) floats of workspace (T = rows of the step)
+// beta != nullptr: the delta rule; bonus != nullptr ([H][dk], Gk == H): the bonus form; neither: plain.
+// dkind: 0 exp(-exp(a_log) softplus(x)), 1 sigmoid(x)^(inv_tau), 2 exp(-exp(x)).  per_head: z and z_bias hold
+// one decay logit per head.  ws != nullptr: the two-launch form for prompts, with
+// k8sllm_hy_decay_scan_ws(T, ...) floats of workspace (T = rows of the step)
 int k8sllm_hy_decay_scan(float* o, const void* qkv, long stride, int q_col, int k_col, int v_col, const void* z,
-                         long z_stride, const float* z_bias, const float* a_log, float inv_tau, const void* beta,
-                         long b_stride, float* state, const int* cu, const int* ctx, const int* slot, int S, int H, int Gk,
-                         int dk, int dv, float q_scale, int unit, int f32, float* ws, long T, hipStream_t s) {
+                         long z_stride, const float* z_bias, const float* a_log, float inv_tau, int dkind, int per_head,
+                         const void* beta, long b_stride, const float* bonus, float* state, const int* cu,
+                         const int* ctx, const int* slot, int S, int H, int Gk, int dk, int dv, float q_scale, int unit,
+                         int f32, float* ws, long T, hipStream_t s) {
   if (S <= 0) return 0;
-  if (Gk < 1 || H % Gk || dk < 1 || dv < 1) return -1;
-  if (ws != nullptr) {
-#define K8SLLM_ARGS2                                                                                                 \
-  o, qkv, stride, q_col, k_col, v_col, z, z_stride, z_bias, a_log, inv_tau, beta, b_stride, state, cu, ctx, slot, S, H, \
-      Gk, dk, dv, q_scale, unit, ws, T, s
-    if (beta != nullptr)
-      return f32 ? launch_decay_staged<float, true>(K8SLLM_ARGS2) : launch_decay_staged<bf16_t, true>(K8SLLM_ARGS2);
-    return f32 ? launch_decay_staged<float, false>(K8SLLM_ARGS2) : launch_decay_staged<bf16_t, false>(K8SLLM_ARGS2);
-#undef K8SLLM_ARGS2
-  }
-#define K8SLLM_ARGS                                                                                                  \
-  o, qkv, stride, q_col, k_col, v_col, z, z_stride, z_bias, a_log, inv_tau, beta, b_stride, state, cu, ctx, slot, S, H, \
-      Gk, dk, dv, q_scale, unit, s
-  if (beta != nullptr) return f32 ? launch_decay_scan<float, true>(K8SLLM_ARGS) : launch_decay_scan<bf16_t, true>(K8SLLM_ARGS);
-  return f32 ? launch_decay_scan<float, false>(K8SLLM_ARGS) : launch_decay_scan<bf16_t, false>(K8SLLM_ARGS);
-#undef K8SLLM_ARGS
+  if (Gk < 1 || H % Gk || dk < 1 || dv < 1 || dkind < 0 || dkind > 2 || (dkind == 0 && a_log == nullptr)) return -1;
+  if (bonus != nullptr && (beta != nullptr || Gk != H)) return -1;
+  const ScanArgs a = {o, qkv, stride, q_col, k_col, v_col, z, z_stride, z_bias, a_log, inv_tau, dkind, beta, b_stride, bonus,
+                      state, cu, ctx, slot, S, H, Gk, dk, dv, q_scale, unit, ws, T};
+  const int mode = beta != nullptr ? kDelta : bonus != nullptr ? kBonus : kPlain;
+  return f32 ? launch_scan_t<float>(a, mode, per_head, s) : launch_scan_t<bf16_t>(a, mode, per_head, s);
 }
 }

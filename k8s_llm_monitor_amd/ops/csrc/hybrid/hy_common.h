@@ -79,6 +79,20 @@ __device__ __forceinline__ float wave_max_dpp(float v) {
 __device__ __forceinline__ float silu_f(float z) { return z / (1.f + __expf(-z)); }
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
 
+// sum over groups of CH neighbouring lanes (CH a power of two <= 32, groups aligned); every lane of a group
+// ends with its total
+template <int CH>
+__device__ __forceinline__ float lanes_sum(float v) {
+  if (CH >= 2) v += K8SLLM_DPP(v, 0xB1);
+  if (CH >= 4) v += K8SLLM_DPP(v, 0x4E);
+  if (CH >= 8) v += K8SLLM_DPP(v, 0x141);
+  if (CH >= 16) v += K8SLLM_DPP(v, 0x140);
+  if (CH >= 32) v = xor16_sum(v);
+  return v;
+}
+
+__device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
+
 // the segment that holds row r: largest s with cu[s] <= r (cu has S + 1 entries, cu[0] = 0)
 __device__ __forceinline__ int find_segment(const int* __restrict__ cu, int S, int r) {
   int lo = 0, hi = S - 1;

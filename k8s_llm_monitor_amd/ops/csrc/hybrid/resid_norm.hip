@@ -6,7 +6,7 @@
 //   norm_shift        h[t] = x[t] / rms(x[t]) * w;  out[t] = h[t] + (h[t-1] - h[t]) * mu, the row before
 //                     a segment from the sequence's state slot; shift_state advances the slots
 //   depth_mix         stack[n] += addend;  stack[n+1] = sum_j coef[j] * stack[j], j = 0 .. n
-//   activation        erf GELU, tanh GELU, xIELU or SiLU, elementwise in fp32 (also over a column range)
+//   activation        erf GELU, tanh GELU, xIELU, SiLU, squared ReLU or tanh, elementwise in fp32 (also over a column range)
 //   gated_add_norm    residual += mult * y * sigmoid(gate + bias);  out = residual / rms(residual) * w
 //   glu               out = act(gu[:, :f]) * gu[:, f:2f]           (rows may be wider than 2f)
 //   norm_gate         out = y / rms(y) * w * sigmoid(z)            (y fp32)
@@ -14,6 +14,9 @@
 //   softcap           x = cap * tanh(x / cap), in place (fp32 logits)
 //   sum_norm          residual += s0 a0 + s1 a1 + y / rms(y) * wy;  out = RMS or layer norm of it times w
 //                     (or the new residual itself, rounded to the activation dtype)
+//   join_norm         residual += LN(branch) * pw + pb, the branch one result or mix times the sum of two
+//                     RMS-normed ones;  out = LN(residual) * nw + nb
+//   token_mix         out[t][j] = h[t] + (h[t-1] - h[t]) * mu[j], the row before a segment from the sequence's slot
 //   gated_lookup      out = gelu_tanh(gate) * table[id][col : col + n]
 #include "hy_common.h"
 
@@ -335,9 +338,11 @@ __global__ __launch_bounds__(256) void depth_mix_scalar_kernel(float* __restrict
 }
 
 // KIND 0: erf GELU, 1: tanh GELU, 2: xIELU (a z^2 + z/2 above zero, b (exp(z) - 1 - z) + z/2 below), 3: SiLU,
-// 4: ReLU
+// 4: ReLU, 6: squared ReLU, 7: tanh (5 is a gated unit, glu_unit)
 template <int KIND>
 __device__ __forceinline__ float act_f(float z, float a, float b) {
+  if (KIND == 6) return z > 0.f ? z * z : 0.f;
+  if (KIND == 7) return tanhf(z);
   if (KIND == 4) return fmaxf(z, 0.f);
   if (KIND == 0) return 0.5f * z * (1.f + erff(z * 0.70710678118654752f));
   if (KIND == 1) return 0.5f * z * (1.f + tanhf(0.79788456080286536f * (z + 0.044715f * z * z * z)));
@@ -548,6 +553,208 @@ __global__ __launch_bounds__(256) void sum_norm_kernel(T* __restrict__ out, floa
   }
 }
 
+// V consecutive elements as floats and back (V 4: 8 / 16-byte accesses; V 1: one element)
+template <int V>
+__device__ __forceinline__ void ldv(const float* p, float* f) {
+  if constexpr (V == 4) {
+    const float4 a = *reinterpret_cast<const float4*>(p);
+    f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w;
+  } else {
+    f[0] = *p;
+  }
+}
+template <int V>
+__device__ __forceinline__ void ldv_any(const void* p, int dt, long i, float* f) {
+  if (dt == 2) {
+    ldv<V>(reinterpret_cast<const float*>(p) + i, f);
+  } else if constexpr (V == 4) {
+    const uint2 u = *reinterpret_cast<const uint2*>(reinterpret_cast<const bf16_t*>(p) + i);
+    f[0] = __uint_as_float(u.x << 16); f[1] = __uint_as_float(u.x & 0xffff0000u);
+    f[2] = __uint_as_float(u.y << 16); f[3] = __uint_as_float(u.y & 0xffff0000u);
+  } else {
+    f[0] = bf2f(reinterpret_cast<const bf16_t*>(p)[i]);
+  }
+}
+template <int V>
+__device__ __forceinline__ void stv(float* p, const float* f) {
+  if constexpr (V == 4) *reinterpret_cast<float4*>(p) = make_float4(f[0], f[1], f[2], f[3]);
+  else *p = f[0];
+}
+template <int V>
+__device__ __forceinline__ void stv(bf16_t* p, const float* f) {
+  if constexpr (V == 4) {
+    uint2 u;
+    u.x = pack2(f[0], f[1]);
+    u.y = pack2(f[2], f[3]);
+    *reinterpret_cast<uint2*>(p) = u;
+  } else {
+    *p = f2bf(f[0]);
+  }
+}
+
+// The mean of a row held in registers (NV x V elements per thread, zeros beyond d), then 1 / sqrt(variance + eps)
+// with the variance taken from the deviations.
+template <int V, int NV>
+__device__ __forceinline__ void row_stats(const float (&x)[NV][V], int d, float eps, float* red, float& mean, float& inv) {
+  float s = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i)
+#pragma unroll
+    for (int k = 0; k < V; ++k) s += x[i][k];
+  mean = block_sum<256>(s, red) / (float)d;
+  float q = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i)
+    if ((threadIdx.x + 256 * i) * V < d) {
+#pragma unroll
+      for (int k = 0; k < V; ++k) q += (x[i][k] - mean) * (x[i][k] - mean);
+    }
+  inv = 1.0f / sqrtf(block_sum<256>(q, red) / (float)d + eps);
+}
+
+// Post-norm and pre-norm in one launch, one workgroup per row, the row in registers (V = 4: d a multiple of 4):
+//   branch b = y0, or mix * (y0 / rms(y0) * w0 + y1 / rms(y1) * w1) where y1 is given;
+//   residual += LN(b) * pw + pb;   out = LN(residual) * nw + nb.
+// t0 / t1: dtype of y0 / y1 (0 absent, 1 bf16, 2 fp32).  y0 absent: the residual as it is; nw == nullptr: no out.
+template <typename T, int V, int NV>
+__global__ __launch_bounds__(256) void join_norm_kernel(T* __restrict__ out, float* __restrict__ residual,
+                                                        const void* __restrict__ y0, int t0,
+                                                        const void* __restrict__ y1, int t1,
+                                                        const float* __restrict__ w0, const float* __restrict__ w1,
+                                                        float mix, const float* __restrict__ pw,
+                                                        const float* __restrict__ pb, const float* __restrict__ nw,
+                                                        const float* __restrict__ nb, int d, float eps) {
+  __shared__ float red[4];
+  const long row = blockIdx.x, base = row * d;
+  float* r = residual + base;
+  float x[NV][V];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + 256 * i) * V;
+    if (c < d) {
+      ldv<V>(r + c, x[i]);
+    } else {
+#pragma unroll
+      for (int k = 0; k < V; ++k) x[i][k] = 0.f;
+    }
+  }
+  float mean, inv;
+  if (t0) {
+    float y[NV][V];
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = (threadIdx.x + 256 * i) * V;
+      if (c < d) {
+        ldv_any<V>(y0, t0, base + c, y[i]);
+      } else {
+#pragma unroll
+        for (int k = 0; k < V; ++k) y[i][k] = 0.f;
+      }
+    }
+    if (t1) {
+      float u[NV][V], sa = 0.f, sb = 0.f;
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = (threadIdx.x + 256 * i) * V;
+        if (c < d) {
+          ldv_any<V>(y1, t1, base + c, u[i]);
+        } else {
+#pragma unroll
+          for (int k = 0; k < V; ++k) u[i][k] = 0.f;
+        }
+#pragma unroll
+        for (int k = 0; k < V; ++k) {
+          sa += y[i][k] * y[i][k];
+          sb += u[i][k] * u[i][k];
+        }
+      }
+      const float ia = mix / sqrtf(block_sum<256>(sa, red) / (float)d + eps);
+      const float ib = mix / sqrtf(block_sum<256>(sb, red) / (float)d + eps);
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = (threadIdx.x + 256 * i) * V;
+        if (c < d) {
+          float a[V], b[V];
+          ldv<V>(w0 + c, a);
+          ldv<V>(w1 + c, b);
+#pragma unroll
+          for (int k = 0; k < V; ++k) y[i][k] = y[i][k] * ia * a[k] + u[i][k] * ib * b[k];
+        }
+      }
+    }
+    row_stats<V, NV>(y, d, eps, red, mean, inv);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = (threadIdx.x + 256 * i) * V;
+      if (c < d) {
+        float a[V], b[V];
+        ldv<V>(pw + c, a);
+        ldv<V>(pb + c, b);
+#pragma unroll
+        for (int k = 0; k < V; ++k) x[i][k] += (y[i][k] - mean) * inv * a[k] + b[k];
+        stv<V>(r + c, x[i]);
+      }
+    }
+  }
+  if (nw == nullptr) return;
+  row_stats<V, NV>(x, d, eps, red, mean, inv);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + 256 * i) * V;
+    if (c < d) {
+      float a[V], b[V];
+      ldv<V>(nw + c, a);
+      ldv<V>(nb + c, b);
+#pragma unroll
+      for (int k = 0; k < V; ++k) a[k] = (x[i][k] - mean) * inv * a[k] + b[k];
+      stv<V>(out + base + c, a);
+    }
+  }
+}
+
+// Token-shift mixes of normed rows: out[t][j] = h[t] + (h[t-1] - h[t]) * mu[j] for j < n, rows of out n * d wide.
+// The row before a segment's first is the sequence's slot (zeros where the sequence starts here); that first
+// row's workgroup then writes the segment's last row to the slot (each thread replaces only what it has read).
+template <typename T, int V>
+__global__ __launch_bounds__(256) void token_mix_kernel(T* __restrict__ out, const float* __restrict__ h,
+                                                        const float* __restrict__ mu, int n, float* __restrict__ state,
+                                                        const int* __restrict__ cu, const int* __restrict__ ctx,
+                                                        const int* __restrict__ slot, int S, int d) {
+  const long row = blockIdx.x;
+  const int s = find_segment(cu, S, (int)row);
+  const bool first = row == cu[s];
+  const int sl = slot[s];
+  const bool carried = first && sl >= 0 && ctx[s] > 0;
+  const float* hr = h + row * d;
+  float* st = sl >= 0 ? state + (long)sl * d : nullptr;
+  const float* last = h + (long)(cu[s + 1] - 1) * d;
+  T* o = out + row * n * d;
+  for (int c = threadIdx.x * V; c < d; c += 256 * V) {
+    float x[V], p[V], m[V];
+    ldv<V>(hr + c, x);
+    if (!first) {
+      ldv<V>(hr - d + c, p);
+    } else if (carried) {
+      ldv<V>(st + c, p);
+    } else {
+#pragma unroll
+      for (int k = 0; k < V; ++k) p[k] = 0.f;
+    }
+#pragma unroll
+    for (int k = 0; k < V; ++k) p[k] -= x[k];
+    for (int j = 0; j < n; ++j) {
+      ldv<V>(mu + (long)j * d + c, m);
+#pragma unroll
+      for (int k = 0; k < V; ++k) m[k] = x[k] + p[k] * m[k];
+      stv<V>(o + (long)j * d + c, m);
+    }
+    if (first && st != nullptr) {
+      ldv<V>(last + c, x);
+      stv<V>(st + c, x);
+    }
+  }
+}
+
 // out[t][c] = gelu_tanh(gate[t][c]) * table[id(t)][col + c]; ids resolved as in embed_pos
 template <typename T>
 __global__ __launch_bounds__(256) void gated_lookup_kernel(T* __restrict__ out, const T* __restrict__ gate,
@@ -734,9 +941,9 @@ int k8sllm_hy_activation(void* out, const void* x, long n, int kind, float a, fl
   const dim3 g((unsigned)((n + 2047) / 2048));
 #define K8SLLM_ACT(T, K) hipLaunchKernelGGL((activation_kernel<T, K>), g, dim3(256), 0, s, (T*)out, (const T*)x, n, a, b)
   if (f32) {
-    if (kind == 0) K8SLLM_ACT(float, 0); else if (kind == 1) K8SLLM_ACT(float, 1); else if (kind == 2) K8SLLM_ACT(float, 2); else if (kind == 3) K8SLLM_ACT(float, 3); else return -1;
+    if (kind == 0) K8SLLM_ACT(float, 0); else if (kind == 1) K8SLLM_ACT(float, 1); else if (kind == 2) K8SLLM_ACT(float, 2); else if (kind == 3) K8SLLM_ACT(float, 3); else if (kind == 6) K8SLLM_ACT(float, 6); else if (kind == 7) K8SLLM_ACT(float, 7); else return -1;
   } else {
-    if (kind == 0) K8SLLM_ACT(bf16_t, 0); else if (kind == 1) K8SLLM_ACT(bf16_t, 1); else if (kind == 2) K8SLLM_ACT(bf16_t, 2); else if (kind == 3) K8SLLM_ACT(bf16_t, 3); else return -1;
+    if (kind == 0) K8SLLM_ACT(bf16_t, 0); else if (kind == 1) K8SLLM_ACT(bf16_t, 1); else if (kind == 2) K8SLLM_ACT(bf16_t, 2); else if (kind == 3) K8SLLM_ACT(bf16_t, 3); else if (kind == 6) K8SLLM_ACT(bf16_t, 6); else if (kind == 7) K8SLLM_ACT(bf16_t, 7); else return -1;
   }
 #undef K8SLLM_ACT
   return (int)hipGetLastError();
@@ -753,6 +960,47 @@ int k8sllm_hy_sum_norm(void* out, float* residual, const void* a0, int t0, float
   else
     hipLaunchKernelGGL(sum_norm_kernel<bf16_t>, dim3(rows), dim3(256), 0, s, (bf16_t*)out, residual, a0, t0, s0, a1, t1,
                        s1, y, ty, wy, w, d, eps, center, one_plus);
+  return (int)hipGetLastError();
+}
+
+// t0, t1: 0 absent, 1 bf16, 2 fp32.  d up to 8192
+int k8sllm_hy_join_norm(void* out, float* residual, const void* y0, int t0, const void* y1, int t1, const float* w0,
+                        const float* w1, float mix, const float* pw, const float* pb, const float* nw, const float* nb,
+                        long rows, int d, float eps, int f32, hipStream_t s) {
+  if (rows <= 0) return 0;
+#define K8SLLM_JN(V, NV)                                                                                              \
+  if (f32)                                                                                                            \
+    hipLaunchKernelGGL((join_norm_kernel<float, V, NV>), dim3((unsigned)rows), dim3(256), 0, s, (float*)out, residual,  \
+                       y0, t0, y1, t1, w0, w1, mix, pw, pb, nw, nb, d, eps);                                           \
+  else                                                                                                                \
+    hipLaunchKernelGGL((join_norm_kernel<bf16_t, V, NV>), dim3((unsigned)rows), dim3(256), 0, s, (bf16_t*)out,          \
+                       residual, y0, t0, y1, t1, w0, w1, mix, pw, pb, nw, nb, d, eps)
+  if (d % 4 == 0) {
+    if (d <= 1024) { K8SLLM_JN(4, 1); }
+    else if (d <= 2048) { K8SLLM_JN(4, 2); }
+    else if (d <= 4096) { K8SLLM_JN(4, 4); }
+    else if (d <= 8192) { K8SLLM_JN(4, 8); }
+    else return -1;
+  } else if (d <= 256) { K8SLLM_JN(1, 1); }
+  else if (d <= 2048) { K8SLLM_JN(1, 8); }
+  else if (d <= 8192) { K8SLLM_JN(1, 32); }
+  else return -1;
+#undef K8SLLM_JN
+  return (int)hipGetLastError();
+}
+
+int k8sllm_hy_token_mix(void* out, const float* h, const float* mu, int n, float* state, const int* cu, const int* ctx,
+                        const int* slot, int S, long rows, int d, int f32, hipStream_t s) {
+  if (rows <= 0 || S <= 0) return 0;
+#define K8SLLM_TM(T_, V)                                                                                              \
+  hipLaunchKernelGGL((token_mix_kernel<T_, V>), dim3((unsigned)rows), dim3(256), 0, s, (T_*)out, h, mu, n, state, cu, ctx, \
+                     slot, S, d)
+  if (f32) {
+    if (d % 4 == 0) K8SLLM_TM(float, 4); else K8SLLM_TM(float, 1);
+  } else {
+    if (d % 4 == 0) K8SLLM_TM(bf16_t, 4); else K8SLLM_TM(bf16_t, 1);
+  }
+#undef K8SLLM_TM
   return (int)hipGetLastError();
 }
 

@@ -4,7 +4,9 @@
 //   window_attention_decode   one wave per (sequence, query head)
 // Pages: k_cache [blocks][BS][G*dk] (a token's keys contiguous), v_cache [blocks][G][dv][BS] (a value
 // dim's BS tokens contiguous: the layout the PV products read along); a sequence's page list is a row of
-// block_tables.  Row at position p sees positions max(0, p - window + 1) .. p (window 0: 0 .. p).
+// block_tables.  Row at position p sees positions max(0, p - window + 1) .. p (window 0: 0 .. p), or with
+// ``chunked`` the positions from its chunk's first on: floor(p / window) * window .. p (chunks are counted
+// from position 0 of the sequence).  cap > 0: a score s (after the scale) becomes cap * tanh(s / cap).
 // The sink is one more softmax term with no value and a fixed score - 0, or a learned unscaled logit
 // per query head (sinks[h]): the running maximum starts at that score and the running denominator at 1.  Scores, weights and the output accumulation are fp32.
 #include "hy_common.h"
@@ -15,6 +17,17 @@ constexpr int kMaxVC = 4;  // output dims per lane of the vector decode kernel: 
 constexpr int kMaxDK = 512;
 constexpr int kGenVC = 8;  // the any-size kernels: dv <= 64 * kGenVC, dk <= kGenDK
 constexpr int kGenDK = 1024;
+
+// the first position that a row at position p sees
+__device__ __forceinline__ int first_key(int p, int window, int chunked) {
+  if (window <= 0) return 0;
+  return chunked ? p - p % window : max(0, p - window + 1);
+}
+// tanh from one exponential and one reciprocal: absolute error about 1e-7 (the bf16 kernels' scores; the
+// any-size kernels call tanhf)
+__device__ __forceinline__ float tanh_exp2(float x) {
+  return 1.f - 2.f * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x * 2.88539008177792681f));
+}
 
 template <typename T>
 __global__ __launch_bounds__(256) void qk_norm_cache_kernel(T* __restrict__ qkv, long stride,
@@ -52,7 +65,8 @@ template <typename T>
 __device__ __forceinline__ void attend_wave(T* __restrict__ out_row, const T* __restrict__ q_row,
                                             const T* __restrict__ k_cache, const T* __restrict__ v_cache,
                                             const int* __restrict__ bt, int lo, int hi, int g, int G, int dk, int dv,
-                                            int bs, float scale, int sink, float sink_z, float* q_s, float* p_s) {
+                                            int bs, float scale, float cap, int sink, float sink_z, float* q_s,
+                                            float* p_s) {
   const int lane = threadIdx.x & 63;
   for (int c = lane; c < dk; c += 64) q_s[c] = ldf(q_row + c) * scale;
   __syncthreads();  // one wave per workgroup: orders the LDS writes before the other lanes' reads
@@ -68,7 +82,7 @@ __device__ __forceinline__ void attend_wave(T* __restrict__ out_row, const T* __
       const T* kp = k_cache + ((long)bt[j / bs] * bs + j % bs) * krow + (long)g * dk;
       float a = 0.f;
       for (int c = 0; c < dk; ++c) a += q_s[c] * ldf(kp + c);
-      s = a;
+      s = cap > 0.f ? cap * tanhf(a / cap) : a;
     }
     const float mt = fmaxf(m, wave_max_dpp(s));
     const float p = j < hi ? expf(s - mt) : 0.f;
@@ -106,15 +120,16 @@ __global__ __launch_bounds__(64) void window_prefill_kernel(T* __restrict__ out,
                                                             const int* __restrict__ cu, const int* __restrict__ ctx,
                                                             const int* __restrict__ block_tables, int bt_stride, int S,
                                                             int Hq, int G, int dk, int dv, int bs, float scale,
-                                                            int window, int sink, const float* __restrict__ sinks) {
+                                                            int window, int chunked, float cap, int sink,
+                                                            const float* __restrict__ sinks) {
   __shared__ float q_s[kGenDK];
   __shared__ float p_s[64];
   const int r = blockIdx.x, h = blockIdx.y;
   const int s = find_segment(cu, S, r);
   const int p = ctx[s] + r - cu[s];
-  const int lo = window > 0 ? max(0, p - window + 1) : 0;
+  const int lo = first_key(p, window, chunked);
   attend_wave<T>(out + (long)r * Hq * dv + (long)h * dv, qkv + (long)r * q_stride + (long)h * dk, k_cache, v_cache,
-                 block_tables + (long)s * bt_stride, lo, p + 1, h / (Hq / G), G, dk, dv, bs, scale, sink,
+                 block_tables + (long)s * bt_stride, lo, p + 1, h / (Hq / G), G, dk, dv, bs, scale, cap, sink,
                  sinks != nullptr ? sinks[h] : 0.f, q_s, p_s);
 }
 
@@ -124,8 +139,8 @@ __global__ __launch_bounds__(64) void window_decode_kernel(T* __restrict__ out, 
                                                            const T* __restrict__ v_cache,
                                                            const int* __restrict__ block_tables, int bt_stride,
                                                            const int* __restrict__ seq_lens, int Hq, int G, int dk,
-                                                           int dv, int bs, float scale, int window, int sink,
-                                                           const float* __restrict__ sinks) {
+                                                           int dv, int bs, float scale, int window, int chunked,
+                                                           float cap, int sink, const float* __restrict__ sinks) {
   __shared__ float q_s[kGenDK];
   __shared__ float p_s[64];
   const int b = blockIdx.x, h = blockIdx.y;
@@ -135,9 +150,9 @@ __global__ __launch_bounds__(64) void window_decode_kernel(T* __restrict__ out, 
     for (int c = threadIdx.x; c < dv; c += 64) stf(o + c, 0.f);
     return;
   }
-  const int lo = window > 0 ? max(0, n - window) : 0;
+  const int lo = first_key(n - 1, window, chunked);
   attend_wave<T>(o, qkv + (long)b * q_stride + (long)h * dk, k_cache, v_cache, block_tables + (long)b * bt_stride, lo,
-                 n, h / (Hq / G), G, dk, dv, bs, scale, sink, sinks != nullptr ? sinks[h] : 0.f, q_s, p_s);
+                 n, h / (Hq / G), G, dk, dv, bs, scale, cap, sink, sinks != nullptr ? sinks[h] : 0.f, q_s, p_s);
 }
 
 // bf16 decode with 16-byte loads, 16-token pages: one workgroup (NW = 8 waves; 4 for 8 query heads
@@ -154,8 +169,8 @@ __global__ __launch_bounds__(64 * NW) void window_decode_vec_kernel(bf16_t* __re
                                                                 const bf16_t* __restrict__ v_cache,
                                                                 const int* __restrict__ block_tables, int bt_stride,
                                                                 const int* __restrict__ seq_lens, int Hq, int G, int dk,
-                                                                int dv, float scale, int window, int sink,
-                                                                const float* __restrict__ sinks) {
+                                                                int dv, float scale, int window, int chunked, float cap,
+                                                                int sink, const float* __restrict__ sinks) {
   constexpr int bs = 16;
   __shared__ __attribute__((aligned(16))) float q_s[R * kMaxDK];
   __shared__ __attribute__((aligned(16))) float p_s[NW][R][64];
@@ -172,7 +187,8 @@ __global__ __launch_bounds__(64 * NW) void window_decode_vec_kernel(bf16_t* __re
   for (int c = threadIdx.x; c < R * dk; c += 64 * NW) q_s[(c / dk) * kMaxDK + c % dk] = bf2f(q[c]) * (scale * 1.44269504088896341f);  // base-2 scores
   __syncthreads();
   const int* bt = block_tables + (long)b * bt_stride;
-  const int lo = window > 0 ? max(0, n - window) : 0;
+  const int lo = first_key(n - 1, window, chunked);
+  const float cap2 = cap * 1.44269504088896341f, icap2 = cap > 0.f ? 1.f / cap2 : 0.f;  // base-2 scores
   const bool first = sink && wave == 0;
   float m[R], l[R], acc[R][kMaxVC];
 #pragma unroll
@@ -233,6 +249,7 @@ __global__ __launch_bounds__(64 * NW) void window_decode_vec_kernel(bf16_t* __re
     __builtin_amdgcn_wave_barrier();  // this wave's previous reads of its p_s rows come first
 #pragma unroll
     for (int r = 0; r < R; ++r) {
+      if (cap > 0.f) sc[r] = cap2 * tanh_exp2(sc[r] * icap2);
       const float sv = valid ? sc[r] : -INFINITY;
       const float mt = fmaxf(m[r], wave_max_dpp(sv));  // the tile holds at least one live key, or m is the sink's
       const float pw = (valid && mt != -INFINITY) ? __builtin_amdgcn_exp2f(sv - mt) : 0.f;
@@ -303,15 +320,16 @@ __global__ __launch_bounds__(64 * NW) void window_decode_vec_kernel(bf16_t* __re
 // With the query on the lane the running maximum, denominator and the rescale of O are lane-local
 // (two xor-shuffles per reduction).  Scores, weights and sums are fp32 (base-2 exponentials: the
 // scale carries log2 e); P is rounded to bf16 for the PV product.
-template <int DK, int DV, int QT>
+template <int DK, int DV, int QT, bool CAP>
 __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
     bf16_t* __restrict__ out, const bf16_t* __restrict__ qkv, long q_stride, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int* __restrict__ cu, const int* __restrict__ ctx,
     const int* __restrict__ block_tables, int bt_stride, int S, int Hq, int G, float scale, int window,
-    int sink, const float* __restrict__ sinks) {
+    int chunked, float cap, int sink, const float* __restrict__ sinks) {
   // pages hold 16 tokens; scores live in the base-2 domain (scale * log2 e folded in) so that every
   // exponential is one v_exp_f32
   const float sc2 = scale * 1.44269504088896341f;
+  const float cap2 = CAP ? cap * 1.44269504088896341f : 0.f, icap = CAP ? scale / cap : 0.f;
   constexpr int QB = 16 * QT;  // query rows per wave: QT tiles of 16 share every K and V^T fragment
   int tile = blockIdx.x, s = 0, n = 0;
   for (; s < S; ++s) {  // q-blocks are numbered segment by segment
@@ -335,7 +353,7 @@ __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
   for (int t = 0; t < QT; ++t) {
     const int myq = min(16 * t + c16, nq - 1);
     my_p[t] = p0 + myq;
-    my_lo[t] = window > 0 ? max(0, my_p[t] - window + 1) : 0;
+    my_lo[t] = first_key(my_p[t], window, chunked);
     q_live[t] = 16 * t + c16 < nq;
     const bf16_t* qrow = qkv + (long)(row0 + myq) * q_stride + (long)h * DK;
 #pragma unroll
@@ -345,7 +363,7 @@ __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
     m[t] = sink ? (sinks != nullptr ? sinks[blockIdx.y] * 1.44269504088896341f : 0.f) : -INFINITY;
     l[t] = sink ? 1.f : 0.f;
   }
-  const int lo_t = window > 0 ? max(0, p0 - window + 1) : 0, hi = p0 + nq;
+  const int lo_t = first_key(p0, window, chunked), hi = p0 + nq;
   const long krs = (long)G * DK, vrs = (long)G * DV;
   // Register double buffer: while tile j0 is computed, the K and V^T fragments of tile j0 + 16 are
   // in flight, and the page id of tile j0 + 32 behind them (no load waits on a load issued in the
@@ -391,7 +409,7 @@ __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
 #pragma unroll
       for (int i = 0; i < 4; ++i) {  // sacc[i]: key j0 + 4 quad + i, query 16 t + c16
         const int j = j0 + 4 * quad + i;
-        sv[i] = (q_live[t] && j >= my_lo[t] && j <= my_p[t]) ? sacc[i] * sc2 : -INFINITY;
+        sv[i] = (q_live[t] && j >= my_lo[t] && j <= my_p[t]) ? (CAP ? cap2 * tanh_exp2(sacc[i] * icap) : sacc[i] * sc2) : -INFINITY;
         tmax = fmaxf(tmax, sv[i]);
       }
       tmax = xor32_max_f(xor16_max(tmax));
@@ -462,8 +480,8 @@ int k8sllm_hy_qk_norm_cache(void* qkv, long stride, const float* qw, const float
 
 int k8sllm_hy_window_prefill(void* out, const void* qkv, long q_stride, const void* k_cache, const void* v_cache,
                              const int* cu, const int* ctx, const int* block_tables, int bt_stride, int S, long T,
-                             int Hq, int G, int dk, int dv, int bs, float scale, int window, int sink,
-                             const float* sinks, int f32, int mfma, hipStream_t s) {
+                             int Hq, int G, int dk, int dv, int bs, float scale, int window, int chunked, float cap,
+                             int sink, const float* sinks, int f32, int mfma, hipStream_t s) {
   if (T <= 0 || S <= 0) return 0;
   if (dk > kGenDK || dv > 64 * kGenVC || G < 1 || Hq % G) return -1;
   // bf16 with matrix-core head sizes and 16-byte aligned rows: the MFMA kernel
@@ -472,14 +490,16 @@ int k8sllm_hy_window_prefill(void* out, const void* qkv, long q_stride, const vo
     // share every K / V^T fragment), else 16; mfma = 16 / 32 / 64 forces one (tests, measurements)
     const int qrows = mfma >= 16 ? mfma : (T * Hq >= 64 * 1024 ? 32 : 16);
     const dim3 grid((unsigned)(T / qrows + S), (unsigned)Hq);
-#define K8SLLM_WP(DK, DV, QT)                                                                                          \
-  hipLaunchKernelGGL((window_prefill_mfma_kernel<DK, DV, QT>), grid, dim3(64), 0, s, (bf16_t*)out, (const bf16_t*)qkv,  \
-                     q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, cu, ctx, block_tables, bt_stride, S, Hq, \
-                     G, scale, window, sink, sinks)
+#define K8SLLM_WPC(DK, DV, QT, CAP)                                                                                    \
+  hipLaunchKernelGGL((window_prefill_mfma_kernel<DK, DV, QT, CAP>), grid, dim3(64), 0, s, (bf16_t*)out,                 \
+                     (const bf16_t*)qkv, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, cu, ctx,             \
+                     block_tables, bt_stride, S, Hq, G, scale, window, chunked, cap, sink, sinks)
+#define K8SLLM_WP(DK, DV, QT) \
+  if (cap > 0.f) K8SLLM_WPC(DK, DV, QT, true); else K8SLLM_WPC(DK, DV, QT, false)
 #define K8SLLM_WPQ(DK, DV)                                       \
-  if (qrows == 64) K8SLLM_WP(DK, DV, 4);                         \
-  else if (qrows == 32) K8SLLM_WP(DK, DV, 2);                    \
-  else K8SLLM_WP(DK, DV, 1)
+  if (qrows == 64) { K8SLLM_WP(DK, DV, 4); }                     \
+  else if (qrows == 32) { K8SLLM_WP(DK, DV, 2); }                \
+  else { K8SLLM_WP(DK, DV, 1); }
     if (mfma >= 16 && mfma != 16 && mfma != 32 && mfma != 64) return -1;
     if (dk == 64 && dv == 64) { K8SLLM_WPQ(64, 64); }
     else if (dk == 64) { K8SLLM_WPQ(64, 128); }
@@ -487,23 +507,24 @@ int k8sllm_hy_window_prefill(void* out, const void* qkv, long q_stride, const vo
     else { K8SLLM_WPQ(128, 128); }
 #undef K8SLLM_WPQ
 #undef K8SLLM_WP
+#undef K8SLLM_WPC
     return (int)hipGetLastError();
   }
   if (f32)
     hipLaunchKernelGGL(window_prefill_kernel<float>, dim3(T, Hq), dim3(64), 0, s, (float*)out, (const float*)qkv,
                        q_stride, (const float*)k_cache, (const float*)v_cache, cu, ctx, block_tables, bt_stride, S, Hq,
-                       G, dk, dv, bs, scale, window, sink, sinks);
+                       G, dk, dv, bs, scale, window, chunked, cap, sink, sinks);
   else
     hipLaunchKernelGGL(window_prefill_kernel<bf16_t>, dim3(T, Hq), dim3(64), 0, s, (bf16_t*)out, (const bf16_t*)qkv,
                        q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, cu, ctx, block_tables, bt_stride, S,
-                       Hq, G, dk, dv, bs, scale, window, sink, sinks);
+                       Hq, G, dk, dv, bs, scale, window, chunked, cap, sink, sinks);
   return (int)hipGetLastError();
 }
 
 int k8sllm_hy_window_decode(void* out, const void* qkv, long q_stride, const void* k_cache, const void* v_cache,
                             const int* block_tables, int bt_stride, const int* seq_lens, int B, int Hq, int G, int dk,
-                            int dv, int bs, float scale, int window, int sink, const float* sinks, int f32, int vec,
-                            hipStream_t s) {
+                            int dv, int bs, float scale, int window, int chunked, float cap, int sink,
+                            const float* sinks, int f32, int vec, hipStream_t s) {
   if (B <= 0) return 0;
   if (dk > kGenDK || dv > 64 * kGenVC || G < 1 || Hq % G) return -1;
   const int R = Hq / G;
@@ -513,7 +534,7 @@ int k8sllm_hy_window_decode(void* out, const void* qkv, long q_stride, const voi
   hipLaunchKernelGGL((window_decode_vec_kernel<RR, (RR == 8 ? 4 : 8)>), dim3(B, G), dim3(RR == 8 ? 256 : 512), 0, s,     \
                      (bf16_t*)out, (const bf16_t*)qkv,                                                                  \
                      q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, bt_stride, seq_lens, Hq, G, \
-                     dk, dv, scale, window, sink, sinks)
+                     dk, dv, scale, window, chunked, cap, sink, sinks)
     if (R == 1) K8SLLM_WD(1);
     else if (R == 2) K8SLLM_WD(2);
     else if (R == 4) K8SLLM_WD(4);
@@ -524,11 +545,11 @@ int k8sllm_hy_window_decode(void* out, const void* qkv, long q_stride, const voi
   if (f32)
     hipLaunchKernelGGL(window_decode_kernel<float>, dim3(B, Hq), dim3(64), 0, s, (float*)out, (const float*)qkv,
                        q_stride, (const float*)k_cache, (const float*)v_cache, block_tables, bt_stride, seq_lens, Hq, G,
-                       dk, dv, bs, scale, window, sink, sinks);
+                       dk, dv, bs, scale, window, chunked, cap, sink, sinks);
   else
     hipLaunchKernelGGL(window_decode_kernel<bf16_t>, dim3(B, Hq), dim3(64), 0, s, (bf16_t*)out, (const bf16_t*)qkv,
                        q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, bt_stride, seq_lens, Hq,
-                       G, dk, dv, bs, scale, window, sink, sinks);
+                       G, dk, dv, bs, scale, window, chunked, cap, sink, sinks);
   return (int)hipGetLastError();
 }
 }

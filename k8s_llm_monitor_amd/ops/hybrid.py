@@ -6,7 +6,9 @@ average of layer results, latent (low-rank compressed) attention with rotary pos
 per-head sinks, and ungated experts with a softmax-over-all router; and the gated residual
 (a sublayer's result times the sigmoid of a projection of its input, scaled, then the norm),
 rotary grouped-query attention with per-head temperatures, the fixed-decay linear-attention
-recurrence, gated linear units and the logit soft cap.
+recurrence, gated linear units and the logit soft cap; and layer norms before and after a sublayer,
+token-shift mixes, attention within position chunks with capped scores, the selective scan (a decay per
+channel and state), linear attention with a current-token bonus and the delta rule with a decay per head.
 
 GPU tensors run the gfx950 kernels of ``_k8sllm_hybrid`` (``ops/csrc/hybrid``; built by
 ``python -m k8s_llm_monitor_amd.ops.build --only hybrid``) for bfloat16 and float32 activations
@@ -135,6 +137,61 @@ def sum_norm(residual: torch.Tensor, addends: tuple, normed: Optional[tuple], w:
     return out
 
 
+def join_norm(residual: torch.Tensor, branch: tuple, post: Optional[tuple], pre: Optional[tuple], eps: float,
+              out_dtype: torch.dtype, branch_w: Optional[tuple] = None, mix: float = 1.0) -> Optional[torch.Tensor]:
+    """A sublayer's result through a layer norm of its own into the stream, then the next sublayer's norm.
+    ``branch``: () (nothing joins), (y,) or (y0, y1) ([T, d] of any float dtype); two results are first
+    RMS-normed each and combined, ``b = mix * (y0 / rms(y0) * w0 + y1 / rms(y1) * w1)`` with ``branch_w`` =
+    (w0, w1).  ``residual`` (fp32 [T, d], updated in place) += ``LN(b) * post[0] + post[1]``; returns
+    ``LN(residual) * pre[0] + pre[1]`` in ``out_dtype`` (``pre`` None: nothing).  LN(x) = (x - mean) /
+    sqrt(mean((x - mean)^2) + eps).  Norms and sums are fp32."""
+    if not residual.is_cuda:
+        def ln(x, wb):
+            x = x - x.mean(-1, keepdim=True)
+            return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * wb[0].float() + wb[1].float()
+
+        if branch:
+            b = branch[0].float()
+            if len(branch) == 2:
+                ys = [y.float() for y in branch]
+                ys = [y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps) * w.float() for y, w in zip(ys, branch_w)]
+                b = mix * (ys[0] + ys[1])
+            residual += ln(b, post)
+        return ln(residual, pre).to(out_dtype) if pre is not None else None
+    out = torch.empty(residual.shape, dtype=out_dtype, device=residual.device) if pre is not None else None
+    y = list(branch) + [None] * (2 - len(branch))
+    w0, w1 = branch_w if len(branch) == 2 else (None, None)
+    pw, pb = post if branch else (None, None)
+    nw, nb = pre if pre is not None else (None, None)
+    native().join_norm(out, residual, y[0], y[1], w0, w1, float(mix), pw, pb, nw, nb, float(eps))
+    return out
+
+
+def token_mix(h: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, seg_cu: torch.Tensor, seg_ctx: torch.Tensor,
+              seg_slot: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """Token-shift mixes of normed rows ``h`` (fp32 [T, d]): [T, n, d] in ``out_dtype`` with
+    ``h[t] + (h[t-1] - h[t]) * mu[j]`` for the ``n`` rows of ``mu`` (fp32, up to 8).  The row before a
+    segment's first comes from ``state[slot]`` ([slots, d] fp32; zeros where seg_ctx is 0), which then
+    takes the segment's last row."""
+    T, d = h.shape
+    n = mu.shape[0]
+    if not h.is_cuda:
+        prev = torch.zeros_like(h)
+        prev[1:] = h[:-1]
+        cul = seg_cu.tolist()
+        for s, (c0, slot) in enumerate(zip(seg_ctx.tolist(), seg_slot.tolist())):
+            a, b = cul[s], cul[s + 1]
+            if b <= a:
+                continue
+            prev[a] = state[slot] if (c0 > 0 and slot >= 0) else 0.0
+            if slot >= 0:
+                state[slot] = h[b - 1]
+        return (h[:, None] + (prev - h)[:, None] * mu[None]).to(out_dtype)
+    out = torch.empty(T, n, d, dtype=out_dtype, device=h.device)
+    native().token_mix(out, h, mu, state, seg_cu, seg_ctx, seg_slot)
+    return out
+
+
 def gated_lookup(gate: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, col: int,
                  src: Optional[torch.Tensor] = None, prev: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``gelu_tanh(gate) * table[id, col : col + n]`` for ``gate`` [T, n]: a per-token table slice gated
@@ -220,7 +277,7 @@ def depth_mix(stack: torch.Tensor, n: int, addend: Optional[torch.Tensor], coef:
     return stack[n + 1]
 
 
-ACTS = {"gelu": 0, "gelu_tanh": 1, "xielu": 2, "silu": 3, "relu": 4, "clamped_swish": 5}
+ACTS = {"gelu": 0, "gelu_tanh": 1, "xielu": 2, "silu": 3, "relu": 4, "clamped_swish": 5, "relu_sq": 6, "tanh": 7}
 
 
 def _act_torch(z: torch.Tensor, kind: str) -> torch.Tensor:
@@ -232,6 +289,10 @@ def _act_torch(z: torch.Tensor, kind: str) -> torch.Tensor:
         return _silu(z)
     if kind == "relu":
         return torch.relu(z)
+    if kind == "relu_sq":
+        return torch.relu(z) ** 2
+    if kind == "tanh":
+        return torch.tanh(z)
     raise ValueError(kind)
 
 
@@ -244,7 +305,7 @@ def _clamped_unit(g: torch.Tensor, u: torch.Tensor, limit: float) -> torch.Tenso
 
 
 def activation(x: torch.Tensor, kind: str, a: float = 0.0, b: float = 0.0) -> torch.Tensor:
-    """Elementwise on [T, f] rows, evaluated in fp32: ``gelu`` (erf form), ``gelu_tanh``, ``silu``, or
+    """Elementwise on [T, f] rows, evaluated in fp32: ``gelu`` (erf form), ``gelu_tanh``, ``silu``, ``relu_sq``, ``tanh``, or
     ``xielu`` with the two positive constants ``a``, ``b``:  z > 0: a z^2 + z / 2;  z <= 0:
     b (exp(z) - 1 - z) + z / 2."""
     if not x.is_cuda:
@@ -384,13 +445,15 @@ def rotary_cache(qkv: torch.Tensor, Hq: int, Hkv: int, dk: int, dv: int, positio
 
 
 def _attend(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, scale: float, sink: bool,
-            sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+            sinks: Optional[torch.Tensor] = None, cap: float = 0.0) -> torch.Tensor:
     """q [H, dk], k [n, G, dk], v [n, G, dv] (fp32) -> [H, dv].  ``sinks`` [H]: the sink's logit per
     head (absent: 0)."""
     H, G = q.shape[0], k.shape[1]
     kk = k.repeat_interleave(H // G, dim=1)
     vv = v.repeat_interleave(H // G, dim=1)
     s = torch.einsum("hd,nhd->hn", q, kk) * scale
+    if cap > 0:
+        s = cap * torch.tanh(s / cap)
     m = s.max(-1, keepdim=True).values
     z = sinks.float().view(H, 1) if sinks is not None else torch.zeros(H, 1)
     if sink:
@@ -400,13 +463,23 @@ def _attend(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, scale: float, sin
     return torch.einsum("hn,nhd->hd", e / den, vv)
 
 
+def _first_key(p: int, window: int, chunked: bool) -> int:
+    """The first position that a row at position ``p`` sees."""
+    if window <= 0:
+        return 0
+    return p - p % window if chunked else max(0, p - window + 1)
+
+
 def window_attention_prefill(qkv: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, cu: torch.Tensor,
                              ctx: torch.Tensor, block_tables: torch.Tensor, Hq: int, Hkv: int, dk: int, dv: int,
                              scale: float, window: int, sink: bool, mfma: int = 1,
-                             sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                             sinks: Optional[torch.Tensor] = None, chunked: bool = False,
+                             cap: float = 0.0) -> torch.Tensor:
     """Attention of the step's prompt chunks over the paged cache (which already holds their own
     keys): row r of segment s at position p = ctx[s] + r sees positions max(0, p - window + 1) .. p
-    (``window`` 0: all of 0 .. p).  ``sink``: the softmax denominator has one more term that carries
+    (``window`` 0: all of 0 .. p), or with ``chunked`` those of its own chunk of ``window`` positions,
+    p - p % window .. p (chunks count from position 0).  ``cap`` > 0: a score s (after ``scale``) becomes
+    ``cap * tanh(s / cap)``.  ``sink``: the softmax denominator has one more term that carries
     no value - exp(0), or exp(sinks[h]) for head h where ``sinks`` [Hq] fp32 is given (a learned,
     unscaled logit).  Scores and weights are fp32.  Returns [T, Hq*dv].  GPU, bf16, head sizes
     64 / 128: the matrix-core kernel, 16 query rows per wave or 32 in large steps (``mfma`` 0: the
@@ -423,22 +496,24 @@ def window_attention_prefill(qkv: torch.Tensor, k_cache: torch.Tensor, v_cache: 
             vs = v_cache[bt].permute(0, 3, 1, 2).reshape(-1, Hkv, dv)[:n_all].float()
             for r in range(cul[s], cul[s + 1]):
                 p = ctxl[s] + r - cul[s]
-                lo = max(0, p - window + 1) if window > 0 else 0
-                o = _attend(qkv[r, : Hq * dk].float().view(Hq, dk), ks[lo:p + 1], vs[lo:p + 1], scale, sink, sinks)
+                lo = _first_key(p, window, chunked)
+                o = _attend(qkv[r, : Hq * dk].float().view(Hq, dk), ks[lo:p + 1], vs[lo:p + 1], scale, sink, sinks, cap)
                 out[r] = o.reshape(-1).to(qkv.dtype)
         return out
     out = torch.empty(T, Hq * dv, dtype=qkv.dtype, device=qkv.device)
     native().window_attention_prefill(out, qkv, k_cache, v_cache, cu, ctx, block_tables, Hq, Hkv, dk, dv, float(scale),
-                                      int(window), bool(sink), sinks, int(mfma))
+                                      int(window), bool(sink), sinks, int(mfma), bool(chunked), float(cap))
     return out
 
 
 def window_attention_decode(qkv: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                             block_tables: torch.Tensor, seq_lens: torch.Tensor, Hq: int, Hkv: int, dk: int, dv: int,
                             scale: float, window: int, sink: bool, vec: bool = True,
-                            sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                            sinks: Optional[torch.Tensor] = None, chunked: bool = False,
+                            cap: float = 0.0) -> torch.Tensor:
     """One query per sequence (its newest token, already in the cache) over the last ``window``
-    cached positions; ``seq_lens`` count that token (0: a padding row, output zero)."""
+    cached positions (``chunked``: those of its own chunk; ``cap``: as in window_attention_prefill);
+    ``seq_lens`` count that token (0: a padding row, output zero)."""
     B = qkv.shape[0]
     if not qkv.is_cuda:
         out = torch.zeros(B, Hq * dv, dtype=qkv.dtype)
@@ -446,16 +521,16 @@ def window_attention_decode(qkv: torch.Tensor, k_cache: torch.Tensor, v_cache: t
         for b, n in enumerate(seq_lens.tolist()):
             if n <= 0:
                 continue
-            lo = max(0, n - window) if window > 0 else 0
+            lo = _first_key(n - 1, window, chunked)
             bt = block_tables[b, : (n + bs - 1) // bs].long()
             ks = k_cache[bt].reshape(-1, Hkv, dk)[lo:n].float()
             vs = v_cache[bt].permute(0, 3, 1, 2).reshape(-1, Hkv, dv)[lo:n].float()
             out[b] = _attend(qkv[b, : Hq * dk].float().view(Hq, dk), ks, vs, scale, sink,
-                             sinks).reshape(-1).to(qkv.dtype)
+                             sinks, cap).reshape(-1).to(qkv.dtype)
         return out
     out = torch.empty(B, Hq * dv, dtype=qkv.dtype, device=qkv.device)
     native().window_attention_decode(out, qkv, k_cache, v_cache, block_tables, seq_lens, Hq, Hkv, dk, dv, float(scale),
-                                     int(window), bool(sink), sinks, bool(vec))
+                                     int(window), bool(sink), sinks, bool(vec), bool(chunked), float(cap))
     return out
 
 
@@ -711,20 +786,26 @@ def linear_attention(vkq: torch.Tensor, decay: torch.Tensor, state: torch.Tensor
 def decay_scan(qkv: torch.Tensor, q_col: int, k_col: int, v_col: int, z: torch.Tensor, z_bias: torch.Tensor,
                state: torch.Tensor, seg_cu: torch.Tensor, seg_ctx: torch.Tensor, seg_slot: torch.Tensor, H: int, Gk: int,
                dk: int, dv: int, q_scale: float, a_log: Optional[torch.Tensor] = None, tau: float = 1.0,
-               beta: Optional[torch.Tensor] = None, beta_col: int = 0, unit: bool = False, mode: int = 0) -> torch.Tensor:
-    """Linear attention with a decay per head and key channel, optionally with the delta rule, as an
-    fp32 recurrence over each segment.  Per head h (reading query / key head ``h // (H / Gk)``) and token:
+               beta: Optional[torch.Tensor] = None, beta_col: int = 0, unit: bool = False, mode: int = 0, z_col: int = 0,
+               decay: Optional[str] = None, bonus: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Linear attention with a decay per head and key channel (or per head), optionally with the delta rule
+    or a bonus for the current token, as an fp32 recurrence over each segment.  Per head h (reading query / key head ``h // (H / Gk)``) and token:
 
         S <- diag(g_t) S                       g_t [dk]: this token's decays
         delta rule:   u = beta_t (v_t - S^T k_t);   S <- S + k_t u^T
         otherwise:                                  S <- S + k_t v_t^T
         o_t = S^T q_t
 
+    or with ``bonus`` [H, dk] fp32 (the read-out sees the state before this token's decay and write):
+
+        o_t = (S + diag(bonus) k_t v_t^T)^T q_t;   S <- diag(g_t) S + k_t v_t^T
+
     ``qkv`` [T, *] holds q, k ([Gk*dk] each) and v ([H*dv]) from columns ``q_col``, ``k_col``, ``v_col``
     on; q is multiplied by ``q_scale``.  ``unit``: q and k heads are first made unit vectors,
     ``x / sqrt(sum(x^2) + 1e-6)``.  The decays come from ``z`` [T, H*dk] (a projection, activation dtype)
-    and ``z_bias`` [H*dk] fp32:  ``a_log`` [H] given: ``g = exp(-exp(a_log[h]) softplus(z + z_bias))``;
-    else ``g = sigmoid(z + z_bias)^(1 / tau)``.  ``beta`` [T, *] (given = the delta rule): column
+    (columns from ``z_col`` on) and ``z_bias`` [H*dk] fp32 - or [H]: one decay per head (delta rule) -:
+    ``a_log`` [H] given: ``g = exp(-exp(a_log[h]) softplus(z + z_bias))``; ``decay`` "exp_exp":
+    ``g = exp(-exp(z + z_bias))``; else ``g = sigmoid(z + z_bias)^(1 / tau)``.  ``beta`` [T, *] (given = the delta rule): column
     ``beta_col + h`` holds head h's logit, ``beta_t = sigmoid(logit)``.  ``state`` [slots, H, dv, dk] fp32
     (a value row's key channels contiguous) is read at a segment's start (zero where seg_ctx is 0) and
     written back at its end.  Returns o [T, H*dv] fp32.  Decays, unit norms, gates, state, products and
@@ -735,6 +816,8 @@ def decay_scan(qkv: torch.Tensor, q_col: int, k_col: int, v_col: int, z: torch.T
     workspace, then the recurrence over it; decode steps run as one launch.  ``mode`` 1 / 2 force the
     one-launch / two-launch form (tests)."""
     T = qkv.shape[0]
+    nz = z_bias.numel()
+    dkind = 0 if a_log is not None else 2 if decay == "exp_exp" else 1
     if not qkv.is_cuda:
         o = torch.zeros(T, H * dv, dtype=torch.float32)
         rep = H // Gk
@@ -752,14 +835,21 @@ def decay_scan(qkv: torch.Tensor, q_col: int, k_col: int, v_col: int, z: torch.T
                 k = k * torch.rsqrt(k.pow(2).sum(-1, keepdim=True) + 1e-6)
             q = (q * q_scale).repeat_interleave(rep, dim=1)
             k = k.repeat_interleave(rep, dim=1)
-            zz = (z[a:b].float() + z_bias.float()).view(n, H, dk)
-            if a_log is not None:
+            zz = (z[a:b, z_col:z_col + nz].float() + z_bias.float()).view(n, H, nz // H)
+            if dkind == 2:
+                g = torch.exp(-torch.exp(zz))
+            elif a_log is not None:
                 g = torch.exp(-torch.exp(a_log.float()).view(1, H, 1) * F.softplus(zz, threshold=30.0))
             else:
                 g = torch.exp(F.logsigmoid(zz) / tau)
             bt = torch.sigmoid(beta[a:b, beta_col:beta_col + H].float()) if beta is not None else None
             S = state[slot].clone() if c0 > 0 else torch.zeros_like(state[slot])  # [H, dv, dk]
             for t in range(n):
+                if bonus is not None:
+                    kq = (k[t] * q[t] * bonus.float().view(H, dk)).sum(-1, keepdim=True)
+                    o[a + t] = (torch.einsum("hpn,hn->hp", S, q[t]) + v[t] * kq).reshape(-1)
+                    S = S * g[t, :, None, :] + v[t][:, :, None] * k[t, :, None, :]
+                    continue
                 S = S * g[t, :, None, :]
                 if bt is not None:
                     u = bt[t, :, None] * (v[t] - torch.einsum("hpn,hn->hp", S, k[t]))
@@ -774,8 +864,48 @@ def decay_scan(qkv: torch.Tensor, q_col: int, k_col: int, v_col: int, z: torch.T
     if mode == 2 or (mode == 0 and T >= 32 * seg_slot.numel()):
         ws = torch.empty(T * (2 * Gk * dk + H * dk + Gk + H), dtype=torch.float32, device=qkv.device)
     native().decay_scan(o, qkv, int(q_col), int(k_col), int(v_col), z, z_bias, a_log, float(tau), beta, int(beta_col),
-                        state, seg_cu, seg_ctx, seg_slot, int(H), int(Gk), int(dk), int(dv), float(q_scale), bool(unit), ws)
+                        state, seg_cu, seg_ctx, seg_slot, int(H), int(Gk), int(dk), int(dv), float(q_scale), bool(unit), ws, int(z_col), dkind,
+                        bonus)
     return o
+
+
+def selective_scan(xc: torch.Tensor, q: torch.Tensor, b_col: int, c_col: int, dt: torch.Tensor, dt_bias: torch.Tensor,
+                   a_log: torch.Tensor, d_skip: torch.Tensor, proj: torch.Tensor, z_col: int, state: torch.Tensor,
+                   seg_cu: torch.Tensor, seg_ctx: torch.Tensor, seg_slot: torch.Tensor) -> torch.Tensor:
+    """The selective state-space recurrence with a decay per channel and state, fp32, token by token within
+    each segment, and its output gate.  Per channel c and state n:
+
+        d = softplus(dt[t, c] + dt_bias[c]);   S[c, n] <- exp(-exp(a_log[c, n]) d) S[c, n] + d x_c B_n
+        y_c = sum_n S[c, n] C_n + d_skip[c] x_c;   out = y_c silu(proj[t, z_col + c])
+
+    ``xc`` [T, C] (contiguous), ``dt`` [T, C] (a projection), B and C: columns ``b_col`` / ``c_col`` .. of ``q``
+    (N each); ``state`` [slots, C, N] fp32 is read at the segment's start (zero where seg_ctx is 0) and
+    written back at its end.  Returns out [T, C] in the activation dtype."""
+    T, C = xc.shape
+    N = a_log.shape[1]
+    if not xc.is_cuda:
+        out = torch.zeros(T, C, dtype=xc.dtype)
+        A = -torch.exp(a_log.float())
+        cul = seg_cu.tolist()
+        for s, (c0, slot) in enumerate(zip(seg_ctx.tolist(), seg_slot.tolist())):
+            a, b = cul[s], cul[s + 1]
+            if slot < 0 or b <= a:
+                continue
+            S = state[slot].clone() if c0 > 0 else torch.zeros_like(state[slot])
+            d = F.softplus(dt[a:b].float() + dt_bias.float(), threshold=30.0)
+            x = xc[a:b].float()
+            y = d_skip.float() * x
+            B, Cc = q[a:b, b_col:b_col + N].float(), q[a:b, c_col:c_col + N].float()
+            for t in range(b - a):
+                S = torch.exp(d[t, :, None] * A) * S + (d[t] * x[t])[:, None] * B[t]
+                y[t] += S @ Cc[t]
+            state[slot] = S
+            out[a:b] = (y * _silu(proj[a:b, z_col:z_col + C].float())).to(xc.dtype)
+        return out
+    out = torch.empty(T, C, dtype=xc.dtype, device=xc.device)
+    native().selective_scan(out, xc, q, int(b_col), int(c_col), dt, dt_bias, a_log, d_skip, proj, int(z_col), state, seg_cu,
+                            seg_ctx, seg_slot)
+    return out
 
 
 def gated_group_norm(y: torch.Tensor, proj: torch.Tensor, z_col: int, w: torch.Tensor, eps: float, groups: int,

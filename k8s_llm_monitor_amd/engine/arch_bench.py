@@ -8,7 +8,9 @@ attention and Mamba-2 layers with the same heads, head sizes, recurrent state si
 width (one expert, so every token takes it); Levovik (softmax attention beside gated linear attention
 or the gated delta rule in every layer, routed clamped experts) beside a Dunesun model that has one
 attention layer with the same experts and one Mamba-2 layer of equal state size for every Levovik
-layer.  Both models run through the same
+layer; Dopivik (selective scan, wkv, and attention beside the delta rule, in turn, norms on both sides of
+every sublayer) beside a Dunesun model with a Mamba-2 layer of equal state size for every recurrence and
+an attention layer with the same heads and window size for every attention.  Both models run through the same
 ModelRunner step functions the engine uses: one prefill step of ``seqs`` whole prompts, then decode
 steps of ``batch`` sequences (hipGraph replay where the model's decode is captured)."""
 from __future__ import annotations
@@ -169,7 +171,49 @@ def _levovik_pair(size: str, window: int) -> tuple:
     return new, ref
 
 
-PAIRS = {"dunesun": _pair, "kisutar": _kisutar_pair, "bitonex": _bitonex_pair, "levovik": _levovik_pair}
+# Dopivik: (name, width, heads, kv heads, head dim, rotating dims, chunk, delta heads, delta dim, wkv dim, scan state,
+#           ff, reference ff (three matrices instead of two), layers)
+DOPIVIK_SIZES = {
+    "s": ("d1024", 1024, 8, 2, 128, 64, 1024, 8, 128, 64, 16, 4096, 2816, 6),
+    "m": ("d2048", 2048, 16, 4, 128, 64, 1024, 16, 128, 64, 16, 8192, 5632, 6),
+    "l": ("d4096", 4096, 32, 8, 128, 64, 1024, 32, 128, 64, 16, 16384, 11008, 3),
+}
+
+
+def _dopivik_pair(size: str, window: int) -> tuple:
+    """Dopivik (layers: selective scan, wkv, attention beside the delta rule, in turn) and a Dunesun model in
+    which every recurrence is a Mamba-2 layer with as many state entries per token and every attention
+    an attention layer with the same heads and a window of the chunk's size; one expert per feed-forward,
+    with as many weights."""
+    name, d, H, G, D, rd, chunk, Hr, dr, dw, N, ff, ff_ref, L = DOPIVIK_SIZES[size]
+    flat = lambda m: tuple(sorted(m.items()))
+
+    def layer(i):
+        if i % 3 == 0:
+            return LayerSpec("mamba1", flat({"inner": 2 * d, "state": N, "conv": 4, "dt_rank": d // 16}), DenseSpec(ff))
+        if i % 3 == 1:
+            return LayerSpec("wkv", flat({"heads": d // dw, "dim": dw, "w_rank": d // 32}), DenseSpec(ff))
+        m = {"left." + k: v for k, v in {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "softcap": 50.0,
+                                         "mask.size": chunk, "rot.dims": rd, "rot.base": 5e5}.items()}
+        m.update({"right." + k: v for k, v in {"heads": Hr, "kv_heads": max(1, Hr // 2), "dim": dr, "vdim": dr, "conv": 4}.items()})
+        return LayerSpec("parallel", flat(m), DenseSpec(ff))
+
+    new = HybridConfig(name=f"dopivik-{name}", arch="dopivik", vocab_size=32000, d_model=d,
+                       layers=tuple(layer(i) for i in range(L)), max_position=8192, norm_eps=1e-5, embed_scale=float(d) ** 0.5)
+    one = MoESpec(1, 1, ff_ref, 0)
+    ssm = lambda inner, state, mlp: LayerSpec("mamba2", flat({"heads": inner // 64, "vdim": 64, "state": state, "groups": 1,
+                                                              "conv": 4, "norm_groups": 1}), mlp)
+    att = LayerSpec("attention", flat({"heads": H, "kv_heads": G, "dim": D, "vdim": D, "mask.size": chunk, "scale": D ** -0.5}), one)
+    ref_layers = []
+    for i in range(L):
+        ref_layers += [[ssm(2 * d, N, one)], [ssm(d, dw, one)], [att, ssm(Hr * dr, dr, None)]][i % 3]
+    ref = HybridConfig(name=f"dunesun-scans-{name}", arch="dunesun", vocab_size=32000, d_model=d, layers=tuple(ref_layers),
+                       max_position=8192)
+    return new, ref
+
+
+PAIRS = {"dunesun": _pair, "kisutar": _kisutar_pair, "bitonex": _bitonex_pair, "levovik": _levovik_pair,
+         "dopivik": _dopivik_pair}
 
 
 def _measure(cfg, seqs: int, prompt: int, batch: int, steps: int, warmup: int, graphs: bool) -> dict:

@@ -63,16 +63,26 @@ __device__ __forceinline__ float scan_token(float (&S)[8], const float* __restri
   const float4 q0 = *reinterpret_cast<const float4*>(qp), q1 = *reinterpret_cast<const float4*>(qp + 4);
   const float kv[8] = {k0.x, k0.y, k0.z, k0.w, k1.x, k1.y, k1.z, k1.w};
   const float qv[8] = {q0.x, q0.y, q0.z, q0.w, q1.x, q1.y, q1.z, q1.w};
-  float pk = 0.f, pq = 0.f;
+  float pk0 = 0.f, pk1 = 0.f, pq0 = 0.f, pq1 = 0.f;  // two accumulators per sum: half the dependent adds
 #pragma unroll
-  for (int i = 0; i < 8; ++i) {
-    if (MODE == kBonus) pq += S[i] * qv[i];
+  for (int i = 0; i < 8; i += 2) {
+    if (MODE == kBonus) {
+      pq0 += S[i] * qv[i];
+      pq1 += S[i + 1] * qv[i + 1];
+    }
     S[i] *= gv[i];
-    if (MODE == kDelta) pk += S[i] * kv[i];
-    if (MODE != kBonus) pq += S[i] * qv[i];
+    S[i + 1] *= gv[i + 1];
+    if (MODE == kDelta) {
+      pk0 += S[i] * kv[i];
+      pk1 += S[i + 1] * kv[i + 1];
+    }
+    if (MODE != kBonus) {
+      pq0 += S[i] * qv[i];
+      pq1 += S[i + 1] * qv[i + 1];
+    }
   }
-  if (MODE == kDelta) pk = lanes_sum<CH>(pk);
-  pq = lanes_sum<CH>(pq);
+  const float pk = MODE == kDelta ? lanes_sum<CH>(pk0 + pk1) : 0.f;
+  const float pq = lanes_sum<CH>(pq0 + pq1);
   const float u = MODE == kDelta ? bt * (v - pk) : v;
 #pragma unroll
   for (int i = 0; i < 8; ++i) S[i] += kv[i] * u;
@@ -307,48 +317,47 @@ __global__ __launch_bounds__(256) void decay_scan_staged_kernel(float* __restric
   }
   const int boff = n0 + (n0 >> 6) * 4;
   const bool vec4 = (dk & 3) == 0;
-  // the next tile's inputs, in registers while this tile's tokens are processed
+  // the next tile's inputs, in registers while this tile's tokens are processed.  Loads are not predicated (a
+  // branch around a load would wait for it there): a token past the segment reads its last row, channels
+  // past dk the row's last ones, and what they must not contribute is dropped when it is staged
   float4 rq[NB], rk[NB], rg[HD ? 1 : NB];
-  float rv[NV], rs = 0.f;
+  T rv[NV];
+  float rs;
+  const int gp_col = min((int)blockIdx.z * PB + (int)(threadIdx.x % PB), dv - 1);  // 256 % PB == 0: one column per thread
   auto fetch = [&](int tb) {
-    const int nt = min(TB, t1 - tb);
 #pragma unroll
     for (int u = 0; u < NB; ++u) {
       const int i = threadIdx.x + 256 * u;
-      const int tt = i / Q4, n = (i % Q4) * 4;
-      rq[u] = rk[u] = make_float4(0.f, 0.f, 0.f, 0.f);
-      if (!HD) rg[u] = make_float4(0.f, 0.f, 0.f, 0.f);
-      if (tt < nt && n < dk) {
-        const float* qp = qn + ((long)(tb + tt) * Gk + g) * dk + n;
-        const float* kp = kn + ((long)(tb + tt) * Gk + g) * dk + n;
-        const float* gp = HD ? nullptr : gd + ((long)(tb + tt) * H + h) * dk + n;
-        if (vec4) {
-          rq[u] = *reinterpret_cast<const float4*>(qp);
-          rk[u] = *reinterpret_cast<const float4*>(kp);
-          if (!HD) rg[u] = *reinterpret_cast<const float4*>(gp);
-        } else {
-          rq[u].x = qp[0]; rk[u].x = kp[0];
-          if (n + 1 < dk) { rq[u].y = qp[1]; rk[u].y = kp[1]; }
-          if (n + 2 < dk) { rq[u].z = qp[2]; rk[u].z = kp[2]; }
-          if (n + 3 < dk) { rq[u].w = qp[3]; rk[u].w = kp[3]; }
-          if (!HD) {
-            rg[u].x = gp[0];
-            if (n + 1 < dk) rg[u].y = gp[1];
-            if (n + 2 < dk) rg[u].z = gp[2];
-            if (n + 3 < dk) rg[u].w = gp[3];
-          }
-        }
+      const long t = min(tb + i / Q4, t1 - 1);
+      const int n = (i % Q4) * 4;
+      const float* qp = qn + (t * Gk + g) * dk;
+      const float* kp = kn + (t * Gk + g) * dk;
+      const float* gp = HD ? nullptr : gd + (t * H + h) * dk;
+      if (vec4) {
+        const int m = min(n, dk - 4);
+        rq[u] = *reinterpret_cast<const float4*>(qp + m);
+        rk[u] = *reinterpret_cast<const float4*>(kp + m);
+        if (!HD) rg[u] = *reinterpret_cast<const float4*>(gp + m);
+      } else {
+        const int m0 = min(n, dk - 1), m1 = min(n + 1, dk - 1), m2 = min(n + 2, dk - 1), m3 = min(n + 3, dk - 1);
+        rq[u] = make_float4(qp[m0], qp[m1], qp[m2], qp[m3]);
+        rk[u] = make_float4(kp[m0], kp[m1], kp[m2], kp[m3]);
+        if (!HD) rg[u] = make_float4(gp[m0], gp[m1], gp[m2], gp[m3]);
       }
     }
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
-      const int i = threadIdx.x + 256 * u;
-      const int tt = i / PB, pg = blockIdx.z * PB + i % PB;
-      rv[u] = (tt < nt && pg < dv) ? ldf(qkv + (long)(tb + tt) * stride + v_col + (long)h * dv + pg) : 0.f;
+      const long t = min(tb + (int)(threadIdx.x + 256 * u) / PB, t1 - 1);
+      rv[u] = qkv[t * stride + v_col + (long)h * dv + gp_col];
     }
-    if (threadIdx.x < nt) rs = kq[(long)(tb + threadIdx.x) * Gk + g];
-    else if (MODE == kDelta && threadIdx.x >= TB && threadIdx.x - TB < nt) rs = bt[(long)(tb + threadIdx.x - TB) * H + h];
-    else if (HD && threadIdx.x >= 2 * TB && threadIdx.x - 2 * TB < nt) rs = gd[(long)(tb + threadIdx.x - 2 * TB) * H + h];
+    {  // threads 0 .. 15: k . q; the next 16: beta; the next 16: the head's decay
+      const long t = min(tb + (int)(threadIdx.x % TB), t1 - 1);
+      const int w = threadIdx.x / TB;
+      const float* src = kq + t * Gk + g;
+      if (MODE == kDelta && w == 1) src = bt + t * H + h;
+      if (HD && w == 2) src = gd + t * H + h;
+      rs = *src;
+    }
   };
   fetch(t0);
   float* op = o + (long)t0 * inner + (long)h * dv + p;  // this lane's output column, advanced per tile
@@ -361,26 +370,49 @@ __global__ __launch_bounds__(256) void decay_scan_staged_kernel(float* __restric
       const int tt = i / Q4, n = (i % Q4) * 4;
       if (tt < TB) {
         const int off = tt * ROW + n + (n >> 6) * 4;
-        *reinterpret_cast<float4*>(&qs[0][0] + off) = rq[u];
-        *reinterpret_cast<float4*>(&ks[0][0] + off) = rk[u];
+        float4 q4 = rq[u], k4 = rk[u];
+        if (n + 4 > dk) {  // channels beyond dk: zero keys and queries leave the state and the sums alone
+          if (n >= dk) q4.x = k4.x = 0.f;
+          if (n + 1 >= dk) q4.y = k4.y = 0.f;
+          if (n + 2 >= dk) q4.z = k4.z = 0.f;
+          q4.w = k4.w = 0.f;
+        }
+        *reinterpret_cast<float4*>(&qs[0][0] + off) = q4;
+        *reinterpret_cast<float4*>(&ks[0][0] + off) = k4;
         if (!HD) *reinterpret_cast<float4*>(&gs[0][0] + off) = rg[u];
       }
     }
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
       const int i = threadIdx.x + 256 * u;
-      if (i < TB * PB) (&vs[0][0])[i] = rv[u];
+      if (i < TB * PB) (&vs[0][0])[i] = ldf(&rv[u]);
     }
     if (threadIdx.x < TB) kqs[threadIdx.x] = rs;
     else if (MODE == kDelta && threadIdx.x < 2 * TB) bts[threadIdx.x - TB] = rs;
     else if (HD && threadIdx.x >= 2 * TB && threadIdx.x < 3 * TB) ghs[threadIdx.x - 2 * TB] = rs;
     __syncthreads();
     if (tb + TB < t1) fetch(tb + TB);
-#pragma unroll 2
-    for (int tt = 0; tt < nt; ++tt) {
-      const float r = scan_token<CH, MODE, HD>(S, &gs[HD ? 0 : tt][HD ? 0 : boff], HD ? ghs[tt] : 0.f, &ks[tt][boff],
-                                               &qs[tt][boff], vs[tt][pl], MODE == kDelta ? bts[tt] : 0.f, kqs[tt]);
-      if (live && chunk == 0) op[(long)tt * inner] = r;
+    auto token = [&](int tt) -> float {
+      return scan_token<CH, MODE, HD>(S, &gs[HD ? 0 : tt][HD ? 0 : boff], HD ? ghs[tt] : 0.f, &ks[tt][boff], &qs[tt][boff],
+                                      vs[tt][pl], MODE == kDelta ? bts[tt] : 0.f, kqs[tt]);
+    };
+    if (nt == TB) {  // a lane of the column keeps every KB-th read-out: one store for KB tokens
+      constexpr int KB = CH < TB ? CH : TB;
+#pragma unroll
+      for (int tk = 0; tk < TB; tk += KB) {
+        float keep = 0.f;
+#pragma unroll
+        for (int j = 0; j < KB; ++j) {
+          const float r = token(tk + j);
+          keep = chunk == j ? r : keep;
+        }
+        if (live && chunk < KB) op[(long)(tk + chunk) * inner] = keep;
+      }
+    } else {
+      for (int tt = 0; tt < nt; ++tt) {
+        const float r = token(tt);
+        if (live && chunk == 0) op[(long)tt * inner] = r;
+      }
     }
     op += (long)TB * inner;
   }

@@ -11,11 +11,25 @@
 // with NPL of its states (and their exponents' factors) in registers; the read-out's partial sums are DPP adds
 // over those lanes.  16 tokens at a time are staged in LDS: step sizes after softplus, dt x, B, C; the raw
 // values of the next 16 are fetched into registers while the current ones are processed.  The read-outs of
-// a tile meet in LDS, and the whole workgroup adds the skip term, applies the gate and stores rows.
+// a tile meet in LDS (a lane keeps every LPC-th one, so LPC tokens need one LDS write), and the whole
+// workgroup adds the skip term, applies the gate and stores rows.  Loads are not predicated: a token past
+// the segment reads the segment's last row, a channel past the end the last channel, and what they must
+// not contribute is zeroed when it is staged - a branch around a load would wait for it there.
 // One exponential per state and token (v_exp_f32 in base 2, log2 e folded into the factor) is what bounds it.
 #include "hy_common.h"
 
 namespace k8sllm {
+
+// log(1 + exp(x)) to a few units in the last place without the library's branches: max(x, 0) + log1p(e),
+// e = exp(-|x|); log1p by its series below 1/32, by v_log_f32 above
+__device__ __forceinline__ float softplus_fast(float x) {
+  const float a = -fabsf(x), t = a * 1.44269504088896341f;
+  const float lo = fmaf(a, 1.44269504088896341f, -t);  // what rounding the product dropped
+  const float e2 = __builtin_amdgcn_exp2f(t), e = fmaf(e2, lo * 0.693147180559945309f, e2);
+  const float series = e * fmaf(e, fmaf(e, fmaf(e, -0.25f, 0.333333333f), -0.5f), 1.f);
+  const float lg = __builtin_amdgcn_logf(1.f + e) * 0.693147180559945309f;
+  return fmaxf(x, 0.f) + (e < 0.03125f ? series : lg);
+}
 
 template <typename T, int LPC, int NPL>
 __global__ __launch_bounds__(256) void selective_scan_kernel(
@@ -28,7 +42,8 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(
   constexpr int NB = (TB * NS + 255) / 256;   // B / C elements a thread stages
   __shared__ __attribute__((aligned(16))) float Bs[TB][NS];
   __shared__ __attribute__((aligned(16))) float Cs[TB][NS];
-  __shared__ float dts[TB][PB], us[TB][PB], ys[TB][PB];
+  __shared__ float dts[TB][PB], us[TB][PB];
+  __shared__ float ys[TB][PB + 64 / LPC];  // padded: the lanes of a channel write neighbouring rows to different banks
   const int s = blockIdx.x;
   const int sl = slot[s];
   const int t0 = cu[s], t1 = cu[s + 1];
@@ -70,27 +85,38 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(
     }
   }
   const float bias = slive ? dt_bias[cs] : 0.f, D = slive ? d_skip[cs] : 0.f;
-  float rd[NV], rx[NV], rz[NV], rB[NB], rC[NB];
+  T rd[NV], rx[NV], rz[NV], rB[NB], rC[NB];
+  const int cl = min(cs, C - 1);
   auto fetch = [&](int tb) {
-    const int nt = min(TB, t1 - tb);
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
-      const int tt = tt0 + LPC * u;
-      const bool in = slive && tt < nt;
-      const long t = tb + tt;
-      rd[u] = in ? ldf(dt + t * dt_stride + cs) : 0.f;
-      rx[u] = in ? ldf(xc + t * C + cs) : 0.f;
-      rz[u] = in ? ldf(z + t * z_stride + cs) : 0.f;
+      const long t = min(tb + tt0 + LPC * u, t1 - 1);
+      rd[u] = dt[t * dt_stride + cl];
+      rx[u] = xc[t * C + cl];
+      rz[u] = z[t * z_stride + cl];
     }
 #pragma unroll
     for (int u = 0; u < NB; ++u) {
       const int i = threadIdx.x + 256 * u;
-      const int tt = i / NS, n = i % NS;
-      const bool in = tt < nt && n < N;  // states beyond N: zero
-      const T* row = q + (long)(tb + tt) * q_stride + n;
-      rB[u] = in ? ldf(row + b_col) : 0.f;
-      rC[u] = in ? ldf(row + c_col) : 0.f;
+      const T* row = q + (long)min(tb + i / NS, t1 - 1) * q_stride + min(i % NS, N - 1);
+      rB[u] = row[b_col];
+      rC[u] = row[c_col];
     }
+  };
+  auto token = [&](int tt) -> float {  // the recurrence for one staged token; the channel's read-out on all its lanes
+    const float d = dts[tt][pl], u = us[tt][pl];
+    float acc = 0.f;
+#pragma unroll
+    for (int i = 0; i < NPL; i += 4) {
+      const float4 b = *reinterpret_cast<const float4*>(&Bs[tt][n0 + i]);
+      const float4 g = *reinterpret_cast<const float4*>(&Cs[tt][n0 + i]);
+      S[i] = __builtin_amdgcn_exp2f(d * A[i]) * S[i] + u * b.x;
+      S[i + 1] = __builtin_amdgcn_exp2f(d * A[i + 1]) * S[i + 1] + u * b.y;
+      S[i + 2] = __builtin_amdgcn_exp2f(d * A[i + 2]) * S[i + 2] + u * b.z;
+      S[i + 3] = __builtin_amdgcn_exp2f(d * A[i + 3]) * S[i + 3] + u * b.w;
+      acc += S[i] * g.x + S[i + 1] * g.y + S[i + 2] * g.z + S[i + 3] * g.w;
+    }
+    return lanes_sum<LPC>(acc);
   };
   fetch(t0);
   for (int tb = t0; tb < t1; tb += TB) {
@@ -99,38 +125,39 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
       const int tt = tt0 + LPC * u;
-      const float d = softplus_f(rd[u] + bias);
+      const float d = softplus_fast(ldf(&rd[u]) + bias);
+      ex[u] = ldf(&rx[u]);
+      ez[u] = ldf(&rz[u]);
       dts[tt][pc] = d;
-      us[tt][pc] = d * rx[u];
-      ex[u] = rx[u];
-      ez[u] = rz[u];
+      us[tt][pc] = d * ex[u];
     }
 #pragma unroll
     for (int u = 0; u < NB; ++u) {
       const int i = threadIdx.x + 256 * u;
-      if (i < TB * NS) {
-        (&Bs[0][0])[i] = rB[u];
-        (&Cs[0][0])[i] = rC[u];
+      const bool in = i % NS < N;  // states beyond N stay zero
+      if (NB * 256 == TB * NS || i < TB * NS) {
+        (&Bs[0][0])[i] = in ? ldf(&rB[u]) : 0.f;
+        (&Cs[0][0])[i] = in ? ldf(&rC[u]) : 0.f;
       }
     }
     __syncthreads();
     if (tb + TB < t1) fetch(tb + TB);
-#pragma unroll 4
-    for (int tt = 0; tt < nt; ++tt) {
-      const float d = dts[tt][pl], u = us[tt][pl];
-      float acc = 0.f;
+    if (nt == TB) {
 #pragma unroll
-      for (int i = 0; i < NPL; i += 4) {
-        const float4 b = *reinterpret_cast<const float4*>(&Bs[tt][n0 + i]);
-        const float4 g = *reinterpret_cast<const float4*>(&Cs[tt][n0 + i]);
-        S[i] = __builtin_amdgcn_exp2f(d * A[i]) * S[i] + u * b.x;
-        S[i + 1] = __builtin_amdgcn_exp2f(d * A[i + 1]) * S[i + 1] + u * b.y;
-        S[i + 2] = __builtin_amdgcn_exp2f(d * A[i + 2]) * S[i + 2] + u * b.z;
-        S[i + 3] = __builtin_amdgcn_exp2f(d * A[i + 3]) * S[i + 3] + u * b.w;
-        acc += S[i] * g.x + S[i + 1] * g.y + S[i + 2] * g.z + S[i + 3] * g.w;
+      for (int t4 = 0; t4 < TB; t4 += LPC) {
+        float keep = 0.f;
+#pragma unroll
+        for (int j = 0; j < LPC; ++j) {
+          const float acc = token(t4 + j);
+          keep = chunk == j ? acc : keep;
+        }
+        ys[t4 + chunk][pl] = keep;
       }
-      acc = lanes_sum<LPC>(acc);
-      if (chunk == 0) ys[tt][pl] = acc;
+    } else {
+      for (int tt = 0; tt < nt; ++tt) {
+        const float acc = token(tt);
+        if (chunk == 0) ys[tt][pl] = acc;
+      }
     }
     __syncthreads();  // the tile's inputs are consumed and its read-outs complete
 #pragma unroll

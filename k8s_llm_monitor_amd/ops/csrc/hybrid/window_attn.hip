@@ -320,7 +320,12 @@ __global__ __launch_bounds__(64 * NW) void window_decode_vec_kernel(bf16_t* __re
 // With the query on the lane the running maximum, denominator and the rescale of O are lane-local
 // (two xor-shuffles per reduction).  Scores, weights and sums are fp32 (base-2 exponentials: the
 // scale carries log2 e); P is rounded to bf16 for the PV product.
-template <int DK, int DV, int QT, bool CAP>
+// CAP 1: capped scores.  CAP 2: capped scores with a cap up to kMaxCapPlain and no sink: a score lies within
+// +-cap, so exp(score) cannot leave the fp32 (or bf16) range and the softmax is taken as it stands, without a
+// running maximum, rescaling or a cross-lane sum per tile (the lanes' parts of the denominator meet at the
+// end); only tiles at a row's first or last key are masked.
+constexpr float kMaxCapPlain = 60.f;
+template <int DK, int DV, int QT, int CAP>
 __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
     bf16_t* __restrict__ out, const bf16_t* __restrict__ qkv, long q_stride, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int* __restrict__ cu, const int* __restrict__ ctx,
@@ -363,6 +368,8 @@ __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
     m[t] = sink ? (sinks != nullptr ? sinks[blockIdx.y] * 1.44269504088896341f : 0.f) : -INFINITY;
     l[t] = sink ? 1.f : 0.f;
   }
+  const int lo_max = first_key(p0 + nq - 1, window, chunked);  // from here to p0: keys that every row of the tile sees
+  const float k1 = CAP ? icap * 2.88539008177792681f : 0.f;
   const int lo_t = first_key(p0, window, chunked), hi = p0 + nq;
   const long krs = (long)G * DK, vrs = (long)G * DV;
   // Register double buffer: while tile j0 is computed, the K and V^T fragments of tile j0 + 16 are
@@ -400,11 +407,29 @@ __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
     s16x4 pb[QT];
     float alpha[QT];
     bool rescale[QT];
+    const bool inner = j0 >= lo_max && j0 + 15 <= p0;
 #pragma unroll
     for (int t = 0; t < QT; ++t) {
       f32x4 sacc = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int ks = 0; ks < DK / 32; ++ks) sacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks], qf[t][ks], sacc, 0, 0, 0);
+      if constexpr (CAP == 2) {
+        float pv[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i)  // exp(cap tanh(s / cap)) in base 2
+          pv[i] = __builtin_amdgcn_exp2f(cap2 - 2.f * cap2 * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(sacc[i] * k1)));
+        if (!inner) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int j = j0 + 4 * quad + i;
+            if (j < my_lo[t] || j > my_p[t]) pv[i] = 0.f;
+          }
+        }
+        l[t] += (pv[0] + pv[1]) + (pv[2] + pv[3]);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) pb[t][i] = (short)f2bf(pv[i]);
+        continue;
+      }
       float sv[4], tmax = -INFINITY;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {  // sacc[i]: key j0 + 4 quad + i, query 16 t + c16
@@ -432,7 +457,7 @@ __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
     // the compiler into multiplies on every tile
 #pragma unroll
     for (int t = 0; t < QT; ++t)
-      if (rescale[t]) {
+      if (CAP != 2 && rescale[t]) {
 #pragma unroll
         for (int dt = 0; dt < DV / 16; ++dt)
 #pragma unroll
@@ -447,6 +472,7 @@ __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
   }
 #pragma unroll
   for (int t = 0; t < QT; ++t) {
+    if (CAP == 2) l[t] = xor32_sum_f(xor16_sum(l[t]));
     if (!q_live[t]) continue;  // oacc[t][dt][i] = O[q = 16 t + c16][d = 16 dt + 4 quad + i]
     const float inv = l[t] > 0.f ? 1.f / l[t] : 0.f;
     bf16_t* orow = out + (long)(row0 + 16 * t + c16) * Hq * DV + (long)h * DV;
@@ -495,7 +521,9 @@ int k8sllm_hy_window_prefill(void* out, const void* qkv, long q_stride, const vo
                      (const bf16_t*)qkv, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, cu, ctx,             \
                      block_tables, bt_stride, S, Hq, G, scale, window, chunked, cap, sink, sinks)
 #define K8SLLM_WP(DK, DV, QT) \
-  if (cap > 0.f) K8SLLM_WPC(DK, DV, QT, true); else K8SLLM_WPC(DK, DV, QT, false)
+  if (cap > 0.f && cap <= kMaxCapPlain && !sink) K8SLLM_WPC(DK, DV, QT, 2); \
+  else if (cap > 0.f) K8SLLM_WPC(DK, DV, QT, 1); \
+  else K8SLLM_WPC(DK, DV, QT, 0)
 #define K8SLLM_WPQ(DK, DV)                                       \
   if (qrows == 64) { K8SLLM_WP(DK, DV, 4); }                     \
   else if (qrows == 32) { K8SLLM_WP(DK, DV, 2); }                \

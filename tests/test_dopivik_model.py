@@ -850,7 +850,7 @@ def test_gpu_chunked_capped_attention_kernels(Hq, G, dk, dv):
     scale = 2.0 * dk ** -0.5 / 4
     for dtype, tol in ((torch.float32, 2e-5), (torch.bfloat16, 2e-2)):
         x, kd, vd = qkv.cuda().to(dtype), kc.cuda().to(dtype), vc.cuda().to(dtype)
-        for size, cap in ((1, 5.0), (13, 2.0), (16, 1.0), (17, 3.0), (64, 0.5), (90, 30.0), (500, 4.0)):
+        for size, cap in ((1, 5.0), (13, 2.0), (16, 1.0), (17, 3.0), (64, 0.5), (90, 30.0), (500, 4.0), (40, 90.0)):
             want = O.chunked_attention(q, k, v, scale, cap, size)
             kw = dict(chunked=True, cap=cap)
             for a, b in ((0, 90), (5, 7), (15, 64)):

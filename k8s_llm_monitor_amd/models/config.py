@@ -151,7 +151,8 @@ class MoESpec:
     (DESIGN_TRAITS ``ffn``).  Designs whose experts clamp their pre-activations read ``limit``;
     designs whose router chooses within the best of ``groups`` equal groups of neighbouring experts
     read ``groups`` / ``keep_groups`` (1 group: no restriction) and scale the chosen weights by
-    ``route_scale``."""
+    ``route_scale``.  ``identity``: that many more router outputs behind the experts' stand for experts
+    without tensors whose output is the layer's input."""
 
     experts: int
     top: int
@@ -161,6 +162,7 @@ class MoESpec:
     groups: int = 1
     keep_groups: int = 1
     route_scale: float = 1.0
+    identity: int = 0
 
 
 @dataclass(frozen=True)
@@ -213,6 +215,7 @@ class HybridConfig:
     logit_softcap: float = 0.0  # > 0: logits <- cap * tanh(logits / cap)
     embed_scale: float = 1.0  # the token embedding is multiplied by this
     side_dim: int = 0  # > 0: every layer also reads its own slice of a second token table (``side.embed``)
+    streams: int = 0  # > 0: that many residual streams, read and written with learned weights (``hc1``, ``hc2``)
     loop: Optional[tuple] = None  # (start, stop, times): layers start .. stop-1 run `times` times
     bos_id: int = 1
     eos_ids: tuple = (2,)
@@ -275,17 +278,22 @@ class HybridConfig:
 #                  used as they are, ungated shared expert, dense layers with xIELU), "gated_gelu"
 #                  (dense layers down(gelu_tanh(gate h) * up h)), "relu_glu_grouped" (dense layers
 #                  down(relu(gate h) * up h), clamped gated experts with a group-limited sigmoid
-#                  router) or "relu_sq" (dense layers down(relu(up h)^2))
+#                  router), "relu_sq" (dense layers down(relu(up h)^2)) or "relu_sq_corrected" (ungated
+#                  squared-ReLU experts and identity experts, softmax over all logits, the choice by
+#                  corrected probabilities within the best groups, an ungated shared expert)
 #   max_position   positions a model accepts when its config.json does not say
 # and, where present (absent = the first value):
 #   scalar_norm    False / True: a block or final norm's weight is one number for all coordinates
 #   gated_residual False / True: every sublayer's result is multiplied elementwise by
 #                  sigmoid(W h + b) of the sublayer's input (``l<i>.rg1`` / ``.rg2`` and ``.b``)
 #   mixers         config ``type`` -> entry of models/hybrid.py MIXERS where the design's mixer of that
-#                  name is not the entry of the same name
+#                  name is not the entry of the same name, or (entry, options)
 #   latent         what the design fixes for latent attention: ``rotary`` "half" (entry i turns with
 #                  i + n/2) / "pairs" (2i with 2i + 1), ``sink`` True (a learned logit per head in the
-#                  softmax denominator) / False
+#                  softmax denominator) / False, ``gate`` None / "head" (every head's output is multiplied
+#                  by sigmoid(G h)[head])
+#   loop_step      True / False: every pass of a looped span starts with a learned vector (``loop.step``)
+#                  added to the stream
 #   norm           "rms" / "layer": block and final norms are RMSNorms, or layer norms with a weight
 #                  and no bias ((x - mean) / sqrt(variance + eps) * w)
 #   norm_bias      False / True: the layer norms also have a bias (the norm's name with ``.b``)
@@ -325,6 +333,10 @@ DESIGN_TRAITS = {
                         "parallel": dict(
                             left=("rotary_attention", dict(rotary="half", mask="chunk", temp=False, gate=True)),
                             right=("gated_delta", dict(decay="head", gate="silu")))}),
+    "zifisun": dict(block="sequential", one_plus_norm=False, learned_pos=False, token_shift=False,
+                    depth_average=False, ffn="relu_sq_corrected", max_position=1 << 17, loop_step=False,
+                    mixers={"attention": ("rotary_attention", dict(rotary="none", qk_norm="before", temp=False, gate="head"))},
+                    latent=dict(rotary="pairs", sink=False, gate="head")),
 }
 
 
@@ -341,9 +353,9 @@ def _flat(d: dict, prefix: str = "") -> list:
 def hybrid_config_from_dict(c: dict, name: Optional[str] = None) -> HybridConfig:
     """A :class:`HybridConfig` from a layer-list ``config.json``: ``architecture``, ``vocab``,
     ``width``, ``max_positions``, ``norm.eps``, ``logit_scale``, ``logit_softcap``, ``residual_mult``,
-    ``embedding.scale``, ``token_side.dim``, ``loop`` {start, stop, times} and
+    ``embedding.scale``, ``token_side.dim``, ``streams``, ``loop`` {start, stop, times} and
     ``layers`` [{type, mixer {...}, mlp {kind: moe, expert.ff, expert.limit, router.experts, router.top,
-    router.scale, router.groups {count, keep}, shared.ff} | {kind: dense, ff} | null, weights_of: layer or
+    router.scale, router.identity, router.groups {count, keep}, shared.ff} | {kind: dense, ff} | null, weights_of: layer or
     absent}].  Nested mixer keys are flattened with dots (``mask.size``)."""
     arch = str(c["architecture"]).lower()
     if arch not in DESIGN_TRAITS:
@@ -361,7 +373,8 @@ def hybrid_config_from_dict(c: dict, name: Optional[str] = None) -> HybridConfig
                 moe = MoESpec(experts=int(rt["experts"]), top=int(rt["top"]),
                               ff=int(ml["expert"]["ff"]), shared_ff=int(sh["ff"]) if sh else 0,
                               limit=float(ml["expert"].get("limit", 0.0)), groups=int(gr.get("count", 1)),
-                              keep_groups=int(gr.get("keep", gr.get("count", 1))), route_scale=float(rt.get("scale", 1.0)))
+                              keep_groups=int(gr.get("keep", gr.get("count", 1))), route_scale=float(rt.get("scale", 1.0)),
+                              identity=int(rt.get("identity") or 0))
             elif kind == "dense":
                 moe = DenseSpec(ff=int(ml["ff"]))
             else:
@@ -381,7 +394,7 @@ def hybrid_config_from_dict(c: dict, name: Optional[str] = None) -> HybridConfig
                         residual_mult=float(c.get("residual_mult", 1.0)),
                         logit_softcap=float(c.get("logit_softcap") or 0.0), loop=loop,
                         embed_scale=float((c.get("embedding") or {}).get("scale", 1.0)),
-                        side_dim=int((c.get("token_side") or {}).get("dim", 0)),
+                        side_dim=int((c.get("token_side") or {}).get("dim", 0)), streams=int(c.get("streams") or 0),
                         bos_id=int(c.get("bos_id", min(1, V - 1))), eos_ids=tuple(c.get("eos_ids", (min(2, V - 1),))))
 
 
@@ -411,6 +424,8 @@ def hybrid_config_to_dict(c: HybridConfig) -> dict:
                 ml["router"]["groups"] = {"count": s.mlp.groups, "keep": s.mlp.keep_groups}
             if s.mlp.route_scale != 1.0:
                 ml["router"]["scale"] = s.mlp.route_scale
+            if s.mlp.identity:
+                ml["router"]["identity"] = s.mlp.identity
         layers.append({"type": s.kind, "mixer": nest(s.mixer), "mlp": ml})
         if s.weights_of is not None:
             layers[-1]["weights_of"] = s.weights_of
@@ -425,6 +440,8 @@ def hybrid_config_to_dict(c: HybridConfig) -> dict:
         d["embedding"] = {"scale": c.embed_scale}
     if c.side_dim:
         d["token_side"] = {"dim": c.side_dim}
+    if c.streams:
+        d["streams"] = c.streams
     if c.loop:
         d["loop"] = {"start": c.loop[0], "stop": c.loop[1], "times": c.loop[2]}
     return d
@@ -548,3 +565,20 @@ DOPIVIK_TINY = _reg(HybridConfig(
     name="dopivik-tiny", arch="dopivik", vocab_size=336, d_model=80,
     layers=_DOPIVIK_LAYERS + tuple(dataclasses.replace(_DOPIVIK_LAYERS[j], weights_of=j) for j in (2, 0, 1)),
     max_position=4096, norm_eps=1e-5, embed_scale=4.0, bos_id=1, eos_ids=(2,)))
+
+
+def _head_attn(heads, kv_heads, dim, vdim, window, keep_first, scale):
+    return LayerSpec("attention", tuple(sorted({"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "mask.size": window,
+                                                "mask.keep_first": keep_first, "scale": scale}.items())))
+
+
+# Small Zifisun-design model for CPU tests and GPU smoke runs (random weights): three residual streams, latent
+# attention and windowed attention that keeps the first tokens, routed layers with identity experts and one
+# layer without a feed-forward, layers 1..2 looped twice.
+ZIFISUN_TINY = _reg(HybridConfig(
+    name="zifisun-tiny", arch="zifisun", vocab_size=368, d_model=88,
+    layers=(_with_mlp(_head_attn(4, 2, 24, 16, 20, 3, 0.25), MoESpec(6, 2, 40, 56, groups=2, keep_groups=1, identity=2)),
+            _with_mlp(_latent(3, 16, 8, 24, 36, 32, 28, 0.2, base=5000.0), MoESpec(5, 3, 24, 0, groups=4, keep_groups=2, identity=3)),
+            _with_mlp(_head_attn(2, 1, 32, 40, 12, 5, 0.2), None),
+            _with_mlp(_latent(2, 24, 16, 16, 40, 24, 17, 0.17, base=20000.0), MoESpec(4, 2, 32, 48))),
+    max_position=4096, norm_eps=1e-6, streams=3, loop=(1, 3, 2), bos_id=1, eos_ids=(2,)))

@@ -3,11 +3,19 @@ sink, the Mamba-1 and Mamba-2 recurrences, latent attention, rotary grouped-quer
 attention with fixed or learned decays, the gated delta rule, wkv time mixing, or two of these side by
 side) and an optional feed-forward; a span of layers may run several times with shared
 weights, and a layer may use another layer's tensors (``weights_of``).  ``Dunesun``, ``Kisutar``,
-``Bitonex``, ``Levovik`` and ``Dopivik`` are the designs served; mixers are registered by
+``Bitonex``, ``Levovik``, ``Dopivik`` and ``Zifisun`` are the designs served; mixers are registered by
 name (``MIXERS``) and feed-forward families by the design's ``ffn`` trait (``_ffn_for``), with their
 sizes and constants read from the layer's spec, so another layer-list design can reuse them in
 another order.  What a design fixes (block form, norm form, positions, token shift, depth average,
 gated residual, rotation layout) is models/config.DESIGN_TRAITS.
+
+Zifisun, per layer (sequential block): the residual is ``streams`` fp32 rows per token.  A sublayer reads
+``norm(sum_s in[s] x_s)`` and its result y is written back as ``x_t <- sum_s mix[s, t] x_s + out[t] y``;
+writing one sublayer's result and reading the next one's input is one launch (ops.hybrid.stream_norm).
+Its mixers: latent attention, and grouped-query attention without positions whose sliding window keeps
+the first tokens visible; both with one sigmoid gate per head.  Routed squared-ReLU experts beside
+identity experts, chosen by corrected probabilities within the best groups.  The model's output is the
+sum of the streams.
 
 Dopivik, per layer (sequential block with norms on both sides of a sublayer): ``x += norm1b(mixer(
 norm1(x)))``, then ``x += norm2b(ff(norm2(x)))``, all layer norms with a bias; the norm behind a sublayer,
@@ -197,6 +205,15 @@ class Mamba2Mixer:
         return F.linear(g, self.wo)
 
 
+def _rows8(ws: list, pad: bool = True) -> torch.Tensor:
+    """A projection's weight rows in one tensor; ``pad``: zero rows up to a multiple of 8 (a per-head gate's
+    few rows would leave the result's rows at strides the kernels' 16-byte accesses cannot take)."""
+    n = sum(w.shape[0] for w in ws)
+    if pad and n % 8:
+        ws = list(ws) + [torch.zeros(-n % 8, ws[0].shape[1], dtype=ws[0].dtype, device=ws[0].device)]
+    return torch.cat(ws).contiguous()
+
+
 def _fresh_pages(meta: AttnMeta, T: int, device) -> tuple:
     """Temporary pages for a step of whole prompts: (slot of every row, block tables [S, W], blocks),
     every segment starting on a page of its own.  Computed once per step (cached on ``meta``), on the
@@ -222,7 +239,9 @@ class LatentAttention:
     rotated key part of ``rot_dim`` per token, shared by all heads), rotary positions on the
     ``rot_dim`` part of queries and keys, a sliding window (``mask.size``; 0 / absent: none) and -
     where the design has one - a learned per-head sink.  The design's ``latent`` trait fixes the
-    rotation layout (``rotary`` "half" / "pairs") and ``sink``.
+    rotation layout (``rotary`` "half" / "pairs"), ``sink`` and ``gate`` (None, or "head": a head's output
+    times sigmoid(G h)[head], its logits more rows of the down-projection, applied in the attention
+    kernels' epilogue - the value expansion behind them is linear per head).
     ``kv_from``: j - no key/value projection of its own; reads layer j's pages.
     ``tail``: extra rows [n, d] for the down-projection; forward leaves their outputs in ``tail_out``
     (a [T, n] view) - the block's residual gate rides in the mixer's first GEMM.
@@ -243,6 +262,7 @@ class LatentAttention:
         lt = (traits or {}).get("latent", {})
         self.pairs = lt.get("rotary", "half") == "pairs"
         self.sink = bool(lt.get("sink", True))
+        self.has_gate = lt.get("gate") == "head"
         self.H, self.dn, self.dr, self.dv = int(m["heads"]), int(m["dim"]), int(m["rot_dim"]), int(m["vdim"])
         self.Q, self.R = int(m["q_rank"]), int(m["kv_rank"])
         self.scale = float(m.get("scale", 1.0 / math.sqrt(self.dn + self.dr)))
@@ -261,12 +281,15 @@ class LatentAttention:
         if self.kv_from is None:
             wd.append(p.get(prefix + "dkv", (R + dr, d), 1.0 / math.sqrt(d)))
             self.kn = p.get(prefix + "dkv.norm", (R,), 0.1, 1.0, small=True)
-        self.n_down = sum(w.shape[0] for w in wd)
+        self.n_down = self.n_in = sum(w.shape[0] for w in wd)
+        if self.has_gate:
+            wd.append(p.get(prefix + "g", (H, d), 1.0 / math.sqrt(d)))
+            self.n_in += H
         self.n_tail = 0 if tail is None else tail.shape[0]
         if tail is not None:
             wd.append(tail)
         self.tail_out = None
-        self.w_down = torch.cat(wd).contiguous()  # [q_rank (+ kv_rank + rot_dim) (+ tail), d]: one launch
+        self.w_down = _rows8(wd, self.has_gate)  # [q_rank (+ kv_rank + rot_dim) (+ gate) (+ tail), d]: one launch
         self.qn = p.get(prefix + "dq.norm", (Q,), 0.1, 1.0, small=True)
         self.w_uq = p.get(prefix + "uq", (H * (dn + dr), Q), 1.0 / math.sqrt(Q))
         self.w_uk = p.get(prefix + "uk", (H * dn, R), 1.0 / math.sqrt(R))  # viewed [H, dn, R]
@@ -288,29 +311,34 @@ class LatentAttention:
     def forward(self, h: torch.Tensor, meta: AttnMeta, cache: dict) -> torch.Tensor:
         H, dn, dr, dv, Q, R = self.H, self.dn, self.dr, self.dv, self.Q, self.R
         T = h.shape[0]
-        down = F.linear(h, self.w_down)
+        proj = down = F.linear(h, self.w_down)
         if self.n_tail:
-            self.tail_out = (down, self.n_down)
-            down = down[:, :self.n_down]
+            self.tail_out = (proj, self.n_in)
+        if proj.shape[1] > self.n_down:
+            down = proj[:, :self.n_down]
+        gate = proj[:, self.n_down:self.n_in] if self.has_gate else None
         kc, vc = cache["k"], cache["v"]
         own = self.kv_from is None
         hops.latent_prep(down, Q, R, dr, self.qn, self.kn, self.eps, meta.positions, self.freq,
                          kc if own else None, vc if own else None, meta.slot_mapping if own else None, pairs=self.pairs)
         q = F.linear(down[:, :Q], self.w_uq)
         if self._expand_ok(h, meta):
-            return self._forward_expanded(q, down, meta, kc)
+            return self._forward_expanded(q, down, meta, kc, gate)
         # the per-head key expansion moved to the query: q_lat[h] = q_unrotated[h] @ W_uk[h]  ([H, T, R])
         q_lat = torch.bmm(q.view(T, H, dn + dr)[:, :, :dn].transpose(0, 1), self.w_uk.view(H, dn, R))
         qa = hops.latent_queries(q, q_lat, H, dn, dr, meta.positions, self.freq, self.pitch, pairs=self.pairs)
         args = (H, self.scale, self.window, self.sinks)
         kw = dict(fast=self.fast, sink=self.sink)
         if not meta.is_prefill:
-            o = hops.latent_attention(qa, kc, vc, meta.block_tables, *args, seq_lens=meta.seq_lens, **kw)
+            o = hops.latent_attention(qa, kc, vc, meta.block_tables, *args, seq_lens=meta.seq_lens, gate=gate, **kw)
         else:
             nd = meta.num_decode
-            o = hops.latent_attention(qa[nd:], kc, vc, meta.block_tables, *args, cu=meta.cu_seqlens, ctx=meta.ctx_start, **kw)
+            gc, gd = (gate[nd:], gate[:nd]) if gate is not None else (None, None)
+            o = hops.latent_attention(qa[nd:], kc, vc, meta.block_tables, *args, cu=meta.cu_seqlens, ctx=meta.ctx_start, gate=gc,
+                                      **kw)
             if nd:
-                od = hops.latent_attention(qa[:nd], kc, vc, meta.dec_block_tables, *args, seq_lens=meta.dec_seq_lens, **kw)
+                od = hops.latent_attention(qa[:nd], kc, vc, meta.dec_block_tables, *args, seq_lens=meta.dec_seq_lens, gate=gd,
+                                           **kw)
                 o = torch.cat([od, o])
         # ... and the value expansion to the result: v[h] = o_lat[h] @ W_uv[h]^T, written head by head
         # into the rows the out-projection reads
@@ -323,7 +351,8 @@ class LatentAttention:
                 and bool(self.fast) and h.shape[0] >= self.EXPAND_MIN_ROWS
                 and (self.dn + self.dr) in (64, 128) and self.dv in (64, 128))
 
-    def _forward_expanded(self, q: torch.Tensor, down: torch.Tensor, meta: AttnMeta, kc: torch.Tensor) -> torch.Tensor:
+    def _forward_expanded(self, q: torch.Tensor, down: torch.Tensor, meta: AttnMeta, kc: torch.Tensor,
+                          gate: Optional[torch.Tensor] = None) -> torch.Tensor:
         """Whole prompts: per-head keys and values of this step's rows in temporary pages, windowed
         attention's matrix-core kernel over them.  ``q`` [T, H * (dim + rot_dim)] still unturned."""
         H, dn, dr, dv, Q, R = self.H, self.dn, self.dr, self.dv, self.Q, self.R
@@ -345,7 +374,7 @@ class LatentAttention:
         # the queries' rotated parts turn here; the shared key part was turned by latent_prep
         hops.rotary_cache(fused, H, H, D, dv, meta.positions, self.freq, self.pairs, None, kt, vt, slots, rot_off=dn, rot_k=False)
         o = hops.window_attention_prefill(fused, kt, vt, meta.cu_seqlens, meta.ctx_start, bt, H, H, D, dv, self.scale,
-                                          self.window, self.sink, mfma=self.fast, sinks=self.sinks)
+                                          self.window, self.sink, mfma=self.fast, sinks=self.sinks, gate=gate)
         return F.linear(o, self.wo)
 
 
@@ -353,13 +382,15 @@ class RotaryAttention:
     """Grouped-query softmax attention with rotary positions on the first ``rot.dims`` entries of every
     query / key head (frequencies ``rot.base^(-2i/dims)``, optionally rescaled for long contexts by
     ``rot.scaling`` {factor, low, high, original}, ops.hybrid.rotary_freq).  Causal; ``mask.size`` keys
-    of sliding window where given (0 / absent: all).  Pages and attention kernels are windowed
-    attention's.  What a design fixes comes as ``opts`` (absent: the first value):
+    of sliding window where given (0 / absent: all), beside them the sequence's first ``mask.keep_first``
+    positions (absent: none).  Pages and attention kernels are windowed attention's.  What a design fixes comes as ``opts`` (absent: the first value):
 
-    * ``rotary`` "half" (entry i turns with entry i + rot.dims / 2) / "pairs" (2i with 2i + 1);
+    * ``rotary`` "half" (entry i turns with entry i + rot.dims / 2) / "pairs" (2i with 2i + 1) / "none" (no
+      positions; no ``rot`` constants);
     * ``temp`` True: a learned temperature per query head (``temp``: score = q.k * scale * temp[h]),
       folded into the query in the rotation pass;
-    * ``gate`` True: a sigmoid output gate ``heads * sigmoid(G h)`` in front of the out-projection;
+    * ``gate`` True: a sigmoid output gate ``heads * sigmoid(G h)`` in front of the out-projection / "head": one
+      number per head, applied in the attention kernels' epilogue / False;
     * ``qk_norm`` None / "before" (every q and k head RMS-normed over ``dim`` with the weights ``q.norm`` /
       ``k.norm`` [dim], then turned) / "after" (turned, then divided by its root mean square, no weight);
     * ``sink`` False / True: a learned logit per query head (``sink``) joins the softmax denominator;
@@ -387,12 +418,17 @@ class RotaryAttention:
         self.scale = float(m.get("scale", 1.0 / math.sqrt(self.dk)))
         self.window = int(m.get("mask.size", 0) or 0)
         self.chunked, self.cap = o.get("mask", "window") == "chunk", float(m.get("softcap", 0.0) or 0.0)
-        self.base, self.rdims = float(m.get("rot.base", 10000.0)), int(m.get("rot.dims", self.dk))
+        self.keep = int(m.get("mask.keep_first", 0) or 0) if self.window else 0  # without a window all keys are seen
+        if self.keep < 0 or (self.keep and self.chunked):
+            raise ValueError(f"{prefix}: mask.keep_first {self.keep} goes with a sliding window")
+        self.base = float(m.get("rot.base", 10000.0))
+        self.rdims = 0 if o.get("rotary") == "none" else int(m.get("rot.dims", self.dk))
         if self.rdims % 2 or not 0 <= self.rdims <= self.dk:
             raise ValueError(f"{prefix}: rot.dims {self.rdims} must be even and at most dim {self.dk}")
         self.pairs = o.get("rotary", (traits or {}).get("attention_rotary", "half")) == "pairs"
         self.norm = {None: 0, "before": 1, "after": 2}[o.get("qk_norm")]
         self.has_temp, self.has_gate, self.sink = bool(o.get("temp", True)), bool(o.get("gate", True)), bool(o.get("sink", False))
+        self.gate_heads = o.get("gate", True) == "head"
         self.eps = eps
         self.fast = 1
         nq, nk, nv = self.H * self.dk, self.G * self.dk, (0 if self.v_from_k else self.G * self.dv)
@@ -400,15 +436,16 @@ class RotaryAttention:
         ws = [p.get(prefix + "q", (nq, d), s), p.get(prefix + "k", (nk, d), s)]
         if not self.v_from_k:
             ws.append(p.get(prefix + "v", (nv, d), s))
+        n_gate = 0 if not self.has_gate else self.H if self.gate_heads else self.H * self.dv
         if self.has_gate:
-            ws.append(p.get(prefix + "g", (self.H * self.dv, d), s))
+            ws.append(p.get(prefix + "g", (n_gate, d), s))
         self.g_col = nq + nk + nv
-        self.n_in = self.g_col + (self.H * self.dv if self.has_gate else 0)
+        self.n_in = self.g_col + n_gate
         self.n_tail = 0 if tail is None else tail.shape[0]
         if tail is not None:
             ws.append(tail)
         self.tail_out = None
-        self.w_in = torch.cat(ws).contiguous()  # [q | k (| v) (| gate) (| tail)]: one launch
+        self.w_in = _rows8(ws, self.gate_heads)  # [q | k (| v) (| gate) (| tail)]: one launch
         self.temp = p.get(prefix + "temp", (self.H,), 0.2, 1.0, small=True) if self.has_temp else None
         self.qn = p.get(prefix + "q.norm", (self.dk,), 0.1, 1.0, small=True) if self.norm == 1 else None
         self.kn = p.get(prefix + "k.norm", (self.dk,), 0.1, 1.0, small=True) if self.norm == 1 else None
@@ -434,18 +471,20 @@ class RotaryAttention:
         hops.rotary_cache(proj, H, G, dk, dv, meta.positions, self.freq, self.pairs, self.temp, kc, vc, meta.slot_mapping,
                           norm=self.norm, qw=self.qn, kw=self.kn, eps=self.eps, v_from_k=self.v_from_k)
         args = (H, G, dk, dv, self.scale, self.window, self.sink)
-        kw = dict(sinks=self.sinks, chunked=self.chunked, cap=self.cap)
+        kw = dict(sinks=self.sinks, chunked=self.chunked, cap=self.cap, keep=self.keep, g_col=self.g_col)
+        hg = self.gate_heads
         if not meta.is_prefill:
-            o = hops.window_attention_decode(proj, kc, vc, meta.block_tables, meta.seq_lens, *args, vec=bool(self.fast), **kw)
+            o = hops.window_attention_decode(proj, kc, vc, meta.block_tables, meta.seq_lens, *args, vec=bool(self.fast),
+                                             gate=proj if hg else None, **kw)
         else:
             nd = meta.num_decode
             o = hops.window_attention_prefill(proj[nd:], kc, vc, meta.cu_seqlens, meta.ctx_start, meta.block_tables,
-                                              *args, mfma=self.fast, **kw)
+                                              *args, mfma=self.fast, gate=proj[nd:] if hg else None, **kw)
             if nd:
                 od = hops.window_attention_decode(proj[:nd], kc, vc, meta.dec_block_tables, meta.dec_seq_lens, *args,
-                                                  vec=bool(self.fast), **kw)
+                                                  vec=bool(self.fast), gate=proj[:nd] if hg else None, **kw)
                 o = torch.cat([od, o])
-        if self.has_gate:
+        if self.has_gate and not hg:
             o = hops.sigmoid_gate(o, proj, self.g_col)
         return F.linear(o, self.wo)
 
@@ -1000,6 +1039,43 @@ class GroupRoutedFFN:
                                 tile=self.tile)
 
 
+class CorrectedRoutedFFN:
+    """Top-k routed ungated experts ``down_e(relu(up_e h)^2)`` beside ``identity`` experts whose output is h
+    itself.  fp32 router: softmax over experts and identity experts together; the choice is by score plus
+    ``correction``, within the ``keep_groups`` best of ``groups`` equal groups of neighbours (a group is as
+    good as its best member); the weights are the scores as they are.  An optional shared expert of the same
+    form is added for every token."""
+
+    def __init__(self, spec: MoESpec, d: int, p: _Params, prefix: str):
+        self.E, self.K, self.ff, self.fs, self.ident = spec.experts, spec.top, spec.ff, spec.shared_ff, spec.identity
+        self.groups, self.keep = spec.groups, spec.keep_groups
+        n = self.E + self.ident
+        if self.E < 1 or not 1 <= self.K <= n or n % self.groups or not 1 <= self.keep <= self.groups:
+            raise ValueError(f"{prefix}: top {self.K} of {self.E} + {self.ident} experts in {self.groups} groups, {self.keep} kept")
+        if self.K > self.keep * (n // self.groups):
+            raise ValueError(f"{prefix}: top {self.K} exceeds the experts of {self.keep} groups")
+        s, s2 = 1.0 / math.sqrt(d), 1.0 / math.sqrt(self.ff)
+        self.il = False
+        # large bf16 steps run on the Mixtral path's tile GEMM (ops.hybrid.moe_experts)
+        self.tile = p.device.type == "cuda" and p.dtype == torch.bfloat16 and self.ff % 256 == 0 and d % 256 == 0
+        self.w1 = torch.stack([p.get(f"{prefix}e{e}.up", (self.ff, d), s) for e in range(self.E)])
+        self.w2 = torch.stack([p.get(f"{prefix}e{e}.down", (d, self.ff), s2) for e in range(self.E)])
+        self.wr = p.get(prefix + "router", (n, d), 2 * s, small=True)
+        self.corr = p.get(prefix + "correction", (n,), 0.1, small=True)
+        self.ws1 = self.ws2 = None
+        if self.fs:
+            self.ws1 = p.get(prefix + "shared.up", (self.fs, d), s)
+            self.ws2 = p.get(prefix + "shared.down", (d, self.fs), 1.0 / math.sqrt(self.fs))
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        ids, wts = hops.moe_router_grouped(h, self.wr, self.E + self.ident, self.K, self.groups, self.keep, 1.0, soft=True,
+                                           corr=self.corr, best2=False, renorm=False)
+        shared = None
+        if self.fs:
+            shared = F.linear(hops.activation(F.linear(h, self.ws1), "relu_sq"), self.ws2)
+        return hops.moe_experts(h, ids, wts, self.w1, self.w2, shared, None, act="relu_sq", identity=self.ident)
+
+
 def _ffn_for(family: str, spec, d: int, p: _Params, prefix: str, tail: Optional[torch.Tensor] = None):
     """The feed-forward of a layer in a design's family (models/config.DESIGN_TRAITS ``ffn``)."""
     if spec is None:
@@ -1013,6 +1089,8 @@ def _ffn_for(family: str, spec, d: int, p: _Params, prefix: str, tail: Optional[
             GroupRoutedFFN(spec, d, p, prefix)
     if family == "relu_sq" and isinstance(spec, DenseSpec):
         return UngatedDenseFFN(spec, d, p, prefix, "relu_sq")
+    if family == "relu_sq_corrected" and isinstance(spec, MoESpec):
+        return CorrectedRoutedFFN(spec, d, p, prefix)
     if family == "plain_softmax":
         return DenseFFN(spec, d, p, prefix) if isinstance(spec, DenseSpec) else PlainRoutedFFN(spec, d, p, prefix)
     raise ValueError(f"{prefix}: no {type(spec).__name__} feed-forward in the {family!r} family")
@@ -1060,15 +1138,19 @@ class HybridLM:
                                or self.shifted or self.depth_avg or self.gated):
             raise ValueError(f"{cfg.name}: norms behind the sublayers are built for plain sequential blocks on layer "
                              "norms with a bias, without looped layers")
+        self.S = cfg.streams
+        if self.S < 0 or (self.S and (not self.sequential or self.summed or self.shifted or self.depth_avg or self.gated or self.one_plus)):
+            raise ValueError(f"{cfg.name}: several residual streams are built for plain sequential blocks on RMS norms")
         if not self.post_norm and (tr.get("norm_bias") or tr.get("pair_norm") is not None):
             raise ValueError(f"{cfg.name}: norm biases and normed mixer pairs are built for blocks with norms behind the sublayers")
         nm = 1.0 if not self.one_plus else 0.0  # plain norm weights sit around one
         self.embed = p.get("embed", (V, d), 0.5)
         self.pos = p.get("pos", (cfg.max_position, d), 0.1) if tr["learned_pos"] else None
-        self.loop_step = p.get("loop.step", (cfg.loop[2], d), 0.1, small=True) if cfg.loop else None
+        self.loop_step = p.get("loop.step", (cfg.loop[2], d), 0.1, small=True) if cfg.loop and tr.get("loop_step", True) else None
         self.norms, self.norms2, self.mixers, self.ffns, self.shifts, self.dwa = [], [], [], [], [], []
         self.rg1, self.rg2 = [], []  # gated residual: (bias [d] fp32, weight rows kept for export), per sublayer
-        names = dict(tr.get("mixers", {}))
+        names = {k: v if isinstance(v, str) else v[0] for k, v in tr.get("mixers", {}).items()}
+        options = {k: dict(opts=v[1]) for k, v in tr.get("mixers", {}).items() if not isinstance(v, str)}
         names.update({k: SideBySide.kind for k in tr.get("composite", {})})
         nshape = () if self.scalar_norm else (d,)
         # per-layer token input: layer i reads columns [i * side_dim, (i + 1) * side_dim) of a second table
@@ -1088,8 +1170,14 @@ class HybridLM:
         def rgate(name):
             return p.get(name, (d, d), 1.0 / math.sqrt(d)), p.get(name + ".b", (d,), 0.5, small=True)
 
+        def stream_w(name):  # (read weights [S], mix [S, S] indexed [from, to], write weights [S])
+            n = self.S
+            return (p.get(name + ".in", (n,), 0.2, 1.0 / n, small=True), p.get(name + ".mix", (n, n), 0.3 / n, 1.0 / n, small=True),
+                    p.get(name + ".out", (n,), 0.3, 1.0, small=True))
+
+        self.hc1, self.hc2 = [], []
         per_layer = (self.norms, self.norms2, self.mixers, self.ffns, self.shifts, self.dwa, self.rg1, self.rg2, self.post1,
-                     self.post2, self.bias1, self.bias2, *((self.side_gate, self.side_proj, self.side_norm) if sd else ()))
+                     self.post2, self.bias1, self.bias2, self.hc1, self.hc2, *((self.side_gate, self.side_proj, self.side_norm) if sd else ()))
         owners = [cfg.owner(i) for i in range(len(cfg.layers))]
         for i, spec in enumerate(cfg.layers):
             if owners[i] != i:
@@ -1102,7 +1190,9 @@ class HybridLM:
             self.norms.append(norm_w(f"l{i}.norm1"))
             g1 = rgate(f"l{i}.rg1") if self.gated else None
             self.mixers.append(MIXERS[kind](spec, d, cfg.norm_eps, p, f"l{i}.mix.", traits=tr,
-                                            tail=g1[0] if g1 else None))
+                                            tail=g1[0] if g1 else None, **options.get(spec.kind, {})))
+            self.hc1.append(stream_w(f"l{i}.hc1") if self.S else None)
+            self.hc2.append(stream_w(f"l{i}.hc2") if self.S and spec.mlp is not None else None)
             g2 = rgate(f"l{i}.rg2") if self.gated and spec.mlp is not None else None
             self.ffns.append(_ffn_for(tr["ffn"], spec.mlp, d, p, f"l{i}.mlp.", tail=g2[0] if g2 else None)
                              if self.gated else _ffn_for(tr["ffn"], spec.mlp, d, p, f"l{i}.mlp."))
@@ -1197,6 +1287,7 @@ class HybridLM:
         ts = [self.embed, self.final_norm, self.head] + self.norms + self.side_gate + self.side_proj + self.side_norm
         ts += [t for t in [self.pos, self.loop_step, self.side_embed] + self.norms2 + self.shifts + self.dwa if t is not None]
         ts += [t for t in self.bias1 + self.bias2 + [self.final_bias] if t is not None]
+        ts += [t for hc in self.hc1 + self.hc2 if hc is not None for t in hc]
         ts += [t for pair in self.post1 + self.post2 if pair is not None for t in pair]
         ts += [t for m in self.mixers for t in (getattr(m, "out_w", None) or ())]
         ts += [t for g in self.rg1 + self.rg2 if g is not None for t in g.values() if t is not None]
@@ -1255,6 +1346,8 @@ class HybridLM:
         else:
             x = hops.embed_pos(ids, meta.positions, self.embed, self.pos, meta.dec_src, meta.dec_prev,
                                scale=c.embed_scale)
+        if self.S:
+            return self._forward_streams(x, meta, caches)
         if self.gated:
             return self._forward_gated(x, meta, caches)
         if self.post_norm:
@@ -1356,6 +1449,33 @@ class HybridLM:
             pend = (tuple(a.index_select(0, idx) for a in pend[0]), *pend[1:])
         return self._logits(join(x, (self.final_norm, self.final_bias), self.dtype))
 
+    def _forward_streams(self, x: torch.Tensor, meta: AttnMeta, caches: list) -> torch.Tensor:
+        """Several residual streams: what a sublayer leaves pending is written to the streams in the launch
+        that reads and norms the next sublayer's input (ops.hybrid.stream_norm).  At the start all streams
+        are the embedding output ``x``, which stands for them until the first result is written."""
+        eps, S = self.cfg.norm_eps, self.S
+        xs, y, write = x.unsqueeze(1), None, None
+
+        def step(hc, w):  # the pending result into the streams; the next sublayer's input
+            return hops.stream_norm(xs, y, write, hc[0] if hc is not None else None, w, eps, self.dtype, S)
+
+        for r, (li, t, first) in enumerate(self.runs):
+            if first and self.loop_step is not None:
+                raise ValueError("loop vectors are not built for several residual streams")
+            for hc, w, sub in ((self.hc1[li], self.norms[li], self.mixers[li]), (self.hc2[li], self.norms2[li], self.ffns[li])):
+                if sub is None:
+                    continue
+                h, xs = step(hc, w)
+                y = sub.forward(h, meta, caches[self.kv_run[r]]) if sub is self.mixers[li] else sub.forward(h)
+                write = (hc[1], hc[2])
+            if self.layer_probe is not None:  # the sum of the streams with the pending result
+                full = torch.einsum("nsd,st->nd", xs.expand(-1, S, -1), write[0]) + write[1].sum() * y.float()
+                self.layer_probe.append(full)
+        if meta.logits_idx is not None:
+            idx = meta.logits_idx
+            xs, y = xs.index_select(0, idx), y.index_select(0, idx)
+        return self._logits(step(None, self.final_norm)[0])
+
     def _logits(self, hf: torch.Tensor) -> torch.Tensor:
         c = self.cfg
         z = F.linear(hf, self.head).float()
@@ -1438,16 +1558,22 @@ def state_dict(model: HybridLM) -> dict:
         for key, t in (("shift", model.shifts[i]), ("dwa", model.dwa[i])):
             if t is not None:
                 out[p + key] = t
+        for key, hc in (("hc1", model.hc1[i]), ("hc2", model.hc2[i])):
+            if hc is not None:
+                out.update({p + key + ".in": hc[0], p + key + ".mix": hc[1], p + key + ".out": hc[2]})
         for key, g, sub in (("rg1", model.rg1[i], m), ("rg2", model.rg2[i], f)):
             if g is not None:  # the gate's rows are the tail of the sublayer's input projection, or its own
                 w_in = getattr(sub, "w_in", getattr(sub, "w_down", None))
-                out[p + key] = g["w"] if g["w"] is not None else w_in[w_in.shape[0] - sub.n_tail:]
+                n0 = getattr(sub, "n_in", w_in.shape[0] - sub.n_tail)
+                out[p + key] = g["w"] if g["w"] is not None else w_in[n0:n0 + sub.n_tail]
                 out[p + key + ".b"] = g["b"]
         if isinstance(m, LatentAttention):
             out.update({p + "mix.dq": m.w_down[:m.Q], p + "mix.dq.norm": m.qn, p + "mix.uq": m.w_uq, p + "mix.uk": m.w_uk,
                         p + "mix.uv": m.w_uv, p + "mix.o": m.wo})
             if m.sinks is not None:
                 out[p + "mix.sink"] = m.sinks
+            if m.has_gate:
+                out[p + "mix.g"] = m.w_down[m.n_down:m.n_in]
             if m.kv_from is None:
                 out.update({p + "mix.dkv": m.w_down[m.Q:m.n_down], p + "mix.dkv.norm": m.kn})
         elif hasattr(m, "export"):
@@ -1475,10 +1601,12 @@ def state_dict(model: HybridLM) -> dict:
                 out[f"{p}mlp.e{e}.gate"], out[f"{p}mlp.e{e}.up"] = f.w13[e, :f.ff], f.w13[e, f.ff:]
                 out[f"{p}mlp.e{e}.down"] = f.w2[e]
             out[p + "mlp.router"] = f.wr
-        elif isinstance(f, PlainRoutedFFN):
+        elif isinstance(f, (PlainRoutedFFN, CorrectedRoutedFFN)):
             for e in range(f.E):
                 out[f"{p}mlp.e{e}.up"], out[f"{p}mlp.e{e}.down"] = f.w1[e], f.w2[e]
             out[p + "mlp.router"] = f.wr
+            if isinstance(f, CorrectedRoutedFFN):
+                out[p + "mlp.correction"] = f.corr
             if f.fs:
                 out.update({p + "mlp.shared.up": f.ws1, p + "mlp.shared.down": f.ws2})
         elif f is not None:

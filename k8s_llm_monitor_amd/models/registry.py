@@ -18,7 +18,7 @@ from .llama import CausalLM
 
 # config.arch -> model class
 MODEL_CLASSES = {"llama": CausalLM, "gpt2": CausalLM, "dunesun": HybridLM, "kisutar": HybridLM, "bitonex": HybridLM,
-                 "levovik": HybridLM, "dopivik": HybridLM}
+                 "levovik": HybridLM, "dopivik": HybridLM, "zifisun": HybridLM}
 # layer-list designs by the ``architecture`` value of their config.json (lower case)
 LAYER_LIST_ARCHS = set(DESIGN_TRAITS)
 

@@ -17,15 +17,19 @@ int k8sllm_hy_gated_lookup(void* out, const void* gate, const void* table, long 
 int k8sllm_hy_rotary_norm_cache(void* qkv, long stride, long T, int Hq, int G, int dk, int dv, const int* positions,
                                 const float* freq, int nf, int pairs, int norm, const float* qw, const float* kw,
                                 float eps, const float* q_scale, void* k_cache, void* v_cache, const int* slots, int bs,
-                                int v_from_k, int f32, hipStream_t s);
+                                int v_from_k, int vec, int f32, hipStream_t s);
+int k8sllm_hy_stream_norm(void* out, float* dst, const float* src, long src_row, long src_s, const void* y, int yt,
+                          const float* mix, const float* wout, const float* win, const float* w, long rows, int S, int d,
+                          float eps, int f32, hipStream_t s);
 int k8sllm_hy_decay_scan(float* o, const void* qkv, long stride, int q_col, int k_col, int v_col, const void* z,
                          long z_stride, const float* z_bias, const float* a_log, float inv_tau, int dkind, int per_head,
                          const void* beta, long b_stride, const float* bonus, float* state, const int* cu,
                          const int* ctx, const int* slot, int S, int H, int Gk, int dk, int dv, float q_scale, int unit,
                          int f32, float* ws, long T, hipStream_t s);
 long k8sllm_hy_decay_scan_ws(long T, int H, int Gk, int dk);
-int k8sllm_hy_router_grouped(int* ids, float* wts, const void* h, long T, int d, const float* wr, int E, int K,
-                             int groups, int keep, float scale, int f32, hipStream_t s);
+int k8sllm_hy_router_grouped(int* ids, float* wts, const void* h, long T, int d, const float* wr, const float* corr, int E,
+                             int K, int groups, int keep, float scale, int soft, int best2, int renorm, int f32,
+                             hipStream_t s);
 int k8sllm_hy_add_norm(void* out, float* residual, const void* a0, int t0, const void* a1, int t1, const void* a2,
                        int t2, const float* vec, const float* w, long rows, int d, float eps, int one_plus, int f32,
                        hipStream_t s);
@@ -48,12 +52,13 @@ int k8sllm_hy_qk_norm_cache(void* qkv, long stride, const float* qw, const float
                             int nk, int nv, void* k_cache, void* v_cache, const int* slots, int bs, int f32, hipStream_t s);
 int k8sllm_hy_window_prefill(void* out, const void* qkv, long q_stride, const void* k_cache, const void* v_cache,
                              const int* cu, const int* ctx, const int* block_tables, int bt_stride, int S, long T,
-                             int Hq, int G, int dk, int dv, int bs, float scale, int window, int chunked, float cap, int sink,
-                             const float* sinks, int f32, int mfma, hipStream_t s);
+                             int Hq, int G, int dk, int dv, int bs, float scale, int window, int chunked, int keep,
+                             float cap, int sink, const float* sinks, const void* gate, long g_stride, int f32, int mfma,
+                             hipStream_t s);
 int k8sllm_hy_window_decode(void* out, const void* qkv, long q_stride, const void* k_cache, const void* v_cache,
                             const int* block_tables, int bt_stride, const int* seq_lens, int B, int Hq, int G, int dk,
-                            int dv, int bs, float scale, int window, int chunked, float cap, int sink, const float* sinks, int f32, int vec,
-                            hipStream_t s);
+                            int dv, int bs, float scale, int window, int chunked, int keep, float cap, int sink,
+                            const float* sinks, const void* gate, long g_stride, int f32, int vec, hipStream_t s);
 int k8sllm_hy_conv_silu(void* out, const void* proj, long stride, int col0, int C, const float* cw, const float* cb,
                         int taps, void* state, const int* cu, const int* ctx, const int* slot, int S, long T, int f32,
                         hipStream_t s);
@@ -78,7 +83,8 @@ int k8sllm_hy_grouped_gemm(void* Y, const void* A, const void* W, const int* off
                            int E, long rows, int N, int Kd, long w_es, int act, int il, int f32, int mfma, float limit,
                            hipStream_t s);
 int k8sllm_hy_combine(float* out, const void* ys, const int* inv, const float* wts, const void* shared,
-                      const float* gate, long T, int K, int d, int f32, hipStream_t s);
+                      const float* gate, const int* ids, const void* h, int n_real, long T, int K, int d, int f32,
+                      hipStream_t s);
 int k8sllm_hy_norm_shift(void* out, const float* x, const float* w, const float* mu, float* state, const int* cu,
                          const int* ctx, const int* slot, int S, long rows, int d, float eps, int one_plus,
                          int advance, int multi, int f32, hipStream_t s);
@@ -94,7 +100,7 @@ int k8sllm_hy_latent_queries(void* out, const void* q, long q_stride, const void
 int k8sllm_hy_latent_attention(void* out, const void* q, long q_stride, const void* k_cache, const void* v_cache,
                                const int* cu, const int* ctx, const int* seq_lens, const int* block_tables,
                                int bt_stride, int S, long T, int H, int dkp, int dv, int bs, float scale, int window,
-                               const float* sinks, int split, hipStream_t s);
+                               const float* sinks, const void* gate, long g_stride, int split, hipStream_t s);
 int k8sllm_moe_align(const int* topk_ids, long n, int E, int* expert_offsets, int* sorted_idx, int* inv_idx,
                      hipStream_t s);
 }
@@ -299,6 +305,22 @@ const float* sink_ptr(const OptT& sinks, int64_t Hq) {
   return sinks->data_ptr<float>();
 }
 
+// head gate logits: columns g_col .. g_col + Hq of rows that go with the queries' (absent: no gate)
+struct Gate {
+  const void* p = nullptr;
+  long stride = 0;
+};
+Gate gate_of(const OptT& gate, int64_t g_col, int64_t rows, int64_t Hq, int f) {
+  Gate g;
+  if (!gate.has_value()) return g;
+  same(*gate, f, "gate");
+  TORCH_CHECK(gate->dim() == 2 && gate->stride(1) == 1 && gate->size(0) >= rows && g_col >= 0 && g_col + Hq <= gate->size(1),
+              "gate [T, >= g_col + heads]");
+  g.p = (const char*)gate->data_ptr() + g_col * gate->element_size();
+  g.stride = gate->stride(0);
+  return g;
+}
+
 void qk_norm_cache(Tensor qkv, Tensor qw, Tensor kw, double eps, int64_t Hq, int64_t G, int64_t dk, int64_t dv,
                    OptT k_cache, OptT v_cache, OptT slots) {
   const int f = act(qkv, "qkv");
@@ -326,7 +348,8 @@ void qk_norm_cache(Tensor qkv, Tensor qw, Tensor kw, double eps, int64_t Hq, int
 
 void window_attention_prefill(Tensor out, Tensor qkv, Tensor k_cache, Tensor v_cache, Tensor cu, Tensor ctx,
                               Tensor block_tables, int64_t Hq, int64_t G, int64_t dk, int64_t dv, double scale,
-                              int64_t window, bool sink, OptT sinks, int64_t mfma, bool chunked, double cap) {
+                              int64_t window, bool sink, OptT sinks, int64_t mfma, bool chunked, double cap,
+                              int64_t keep, OptT gate, int64_t g_col) {
   const int f = act(qkv, "qkv");
   same(out, f, "out");
   pages(k_cache, f, G * dk, "k_cache");
@@ -341,17 +364,20 @@ void window_attention_prefill(Tensor out, Tensor qkv, Tensor k_cache, Tensor v_c
   TORCH_CHECK(out.is_contiguous() && out.numel() == T * Hq * dv, "out [T, Hq*dv]");
   TORCH_CHECK(cu.numel() == S + 1 && block_tables.size(0) >= S, "cu [S+1], block_tables [S, W]");
   TORCH_CHECK(window >= 0 && G >= 1 && Hq % G == 0 && cap >= 0, "heads / window / cap");
+  TORCH_CHECK(keep >= 0 && (keep == 0 || (window > 0 && !chunked)), "kept first positions go with a sliding window");
+  const Gate ga = gate_of(gate, g_col, T, Hq, f);
   check(k8sllm_hy_window_prefill(out.data_ptr(), qkv.data_ptr(), qkv.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
                                  cu.data_ptr<int>(), ctx.data_ptr<int>(), block_tables.data_ptr<int>(),
                                  (int)block_tables.stride(0), (int)S, T, (int)Hq, (int)G, (int)dk, (int)dv,
-                                 (int)k_cache.size(1), (float)scale, (int)window, chunked, (float)cap, sink,
-                                 sink_ptr(sinks, Hq), f, (int)mfma, cur()),
+                                 (int)k_cache.size(1), (float)scale, (int)window, chunked, (int)keep, (float)cap, sink,
+                                 sink_ptr(sinks, Hq), ga.p, ga.stride, f, (int)mfma, cur()),
         "window_attention_prefill");
 }
 
 void window_attention_decode(Tensor out, Tensor qkv, Tensor k_cache, Tensor v_cache, Tensor block_tables,
                              Tensor seq_lens, int64_t Hq, int64_t G, int64_t dk, int64_t dv, double scale,
-                             int64_t window, bool sink, OptT sinks, bool vec, bool chunked, double cap) {
+                             int64_t window, bool sink, OptT sinks, bool vec, bool chunked, double cap, int64_t keep,
+                             OptT gate, int64_t g_col) {
   const int f = act(qkv, "qkv");
   same(out, f, "out");
   pages(k_cache, f, G * dk, "k_cache");
@@ -365,10 +391,13 @@ void window_attention_decode(Tensor out, Tensor qkv, Tensor k_cache, Tensor v_ca
   TORCH_CHECK(out.is_contiguous() && out.numel() == B * Hq * dv, "out [B, Hq*dv]");
   TORCH_CHECK(seq_lens.numel() >= B && block_tables.size(0) >= B, "seq_lens [B], block_tables [B, W]");
   TORCH_CHECK(window >= 0 && G >= 1 && Hq % G == 0 && cap >= 0, "heads / window / cap");
+  TORCH_CHECK(keep >= 0 && (keep == 0 || (window > 0 && !chunked)), "kept first positions go with a sliding window");
+  const Gate ga = gate_of(gate, g_col, B, Hq, f);
   check(k8sllm_hy_window_decode(out.data_ptr(), qkv.data_ptr(), qkv.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
                                 block_tables.data_ptr<int>(), (int)block_tables.stride(0), seq_lens.data_ptr<int>(),
                                 (int)B, (int)Hq, (int)G, (int)dk, (int)dv, (int)k_cache.size(1), (float)scale,
-                                (int)window, chunked, (float)cap, sink, sink_ptr(sinks, Hq), f, vec, cur()),
+                                (int)window, chunked, (int)keep, (float)cap, sink, sink_ptr(sinks, Hq), ga.p, ga.stride,
+                                f, vec, cur()),
         "window_attention_decode");
 }
 
@@ -613,7 +642,7 @@ void rotary_norm_cache(Tensor qkv, int64_t Hq, int64_t G, int64_t dk, int64_t dv
   check(k8sllm_hy_rotary_norm_cache(qkv.data_ptr(), qkv.stride(0), T, (int)Hq, (int)G, (int)dk, (int)dv,
                                     positions.data_ptr<int>(), freq.data_ptr<float>(), (int)freq.numel(), pairs, (int)norm,
                                     qwp, kwp, (float)eps, qs, kc, vc, sp, k_cache.has_value() ? (int)k_cache->size(1) : 16,
-                                    v_from_k, f, cur()),
+                                    v_from_k, vec8(qkv, 0, dk) && (kc == nullptr || nk % 8 == 0), f, cur()),
         "rotary_norm_cache");
 }
 
@@ -761,8 +790,17 @@ void token_mix(Tensor out, Tensor h, Tensor mu, Tensor state, Tensor cu, Tensor 
         "token_mix");
 }
 
-void moe_router_grouped(Tensor ids, Tensor wts, Tensor h, Tensor wr, int64_t E, int64_t K, int64_t groups, int64_t keep,
-                        double scale) {
+// soft: softmax over all E logits, else sigmoid scores; corr [E] (optional) is added for the choice only;
+// best2: a group counts as the sum of its two best choice scores, else as its best; renorm: the weights
+// are divided by their sum
+void moe_router_grouped(Tensor ids, Tensor wts, Tensor h, Tensor wr, OptT corr, int64_t E, int64_t K, int64_t groups,
+                        int64_t keep, double scale, bool soft, bool best2, bool renorm) {
+  const float* cp = nullptr;
+  if (corr.has_value()) {
+    f32c(*corr, "correction");
+    TORCH_CHECK(corr->numel() == E, "correction [E]");
+    cp = corr->data_ptr<float>();
+  }
   const int f = act(h, "h");
   i32c(ids, "ids");
   f32c(wts, "wts");
@@ -774,7 +812,7 @@ void moe_router_grouped(Tensor ids, Tensor wts, Tensor h, Tensor wr, int64_t E, 
                   K <= keep * (E / groups),
               "router: up to 256 experts, top 16 within the kept groups");
   check(k8sllm_hy_router_grouped(ids.data_ptr<int>(), wts.data_ptr<float>(), h.data_ptr(), T, (int)d, wr.data_ptr<float>(),
-                                 (int)E, (int)K, (int)groups, (int)keep, (float)scale, f, cur()),
+                                 cp, (int)E, (int)K, (int)groups, (int)keep, (float)scale, soft, best2, renorm, f, cur()),
         "moe_router_grouped");
 }
 
@@ -792,10 +830,10 @@ void moe_align(Tensor ids, int64_t E, Tensor offsets, Tensor sorted_idx, Tensor 
 
 // y [rows, N] = W[e] a over expert-sorted rows; sorted_idx given: a's row of sorted row r is sorted_idx[r] / div
 // act_code: 0 none, 1 SwiGLU (w = [gate rows ; up rows]), 2 erf GELU
-// 3 the clamped gated unit (w = [gate rows ; up rows], limit)
+// 3 the clamped gated unit (w = [gate rows ; up rows], limit), 4 squared ReLU
 void grouped_gemm(Tensor y, Tensor a, Tensor w, Tensor offsets, OptT sorted_idx, int64_t div, int64_t act_code, bool il,
                   bool mfma, double limit) {
-  TORCH_CHECK(act_code >= 0 && act_code <= 3 && (act_code != 3 || limit > 0), "grouped_gemm: activation code");
+  TORCH_CHECK(act_code >= 0 && act_code <= 4 && (act_code != 3 || limit > 0), "grouped_gemm: activation code");
   const bool swiglu = act_code == 1 || act_code == 3;
   const int f = act(a, "a");
   same(y, f, "y");
@@ -819,7 +857,8 @@ void grouped_gemm(Tensor y, Tensor a, Tensor w, Tensor offsets, OptT sorted_idx,
         "grouped_gemm");
 }
 
-void moe_combine(Tensor out, Tensor ys, Tensor inv, Tensor wts, OptT shared, OptT gate) {
+// ids [T, K] and h [T, d] (together, optional): a chosen id >= n_real adds the row of h instead of an expert's
+void moe_combine(Tensor out, Tensor ys, Tensor inv, Tensor wts, OptT shared, OptT gate, OptT ids, OptT h, int64_t n_real) {
   const int f = act(ys, "ys");
   f32c(out, "out");
   f32c(wts, "wts");
@@ -828,6 +867,14 @@ void moe_combine(Tensor out, Tensor ys, Tensor inv, Tensor wts, OptT shared, Opt
   TORCH_CHECK(out.dim() == 2 && ys.dim() == 2 && ys.is_contiguous() && ys.size(1) == d && ys.size(0) == T * K &&
                   inv.numel() == T * K && wts.numel() == T * K,
               "moe_combine: shapes");
+  const int* ip = iptr(ids, "ids");
+  const void* hp = nullptr;
+  TORCH_CHECK((ip != nullptr) == h.has_value(), "moe_combine: ids and h come together");
+  if (ip) {
+    same(*h, f, "h");
+    TORCH_CHECK(ids->numel() == T * K && h->is_contiguous() && h->numel() == T * d, "moe_combine: ids [T, K], h [T, d]");
+    hp = h->data_ptr();
+  }
   const void* sh = nullptr;
   const float* gp = nullptr;
   if (shared.has_value()) {
@@ -840,9 +887,39 @@ void moe_combine(Tensor out, Tensor ys, Tensor inv, Tensor wts, OptT shared, Opt
       gp = gate->data_ptr<float>();
     }
   }
-  check(k8sllm_hy_combine(out.data_ptr<float>(), ys.data_ptr(), inv.data_ptr<int>(), wts.data_ptr<float>(), sh, gp, T,
-                          (int)K, (int)d, f, cur()),
+  check(k8sllm_hy_combine(out.data_ptr<float>(), ys.data_ptr(), inv.data_ptr<int>(), wts.data_ptr<float>(), sh, gp, ip, hp,
+                          (int)n_real, T, (int)K, (int)d, f, cur()),
         "moe_combine");
+}
+
+// streams: src [T, S, d], or [T, 1, d] for S equal ones; y given: dst [T, S, d] takes mix / wout (dst may be src);
+// out = the RMS norm of sum_t win[t] x_t (win absent: the plain sum) times w
+void stream_norm(Tensor out, OptT dst, Tensor src, int64_t S, OptT y, OptT mix, OptT wout, OptT win, Tensor w, double eps) {
+  const int f = act(out, "out");
+  f32c(src, "streams");
+  f32c(w, "w");
+  TORCH_CHECK(src.dim() == 3 && S >= 1 && S <= 16 && (src.size(1) == S || src.size(1) == 1), "streams [T, S | 1, d], S up to 16");
+  const int64_t rows = src.size(0), d = src.size(2);
+  TORCH_CHECK(out.is_contiguous() && out.numel() == rows * d && w.numel() == d, "stream_norm: out [T, d], w [d]");
+  const int yt = any_dt(y, rows * d, "y");
+  auto vec = [&](const OptT& t, int64_t n, const char* name) -> const float* {
+    if (!t.has_value()) return nullptr;
+    f32c(*t, name);
+    TORCH_CHECK(t->numel() == n, "stream_norm: size of ", name);
+    return t->data_ptr<float>();
+  };
+  const float *mp = vec(mix, S * S, "mix"), *op = vec(wout, S, "out weights"), *ip = vec(win, S, "in weights");
+  float* dp = nullptr;
+  if (yt) {
+    TORCH_CHECK(dst.has_value() && mp != nullptr && op != nullptr, "stream_norm: a result needs dst, mix and out weights");
+    f32c(*dst, "new streams");
+    TORCH_CHECK(dst->dim() == 3 && dst->size(0) == rows && dst->size(1) == S && dst->size(2) == d, "new streams [T, S, d]");
+    dp = dst->data_ptr<float>();
+  }
+  check(k8sllm_hy_stream_norm(out.data_ptr(), dp, src.data_ptr<float>(), src.size(1) * d, src.size(1) == 1 ? 0 : d,
+                              yt ? y->data_ptr() : nullptr, yt, mp, op, ip, w.data_ptr<float>(), rows, (int)S, (int)d,
+                              (float)eps, f, cur()),
+        "stream_norm");
 }
 
 void norm_shift(Tensor out, Tensor x, Tensor w, double eps, bool one_plus, Tensor mu, Tensor state, Tensor cu, Tensor ctx,
@@ -941,7 +1018,8 @@ void latent_queries(Tensor out, Tensor q, Tensor q_lat, int64_t H, int64_t dn, i
 // The matrix-core latent attention; false: these sizes or dtype are not the kernel's, nothing was
 // launched.  cu / ctx given: prompt chunks (block_tables per segment); else one row per sequence.
 bool latent_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache, OptT cu, OptT ctx, OptT seq_lens,
-                      Tensor block_tables, int64_t H, double scale, int64_t window, OptT sinks, int64_t split) {
+                      Tensor block_tables, int64_t H, double scale, int64_t window, OptT sinks, int64_t split, OptT gate,
+                      int64_t g_col) {
   if (act(q, "q") != 0) return false;
   same(out, 0, "out");
   TORCH_CHECK(k_cache.dim() == 3 && v_cache.dim() == 4, "pages");
@@ -966,10 +1044,11 @@ bool latent_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache, OptT
     TORCH_CHECK(slp != nullptr && seq_lens->numel() >= T && block_tables.size(0) >= T, "seq_lens [T], block_tables [T, W]");
   }
   TORCH_CHECK(window >= 0 && H >= 1, "heads / window");
+  const Gate ga = gate_of(gate, g_col, T, H, 0);
   const int rc = k8sllm_hy_latent_attention(out.data_ptr(), q.data_ptr(), q.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
                                             cup, ctxp, slp, block_tables.data_ptr<int>(), (int)block_tables.stride(0), (int)S, T,
                                             (int)H, (int)dkp, (int)dv, (int)k_cache.size(1), (float)scale, (int)window,
-                                            sink_ptr(sinks, H), (int)split, cur());
+                                            sink_ptr(sinks, H), ga.p, ga.stride, (int)split, cur());
   if (rc == 1) return false;
   check(rc, "latent_attention");
   return true;
@@ -1012,4 +1091,5 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("join_norm", &join_norm);
   m.def("token_mix", &token_mix);
   m.def("moe_router_grouped", &moe_router_grouped);
+  m.def("stream_norm", &stream_norm);
 }

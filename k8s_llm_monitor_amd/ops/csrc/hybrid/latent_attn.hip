@@ -116,7 +116,8 @@ __global__ __launch_bounds__(256) void latent_queries_kernel(T* __restrict__ out
 // maximum first, then the outputs summed wave after wave into one buffer.  Only wave 0 starts from
 // the sink.  Scores, weights and sums are fp32, base-2 exponentials (the scale carries log2 e).
 // QT consecutive tokens of a prompt chunk share a wave's key and value fragments (their windows
-// differ by one key at each end).
+// differ by one key at each end).  gate (optional): one logit per row and head; the head's output is
+// multiplied by its sigmoid before the one rounding.
 // KS_MAX / DT_MAX bound the key width / 32 and the value width / 16 (register arrays); the real
 // widths are run-time (wave-uniform guards).  cu == nullptr: one row per sequence at seq_lens - 1.
 // how far (base-2 logits) a tile's maximum must exceed the running one before that is moved
@@ -149,7 +150,7 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_mfma_kernel(
     bf16_t* __restrict__ out, const bf16_t* __restrict__ q, long q_stride, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int* __restrict__ cu, const int* __restrict__ ctx,
     const int* __restrict__ seq_lens, const int* __restrict__ block_tables, int bt_stride, int S, int H, int dkp,
-    int dv, float scale, int window, const float* __restrict__ sinks) {
+    int dv, float scale, int window, const float* __restrict__ sinks, const bf16_t* __restrict__ gate, long g_stride) {
   static_assert(NW == 1 || QT == 1, "the window is split over waves only for single tokens");
   constexpr int OP = DT_MAX * 16 + 4;  // LDS row pitch of the merge buffer (floats)
   __shared__ __attribute__((aligned(16))) float o_s[NW > 1 ? 16 * OP : 4];
@@ -312,7 +313,8 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_mfma_kernel(
 #pragma unroll
     for (int t = 0; t < QT; ++t) {
       if (t >= nt) break;
-      const float inv = l[t] > 0.f ? 1.f / l[t] : 0.f;
+      float inv = l[t] > 0.f ? 1.f / l[t] : 0.f;
+      if (gate != nullptr) inv *= sigmoid_f(bf2f(gate[(long)(row0 + t) * g_stride + head]));
       bf16_t* orow = obase + ((long)t * H + c16) * dv;
 #pragma unroll
       for (int dt = 0; dt < DT_MAX; ++dt)
@@ -353,7 +355,8 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_mfma_kernel(
     float L = 0.f;
 #pragma unroll
     for (int w = 0; w < NW; ++w) L += l_s[w][hh];
-    obase[c] = f2bf(L > 0.f ? o_s[hh * OP + dd] / L : 0.f);
+    const float gt = gate != nullptr ? sigmoid_f(bf2f(gate[(long)row0 * g_stride + hg * 16 + hh])) : 1.f;
+    obase[c] = f2bf(L > 0.f ? o_s[hh * OP + dd] / L * gt : 0.f);
   }
 }
 
@@ -368,7 +371,7 @@ __global__ __launch_bounds__(256) void latent_attn_lds_kernel(
     bf16_t* __restrict__ out, const bf16_t* __restrict__ q, long q_stride, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int* __restrict__ cu, const int* __restrict__ ctx,
     const int* __restrict__ block_tables, int bt_stride, int S, int H, int dkp, int dv, float scale, int window,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, const bf16_t* __restrict__ gate, long g_stride) {
   constexpr int TW = 4 * QT;           // tokens per workgroup
   constexpr int KP = KS_MAX * 32 + 8;  // LDS pitch of a key row (elements)
   constexpr int VP = 20;               // LDS pitch of a value dim's 16 tokens
@@ -550,7 +553,8 @@ __global__ __launch_bounds__(256) void latent_attn_lds_kernel(
 #pragma unroll
   for (int t = 0; t < QT; ++t) {
     if (tok0 + t >= nt) break;
-    const float inv = l[t] > 0.f ? 1.f / l[t] : 0.f;
+    float inv = l[t] > 0.f ? 1.f / l[t] : 0.f;
+    if (gate != nullptr) inv *= sigmoid_f(bf2f(gate[(long)(row0 + tok0 + t) * g_stride + head]));
     bf16_t* orow = out + ((long)(row0 + tok0 + t) * H + hg * 16 + c16) * dv;
 #pragma unroll
     for (int dt = 0; dt < DT_MAX; ++dt)
@@ -603,7 +607,7 @@ int k8sllm_hy_latent_queries(void* out, const void* q, long q_stride, const void
 int k8sllm_hy_latent_attention(void* out, const void* q, long q_stride, const void* k_cache, const void* v_cache,
                                const int* cu, const int* ctx, const int* seq_lens, const int* block_tables,
                                int bt_stride, int S, long T, int H, int dkp, int dv, int bs, float scale, int window,
-                               const float* sinks, int split, hipStream_t s) {
+                               const float* sinks, const void* gate, long g_stride, int split, hipStream_t s) {
   if (T <= 0) return 0;
   if (bs != 16 || dkp % 32 || dv % 16 || dkp > 320 || dv > 256 || q_stride % 8) return 1;
   const unsigned hgs = (unsigned)((H + 15) / 16);
@@ -617,7 +621,7 @@ int k8sllm_hy_latent_attention(void* out, const void* q, long q_stride, const vo
 #define K8SLLM_LL(KS, DT, QT)                                                                                          \
   hipLaunchKernelGGL((latent_attn_lds_kernel<KS, DT, QT>), grid, dim3(256), 0, s, (bf16_t*)out, (const bf16_t*)q,        \
                      q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, cu, ctx, block_tables, bt_stride, S, H,  \
-                     dkp, dv, scale, window, sinks)
+                     dkp, dv, scale, window, sinks, (const bf16_t*)gate, g_stride)
     if (dkp <= 128 && dv <= 128) {
       if (qt == 1) K8SLLM_LL(4, 8, 1); else K8SLLM_LL(4, 8, 2);
     } else {
@@ -633,7 +637,7 @@ int k8sllm_hy_latent_attention(void* out, const void* q, long q_stride, const vo
 #define K8SLLM_LA(KS, DT, NW, QT)                                                                                      \
   hipLaunchKernelGGL((latent_attn_mfma_kernel<KS, DT, NW, QT>), grid, dim3(64 * NW), 0, s, (bf16_t*)out,                \
                      (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, cu, ctx, seq_lens,     \
-                     block_tables, bt_stride, S, H, dkp, dv, scale, window, sinks)
+                     block_tables, bt_stride, S, H, dkp, dv, scale, window, sinks, (const bf16_t*)gate, g_stride)
 #define K8SLLM_LAS(KS, DT)                                            \
   if (nw == 8) K8SLLM_LA(KS, DT, 8, 1);                               \
   else if (nw == 4) K8SLLM_LA(KS, DT, 4, 1);                          \

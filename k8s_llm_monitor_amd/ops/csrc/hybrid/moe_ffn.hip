@@ -4,15 +4,18 @@
 //                 only, or (over_all) the chosen experts' probabilities in the softmax over all E
 //                 logits, not renormalised; one more row of Wr, if present, gives
 //                 gate = sigmoid(Wr[E] h) (the shared expert's)
-//   router_grouped  sigmoid scores; the experts form equal groups of neighbours, a group scores the sum of its
-//                 two largest, only the `keep` best groups' experts can be chosen; the K largest scores among
-//                 them, weights = score / (sum of the chosen + 1e-20) * scale
+//   router_grouped  sigmoid scores, or (soft) the softmax over all E logits; a choice by score (+ corr[e]); the
+//                 experts form equal groups of neighbours, a group counts as the sum of its two largest choice
+//                 scores (best2) or as its largest, only the `keep` best groups' experts can be chosen; the K
+//                 largest choice scores among them (lowest index wins a tie), weights = score / (sum of the
+//                 chosen + 1e-20) * scale (renorm), or score * scale
 //   grouped_gemm  Y[r] = W[e(r)] A[row(r)] over expert-sorted rows r (offsets / sorted_idx from the
 //                 counting sort), the A rows gathered on load; ACT 1 (SwiGLU): W = [gate rows ; up
 //                 rows] and Y = silu(gate) * up; ACT 2: Y = gelu(W A) (erf form); ACT 3: gated like 1 with the clamped unit
-//                 g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit).  64 x 64 tiles, fp32
-//                 accumulation.
-//   moe_combine   out[t] = sum_k w[t][k] Y[inv[t*K + k]] + gate[t] * shared[t]   (fp32; no gate: 1)
+//                 g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit); ACT 4: Y =
+//                 relu(W A)^2.  64 x 64 tiles, fp32 accumulation.
+//   moe_combine   out[t] = sum_k w[t][k] Y[inv[t*K + k]] + gate[t] * shared[t]   (fp32; no gate: 1); a chosen id
+//                 >= n_real is an identity expert, its Y is the layer's input h[t]
 #include "hy_common.h"
 
 namespace k8sllm {
@@ -117,25 +120,30 @@ __global__ __launch_bounds__(256) void hy_router_kernel(int* __restrict__ ids, f
   }
 }
 
-// Sigmoid router with a choice restricted to the best groups.  One workgroup per token computes the logits
-// (fp32 weights, h widened; NACC as in hy_router_kernel), thread 0 scores the groups and picks.
+// A choice restricted to the best groups.  One workgroup per token computes the logits (fp32 weights, h widened;
+// NACC as in hy_router_kernel); groups and experts are then ranked by counting what beats them, one thread
+// per group and per expert.
 template <typename T, int NACC>
 __global__ __launch_bounds__(256) void hy_router_grouped_kernel(int* __restrict__ ids, float* __restrict__ wts,
                                                                 const T* __restrict__ h, int d,
-                                                                const float* __restrict__ wr, int E, int K, int groups,
-                                                                int keep, float scale) {
-  __shared__ float sc[kMaxE];
-  __shared__ float gsc[kMaxE];
+                                                                const float* __restrict__ wr,
+                                                                const float* __restrict__ corr, int E, int K, int groups,
+                                                                int keep, float scale, int soft, int best2, int renorm) {
+  __shared__ float sc[kMaxE];   // scores: the weights come from these
+  __shared__ float ch[kMaxE];   // choice scores
+  __shared__ float gsc[kMaxE];  // groups
+  __shared__ int gok[kMaxE];
+  __shared__ int sel[kMaxK];
   __shared__ float part[4][NACC > 0 ? NACC : 1];
   const long t = blockIdx.x;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const T* x = h + t * d;
   if (NACC > 0) {  // at most NACC experts: h is read once, every expert's partial sum stays in a register
     float acc[NACC > 0 ? NACC : 1];
 #pragma unroll
     for (int e = 0; e < NACC; ++e) acc[e] = 0.f;
     if ((d & 7) == 0) {
-      for (int c = threadIdx.x * 8; c < d; c += 2048) {
+      for (int c = tid * 8; c < d; c += 2048) {
         float xv[8];
         load8(x + c, xv);
 #pragma unroll
@@ -149,7 +157,7 @@ __global__ __launch_bounds__(256) void hy_router_grouped_kernel(int* __restrict_
       }
     } else {
 #pragma unroll 4
-      for (int c = threadIdx.x; c < d; c += 256) {
+      for (int c = tid; c < d; c += 256) {
         const float xv = ldf(x + c);
 #pragma unroll
         for (int e = 0; e < NACC; ++e)
@@ -158,81 +166,84 @@ __global__ __launch_bounds__(256) void hy_router_grouped_kernel(int* __restrict_
     }
 #pragma unroll
     for (int e = 0; e < NACC; ++e) {
-      const float v = wave_sum(acc[e]);
+      const float v = wave_sum_dpp(acc[e]);
       if (lane == 0) part[wave][e] = v;
     }
     __syncthreads();
-    if (threadIdx.x < E) {
-      const int e = threadIdx.x;
-      sc[e] = 1.f / (1.f + expf(-(part[0][e] + part[1][e] + part[2][e] + part[3][e])));
-    }
+    if (tid < E) sc[tid] = part[0][tid] + part[1][tid] + part[2][tid] + part[3][tid];
   } else {
     for (int e = wave; e < E; e += 4) {
       const float* w = wr + (long)e * d;
       float a = 0.f;
       for (int c = lane; c < d; c += 64) a += ldf(x + c) * w[c];
-      a = wave_sum(a);
-      if (lane == 0) sc[e] = 1.f / (1.f + expf(-a));
+      a = wave_sum_dpp(a);
+      if (lane == 0) sc[e] = a;
+    }
+  }
+  __syncthreads();
+  if (wave == 0) {  // lane: experts lane, lane + 64, ..
+    float mx = -INFINITY, z = 0.f;
+    if (soft) {
+      for (int e = lane; e < E; e += 64) mx = fmaxf(mx, sc[e]);
+      mx = wave_max_dpp(mx);
+      for (int e = lane; e < E; e += 64) z += expf(sc[e] - mx);
+      z = wave_sum_dpp(z);
+    }
+    for (int e = lane; e < E; e += 64) {
+      const float v = soft ? expf(sc[e] - mx) / z : 1.f / (1.f + expf(-sc[e]));
+      const float c = corr != nullptr ? v + corr[e] : v;
+      sc[e] = v;
+      ch[e] = c == c ? c : -INFINITY;  // ranks are a strict order whatever the input: every slot gets an expert
     }
   }
   __syncthreads();
   const int per = E / groups;
-  if (threadIdx.x < groups) {  // a group's score: its two largest scores (one expert per group: its score)
-    float m1 = -1.f, m2 = -1.f;
-    for (int e = threadIdx.x * per; e < (threadIdx.x + 1) * per; ++e) {
-      const float v = sc[e];
-      if (v > m1) {
-        m2 = m1;
-        m1 = v;
-      } else if (v > m2) {
-        m2 = v;
-      }
-    }
-    gsc[threadIdx.x] = per > 1 ? m1 + m2 : m1;
-  }
-  __syncthreads();
-  if (threadIdx.x == 0) {
-    if (keep < groups) {  // scores of experts outside the best groups drop below every sigmoid
-      for (int k = 0; k < keep; ++k) {
-        int best = -1;
-        float bv = -INFINITY;
-        for (int g = 0; g < groups; ++g)
-          if (gsc[g] > bv) {
-            bv = gsc[g];
-            best = g;
-          }
-        gsc[best] = -INFINITY;  // marks a kept group
-      }
-    }
-    int sel[kMaxK];
-    float val[kMaxK];
-    float z = 0.f;
-    for (int k = 0; k < K; ++k) {
-      int best = -1;
-      float bv = -INFINITY;
-      for (int e = 0; e < E; ++e) {
-        if (keep < groups && gsc[e / per] != -INFINITY) continue;
-        bool taken = false;
-        for (int j = 0; j < k; ++j) taken |= sel[j] == e;
-        if (!taken && (best < 0 || sc[e] > bv)) {
-          bv = sc[e];
-          best = e;
+  if (keep < groups) {
+    if (tid < groups) {
+      float m1 = -INFINITY, m2 = -INFINITY;
+      for (int e = tid * per; e < (tid + 1) * per; ++e) {
+        const float v = ch[e];
+        if (v > m1) {
+          m2 = m1;
+          m1 = v;
+        } else if (v > m2) {
+          m2 = v;
         }
       }
-      sel[k] = best;
-      val[k] = bv;
-      z += bv;
+      gsc[tid] = best2 && per > 1 ? m1 + m2 : m1;
     }
-    for (int k = 0; k < K; ++k) {
-      ids[t * K + k] = sel[k];
-      wts[t * K + k] = val[k] / (z + 1e-20f) * scale;
+    __syncthreads();
+    if (tid < groups) {
+      const float v = gsc[tid];
+      int rank = 0;
+      for (int g = 0; g < groups; ++g) rank += (gsc[g] > v || (gsc[g] == v && g < tid)) ? 1 : 0;
+      gok[tid] = rank < keep;
     }
+    __syncthreads();
+  }
+  if (tid < E && (keep == groups || gok[tid / per])) {
+    const float v = ch[tid];
+    int rank = 0;
+    for (int e = 0; e < E; ++e)
+      if (keep == groups || gok[e / per]) rank += (ch[e] > v || (ch[e] == v && e < tid)) ? 1 : 0;
+    if (rank < K) sel[rank] = tid;
+  }
+  __syncthreads();
+  if (tid < K) {
+    float z = 1.f;
+    if (renorm) {
+      z = 1e-20f;
+      for (int k = 0; k < K; ++k) z += sc[sel[k]];
+    }
+    ids[t * K + tid] = sel[tid];
+    wts[t * K + tid] = sc[sel[tid]] / z * scale;
   }
 }
 
 constexpr int TM = 64, TN = 64, TK = 16;
 
 __device__ __forceinline__ float gelu_erf_f(float z) { return 0.5f * z * (1.f + erff(z * 0.70710678118654752f)); }
+__device__ __forceinline__ float relu_sq_f(float z) { return z > 0.f ? z * z : 0.f; }
 __device__ __forceinline__ float clamped_unit_f(float g, float u, float limit) {
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
@@ -322,10 +333,10 @@ __global__ __launch_bounds__(256) void hy_grouped_gemm_kernel(T* __restrict__ Y,
         stf(&gq, v);
         stf(&uq, accu[i][j]);
         v = ACT == 3 ? clamped_unit_f(ldf(&gq), ldf(&uq), limit) : silu_f(ldf(&gq)) * ldf(&uq);
-      } else if (ACT == 2) {  // the projection is rounded to the storage dtype before the activation
+      } else if (ACT == 2 || ACT == 4) {  // the projection is rounded to the storage dtype before the activation
         T gq;
         stf(&gq, v);
-        v = gelu_erf_f(ldf(&gq));
+        v = ACT == 2 ? gelu_erf_f(ldf(&gq)) : relu_sq_f(ldf(&gq));
       }
       stf(Y + (long)r * N + n, v);
     }
@@ -397,22 +408,47 @@ __global__ __launch_bounds__(64) void hy_grouped_gemm_mfma_kernel(bf16_t* __rest
       if (ACT == 3) v = clamped_unit_f(bf2f(f2bf(v)), bf2f(f2bf(accu[t][i])), limit);
       else if (SWIGLU) v = silu_f(bf2f(f2bf(v))) * bf2f(f2bf(accu[t][i]));
       else if (ACT == 2) v = gelu_erf_f(bf2f(f2bf(v)));
+      else if (ACT == 4) v = relu_sq_f(bf2f(f2bf(v)));
       Y[(long)r * N + n] = f2bf(v);
     }
   }
 }
 
-template <typename T>
+template <typename T, bool V8>
 __global__ __launch_bounds__(256) void hy_combine_kernel(float* __restrict__ out, const T* __restrict__ ys,
                                                          const int* __restrict__ inv, const float* __restrict__ wts,
                                                          const T* __restrict__ shared, const float* __restrict__ gate,
-                                                         int K, int d) {
+                                                         const int* __restrict__ ids, const T* __restrict__ h,
+                                                         int n_real, int K, int d) {
   const long t = blockIdx.x;
-  for (int c = threadIdx.x; c < d; c += 256) {
-    float a = 0.f;
-    for (int k = 0; k < K; ++k) a += wts[t * K + k] * ldf(ys + (long)inv[t * K + k] * d + c);
-    if (shared != nullptr) a += (gate != nullptr ? gate[t] : 1.f) * ldf(shared + t * d + c);
-    out[t * d + c] = a;
+  // the row that slot k of this token adds (wave-uniform)
+  auto source = [&](int k) {
+    return ids != nullptr && ids[t * K + k] >= n_real ? h + t * d : ys + (long)inv[t * K + k] * d;
+  };
+  const float gs = gate != nullptr ? gate[t] : 1.f;
+  if constexpr (V8) {
+    for (int c = threadIdx.x * 8; c < d; c += 2048) {
+      float a[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, v[8];
+      for (int k = 0; k < K; ++k) {
+        const float wk = wts[t * K + k];
+        load8(source(k) + c, v);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) a[i] += wk * v[i];
+      }
+      if (shared != nullptr) {
+        load8(shared + t * d + c, v);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) a[i] += gs * v[i];
+      }
+      store8(out + t * d + c, a);
+    }
+  } else {
+    for (int c = threadIdx.x; c < d; c += 256) {
+      float a = 0.f;
+      for (int k = 0; k < K; ++k) a += wts[t * K + k] * ldf(source(k) + c);
+      if (shared != nullptr) a += gs * ldf(shared + t * d + c);
+      out[t * d + c] = a;
+    }
   }
 }
 
@@ -438,15 +474,16 @@ int k8sllm_hy_router(int* ids, float* wts, float* gate, const void* h, long T, i
   return (int)hipGetLastError();
 }
 
-int k8sllm_hy_router_grouped(int* ids, float* wts, const void* h, long T, int d, const float* wr, int E, int K,
-                             int groups, int keep, float scale, int f32, hipStream_t s) {
+int k8sllm_hy_router_grouped(int* ids, float* wts, const void* h, long T, int d, const float* wr, const float* corr, int E,
+                             int K, int groups, int keep, float scale, int soft, int best2, int renorm, int f32,
+                             hipStream_t s) {
   if (T <= 0) return 0;
   if (E > kMaxE || K > kMaxK || K < 1 || groups < 1 || E % groups || keep < 1 || keep > groups ||
       K > keep * (E / groups))
     return -1;
 #define K8SLLM_RG(T_, NACC)                                                                                        \
-  hipLaunchKernelGGL((hy_router_grouped_kernel<T_, NACC>), dim3(T), dim3(256), 0, s, ids, wts, (const T_*)h, d, wr, E, K, \
-                     groups, keep, scale)
+  hipLaunchKernelGGL((hy_router_grouped_kernel<T_, NACC>), dim3(T), dim3(256), 0, s, ids, wts, (const T_*)h, d, wr, corr, \
+                     E, K, groups, keep, scale, soft, best2, renorm)
   if (f32) {
     if (E <= 8) K8SLLM_RG(float, 8); else if (E <= 16) K8SLLM_RG(float, 16); else K8SLLM_RG(float, 0);
   } else {
@@ -461,7 +498,7 @@ int k8sllm_hy_grouped_gemm(void* Y, const void* A, const void* W, const int* off
                            int E, long rows, int N, int Kd, long w_es, int act, int il, int f32, int mfma, float limit,
                            hipStream_t s) {
   if (rows <= 0) return 0;
-  if (act < 0 || act > 3) return -1;
+  if (act < 0 || act > 4) return -1;
   const bool swiglu = act == 1;
   if (il && (!swiglu || N % 64)) return -1;
   if (!f32 && mfma && Kd % 32 == 0) {
@@ -476,6 +513,8 @@ int k8sllm_hy_grouped_gemm(void* Y, const void* A, const void* W, const int* off
       if (few) K8SLLM_GM(3, 1); else K8SLLM_GM(3, 4);
     } else if (act == 2) {
       if (few) K8SLLM_GM(2, 1); else K8SLLM_GM(2, 4);
+    } else if (act == 4) {
+      if (few) K8SLLM_GM(4, 1); else K8SLLM_GM(4, 4);
     } else {
       if (few) K8SLLM_GM(0, 1); else K8SLLM_GM(0, 4);
     }
@@ -488,24 +527,31 @@ int k8sllm_hy_grouped_gemm(void* Y, const void* A, const void* W, const int* off
                      sorted_idx, div, E, N, Kd, w_es, il, limit)
   if (f32) {
     if (swiglu) K8SLLM_GG(float, 1); else if (act == 3) K8SLLM_GG(float, 3); else if (act == 2) K8SLLM_GG(float, 2);
+    else if (act == 4) K8SLLM_GG(float, 4);
     else K8SLLM_GG(float, 0);
   } else {
     if (swiglu) K8SLLM_GG(bf16_t, 1); else if (act == 3) K8SLLM_GG(bf16_t, 3); else if (act == 2) K8SLLM_GG(bf16_t, 2);
+    else if (act == 4) K8SLLM_GG(bf16_t, 4);
     else K8SLLM_GG(bf16_t, 0);
   }
 #undef K8SLLM_GG
   return (int)hipGetLastError();
 }
 
+// ids, h (may be absent): chosen ids >= n_real take the row of h
 int k8sllm_hy_combine(float* out, const void* ys, const int* inv, const float* wts, const void* shared,
-                      const float* gate, long T, int K, int d, int f32, hipStream_t s) {
+                      const float* gate, const int* ids, const void* h, int n_real, long T, int K, int d, int f32,
+                      hipStream_t s) {
   if (T <= 0) return 0;
-  if (f32)
-    hipLaunchKernelGGL(hy_combine_kernel<float>, dim3(T), dim3(256), 0, s, out, (const float*)ys, inv, wts,
-                       (const float*)shared, gate, K, d);
-  else
-    hipLaunchKernelGGL(hy_combine_kernel<bf16_t>, dim3(T), dim3(256), 0, s, out, (const bf16_t*)ys, inv, wts,
-                       (const bf16_t*)shared, gate, K, d);
+#define K8SLLM_CB(T_, V8)                                                                                              \
+  hipLaunchKernelGGL((hy_combine_kernel<T_, V8>), dim3((unsigned)T), dim3(256), 0, s, out, (const T_*)ys, inv, wts,        \
+                     (const T_*)shared, gate, ids, (const T_*)h, n_real, K, d)
+  if (f32) {
+    if (d % 8 == 0) K8SLLM_CB(float, true); else K8SLLM_CB(float, false);
+  } else {
+    if (d % 8 == 0) K8SLLM_CB(bf16_t, true); else K8SLLM_CB(bf16_t, false);
+  }
+#undef K8SLLM_CB
   return (int)hipGetLastError();
 }
 }

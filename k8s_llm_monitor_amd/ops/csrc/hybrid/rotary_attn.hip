@@ -14,12 +14,46 @@
 //                  the turn, no weight; norm == 0 none.  v_from_k: the row has no value columns and the value
 //                  pages take the keys as projected (before norm and turn; dv == dk).  One wave per head, the
 //                  head staged in LDS as fp32; the token's sines and cosines are evaluated once for all its
-//                  heads; the result is rounded to the activation dtype once.
+//                  heads; the result is rounded to the activation dtype once.  Without rotation, at head
+//                  dims 64 / 128 / 256, a lane group per head with wide accesses (head_norm_cache_kernel).
 #include "hy_common.h"
 
 namespace k8sllm {
 
 constexpr int kMaxHeadDim = 1024;
+
+// The norm-only form (norm == 1, nothing turns, head dims of 8 LPH entries): LPH neighbouring lanes hold a head,
+// 16 / 32-byte accesses, the mean square by lane adds; a workgroup takes one row.
+template <typename T, int LPH>
+__global__ __launch_bounds__(256) void head_norm_cache_kernel(T* __restrict__ qkv, long stride, int Hq, int G, int dv,
+                                                              const float* __restrict__ qw, const float* __restrict__ kw,
+                                                              float eps, const float* __restrict__ q_scale,
+                                                              T* __restrict__ k_cache, T* __restrict__ v_cache,
+                                                              const int* __restrict__ slots, int bs) {
+  constexpr int dk = 8 * LPH;
+  const long t = blockIdx.x;
+  T* row = qkv + t * stride;
+  const int nk = G * dk, nv = G * dv, nh = Hq + G, c = 8 * (threadIdx.x % LPH);
+  const long slot = (slots != nullptr && k_cache != nullptr) ? slots[t] : -1;
+  for (int h0 = 0; h0 < nh; h0 += 256 / LPH) {  // every lane takes part in the adds; dead heads repeat the last one
+    const int h = h0 + threadIdx.x / LPH, hc = min(h, nh - 1);
+    T* hd = row + (long)hc * dk + c;
+    float x[8], g[8], ss = 0.f;
+    load8(hd, x);
+    load8((hc >= Hq ? kw : qw) + c, g);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
+    float inv = 1.0f / sqrtf(lanes_sum<LPH>(ss) / (float)dk + eps);
+    if (h >= nh) continue;
+    if (h < Hq && q_scale != nullptr) inv *= q_scale[h];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) x[i] *= inv * g[i];
+    store8(hd, x);
+    if (h >= Hq && slot >= 0) store8(k_cache + slot * (long)nk + (long)(h - Hq) * dk + c, x);
+  }
+  if (slot >= 0)
+    for (int i = threadIdx.x; i < nv; i += 256) v_cache[((slot / bs) * nv + i) * bs + slot % bs] = row[(long)nh * dk + i];
+}
 
 template <typename T>
 __global__ __launch_bounds__(256) void rotary_norm_cache_kernel(T* __restrict__ qkv, long stride, int Hq, int G, int dk,
@@ -163,14 +197,27 @@ int k8sllm_hy_rotary_cache(void* qkv, long stride, long T, int Hq, int G, int dk
   return (int)hipGetLastError();
 }
 
+// vec: 8-wide accesses of the rows are aligned (checked by the caller)
 int k8sllm_hy_rotary_norm_cache(void* qkv, long stride, long T, int Hq, int G, int dk, int dv, const int* positions,
                                 const float* freq, int nf, int pairs, int norm, const float* qw, const float* kw,
                                 float eps, const float* q_scale, void* k_cache, void* v_cache, const int* slots, int bs,
-                                int v_from_k, int f32, hipStream_t s) {
+                                int v_from_k, int vec, int f32, hipStream_t s) {
   if (T <= 0) return 0;
   if (nf < 0 || 2 * nf > dk || Hq < 1 || G < 1 || dk > kMaxHeadDim || norm < 0 || norm > 2) return -1;
   if (norm == 1 && (qw == nullptr || kw == nullptr)) return -1;
   if (v_from_k && dv != dk) return -1;
+  if (nf == 0 && norm == 1 && !v_from_k && vec && (dk == 64 || dk == 128 || dk == 256)) {
+#define K8SLLM_HN(T_, LPH)                                                                                            \
+  hipLaunchKernelGGL((head_norm_cache_kernel<T_, LPH>), dim3(T), dim3(256), 0, s, (T_*)qkv, stride, Hq, G, dv, qw, kw, eps, \
+                     q_scale, (T_*)k_cache, (T_*)v_cache, slots, bs)
+    if (f32) {
+      if (dk == 64) K8SLLM_HN(float, 8); else if (dk == 128) K8SLLM_HN(float, 16); else K8SLLM_HN(float, 32);
+    } else {
+      if (dk == 64) K8SLLM_HN(bf16_t, 8); else if (dk == 128) K8SLLM_HN(bf16_t, 16); else K8SLLM_HN(bf16_t, 32);
+    }
+#undef K8SLLM_HN
+    return (int)hipGetLastError();
+  }
   const size_t lds = (4 * (size_t)dk + 2 * (size_t)nf) * sizeof(float);
   if (f32)
     hipLaunchKernelGGL(rotary_norm_cache_kernel<float>, dim3(T), dim3(256), lds, s, (float*)qkv, stride, Hq, G, dk, dv,

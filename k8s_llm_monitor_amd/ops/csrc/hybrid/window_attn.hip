@@ -6,7 +6,10 @@
 // dim's BS tokens contiguous: the layout the PV products read along); a sequence's page list is a row of
 // block_tables.  Row at position p sees positions max(0, p - window + 1) .. p (window 0: 0 .. p), or with
 // ``chunked`` the positions from its chunk's first on: floor(p / window) * window .. p (chunks are counted
-// from position 0 of the sequence).  cap > 0: a score s (after the scale) becomes cap * tanh(s / cap).
+// from position 0 of the sequence).  keep > 0 (window form): the first ``keep`` positions of the sequence stay
+// visible to every later row besides its window.  cap > 0: a score s (after the scale) becomes cap * tanh(s / cap).
+// gate (optional, rows g_stride apart, one logit per query head): a head's output is multiplied by
+// sigmoid(gate[row][head]) before its one rounding.
 // The sink is one more softmax term with no value and a fixed score - 0, or a learned unscaled logit
 // per query head (sinks[h]): the running maximum starts at that score and the running denominator at 1.  Scores, weights and the output accumulation are fp32.
 #include "hy_common.h"
@@ -64,9 +67,9 @@ __global__ __launch_bounds__(256) void qk_norm_cache_kernel(T* __restrict__ qkv,
 template <typename T>
 __device__ __forceinline__ void attend_wave(T* __restrict__ out_row, const T* __restrict__ q_row,
                                             const T* __restrict__ k_cache, const T* __restrict__ v_cache,
-                                            const int* __restrict__ bt, int lo, int hi, int g, int G, int dk, int dv,
-                                            int bs, float scale, float cap, int sink, float sink_z, float* q_s,
-                                            float* p_s) {
+                                            const int* __restrict__ bt, int lo, int hi, int keep, int g, int G,
+                                            int dk, int dv, int bs, float scale, float cap, int sink, float sink_z,
+                                            float gate, float* q_s, float* p_s) {
   const int lane = threadIdx.x & 63;
   for (int c = lane; c < dk; c += 64) q_s[c] = ldf(q_row + c) * scale;
   __syncthreads();  // one wave per workgroup: orders the LDS writes before the other lanes' reads
@@ -75,37 +78,41 @@ __device__ __forceinline__ void attend_wave(T* __restrict__ out_row, const T* __
 #pragma unroll
   for (int c = 0; c < kGenVC; ++c) acc[c] = 0.f;
   const long krow = (long)G * dk, vrow = (long)G * dv;
-  for (int j0 = lo; j0 < hi; j0 += 64) {
-    const int j = j0 + lane;
+  // visible key number i is position i below the kept ones' end, then the window's positions from lo on
+  if (keep >= lo) lo = keep = 0;  // nothing lies between them
+  const int nvis = keep + hi - lo, skip = lo - keep;
+  for (int i0 = 0; i0 < nvis; i0 += 64) {
+    const int iv = i0 + lane, j = iv < keep ? iv : iv + skip;
+    const bool live = iv < nvis;
     float s = -INFINITY;
-    if (j < hi) {
+    if (live) {
       const T* kp = k_cache + ((long)bt[j / bs] * bs + j % bs) * krow + (long)g * dk;
       float a = 0.f;
       for (int c = 0; c < dk; ++c) a += q_s[c] * ldf(kp + c);
       s = cap > 0.f ? cap * tanhf(a / cap) : a;
     }
     const float mt = fmaxf(m, wave_max_dpp(s));
-    const float p = j < hi ? expf(s - mt) : 0.f;
+    const float p = live ? expf(s - mt) : 0.f;
     const float alpha = expf(m - mt);  // m = -inf only before the first key (no sink): exp(-inf) = 0
     l = l * alpha + wave_sum_dpp(p);
     m = mt;
     __syncthreads();  // the previous tile's reads of p_s are done
     p_s[lane] = p;
     __syncthreads();
-    const int n = min(64, hi - j0);
+    const int n = min(64, nvis - i0);
 #pragma unroll
     for (int c = 0; c < kGenVC; ++c) {
       const int dcol = lane + 64 * c;
       float a = acc[c] * alpha;
       if (dcol < dv)
         for (int i = 0; i < n; ++i) {
-          const int jj = j0 + i;
+          const int jj = i0 + i < keep ? i0 + i : i0 + i + skip;
           a += p_s[i] * ldf(v_cache + ((long)bt[jj / bs] * vrow + (long)g * dv + dcol) * bs + jj % bs);
         }
       acc[c] = a;
     }
   }
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  const float inv = l > 0.f ? gate / l : 0.f;
 #pragma unroll
   for (int c = 0; c < kGenVC; ++c) {
     const int dcol = lane + 64 * c;
@@ -120,8 +127,9 @@ __global__ __launch_bounds__(64) void window_prefill_kernel(T* __restrict__ out,
                                                             const int* __restrict__ cu, const int* __restrict__ ctx,
                                                             const int* __restrict__ block_tables, int bt_stride, int S,
                                                             int Hq, int G, int dk, int dv, int bs, float scale,
-                                                            int window, int chunked, float cap, int sink,
-                                                            const float* __restrict__ sinks) {
+                                                            int window, int chunked, int keep, float cap, int sink,
+                                                            const float* __restrict__ sinks,
+                                                            const T* __restrict__ gate, long g_stride) {
   __shared__ float q_s[kGenDK];
   __shared__ float p_s[64];
   const int r = blockIdx.x, h = blockIdx.y;
@@ -129,8 +137,9 @@ __global__ __launch_bounds__(64) void window_prefill_kernel(T* __restrict__ out,
   const int p = ctx[s] + r - cu[s];
   const int lo = first_key(p, window, chunked);
   attend_wave<T>(out + (long)r * Hq * dv + (long)h * dv, qkv + (long)r * q_stride + (long)h * dk, k_cache, v_cache,
-                 block_tables + (long)s * bt_stride, lo, p + 1, h / (Hq / G), G, dk, dv, bs, scale, cap, sink,
-                 sinks != nullptr ? sinks[h] : 0.f, q_s, p_s);
+                 block_tables + (long)s * bt_stride, lo, p + 1, keep, h / (Hq / G), G, dk, dv, bs, scale, cap, sink,
+                 sinks != nullptr ? sinks[h] : 0.f, gate != nullptr ? sigmoid_f(ldf(gate + (long)r * g_stride + h)) : 1.f,
+                 q_s, p_s);
 }
 
 template <typename T>
@@ -140,7 +149,9 @@ __global__ __launch_bounds__(64) void window_decode_kernel(T* __restrict__ out, 
                                                            const int* __restrict__ block_tables, int bt_stride,
                                                            const int* __restrict__ seq_lens, int Hq, int G, int dk,
                                                            int dv, int bs, float scale, int window, int chunked,
-                                                           float cap, int sink, const float* __restrict__ sinks) {
+                                                           int keep, float cap, int sink,
+                                                           const float* __restrict__ sinks,
+                                                           const T* __restrict__ gate, long g_stride) {
   __shared__ float q_s[kGenDK];
   __shared__ float p_s[64];
   const int b = blockIdx.x, h = blockIdx.y;
@@ -152,7 +163,8 @@ __global__ __launch_bounds__(64) void window_decode_kernel(T* __restrict__ out, 
   }
   const int lo = first_key(n - 1, window, chunked);
   attend_wave<T>(o, qkv + (long)b * q_stride + (long)h * dk, k_cache, v_cache, block_tables + (long)b * bt_stride, lo,
-                 n, h / (Hq / G), G, dk, dv, bs, scale, cap, sink, sinks != nullptr ? sinks[h] : 0.f, q_s, p_s);
+                 n, keep, h / (Hq / G), G, dk, dv, bs, scale, cap, sink, sinks != nullptr ? sinks[h] : 0.f,
+                 gate != nullptr ? sigmoid_f(ldf(gate + (long)b * g_stride + h)) : 1.f, q_s, p_s);
 }
 
 // bf16 decode with 16-byte loads, 16-token pages: one workgroup (NW = 8 waves; 4 for 8 query heads
@@ -169,8 +181,9 @@ __global__ __launch_bounds__(64 * NW) void window_decode_vec_kernel(bf16_t* __re
                                                                 const bf16_t* __restrict__ v_cache,
                                                                 const int* __restrict__ block_tables, int bt_stride,
                                                                 const int* __restrict__ seq_lens, int Hq, int G, int dk,
-                                                                int dv, float scale, int window, int chunked, float cap,
-                                                                int sink, const float* __restrict__ sinks) {
+                                                                int dv, float scale, int window, int chunked, int keep,
+                                                                float cap, int sink, const float* __restrict__ sinks,
+                                                                const bf16_t* __restrict__ gate, long g_stride) {
   constexpr int bs = 16;
   __shared__ __attribute__((aligned(16))) float q_s[R * kMaxDK];
   __shared__ __attribute__((aligned(16))) float p_s[NW][R][64];
@@ -200,9 +213,13 @@ __global__ __launch_bounds__(64 * NW) void window_decode_vec_kernel(bf16_t* __re
     for (int c = 0; c < kMaxVC; ++c) acc[r][c] = 0.f;
   }
   const long krs = (long)G * dk;
-  for (int j0 = (lo & ~63) + 64 * wave; j0 < n; j0 += 64 * NW) {
+  // the tiles that hold kept keys (kt of them, from position 0), then the window's from w0 on
+  const int kf = min(keep, n), kt = (kf + 63) >> 6, w0 = max(kt, lo >> 6);
+  for (int it = wave;; it += NW) {
+    const int j0 = 64 * (it < kt ? it : w0 + it - kt);
+    if (j0 >= n) break;
     const int j = j0 + lane;
-    const bool valid = j >= lo && j < n;
+    const bool valid = (j >= lo || j < keep) && j < n;
     float sc[R];
 #pragma unroll
     for (int r = 0; r < R; ++r) sc[r] = 0.f;
@@ -232,7 +249,8 @@ __global__ __launch_bounds__(64 * NW) void window_decode_vec_kernel(bf16_t* __re
     }
     // value loads of the tile's pages go out before the softmax arithmetic: 2 x 16 bytes per page and
     // 64 dims (pages at or past the sequence's end are not touched: their weights are zero)
-    const int npg = min(4, (n - j0 + bs - 1) / bs);
+    const int jend = j0 + 64 > lo ? n : kf;  // a tile of kept keys alone: the pages behind them are not needed
+    const int npg = min(4, (jend - j0 + bs - 1) / bs);
     uint4 vq[4][kMaxVC][2];
 #pragma unroll
     for (int pg = 0; pg < 4; ++pg)
@@ -306,7 +324,8 @@ __global__ __launch_bounds__(64 * NW) void window_decode_vec_kernel(bf16_t* __re
       L += ml_s[w][r][1] * f;
       val += acc_s[w][r][dcol] * f;
     }
-    o[c] = f2bf(L > 0.f ? val / L : 0.f);
+    const float gt = gate != nullptr ? sigmoid_f(bf2f(gate[(long)b * g_stride + g * R + r])) : 1.f;
+    o[c] = f2bf(L > 0.f ? val / L * gt : 0.f);
   }
 }
 
@@ -330,7 +349,8 @@ __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
     bf16_t* __restrict__ out, const bf16_t* __restrict__ qkv, long q_stride, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int* __restrict__ cu, const int* __restrict__ ctx,
     const int* __restrict__ block_tables, int bt_stride, int S, int Hq, int G, float scale, int window,
-    int chunked, float cap, int sink, const float* __restrict__ sinks) {
+    int chunked, int keep, float cap, int sink, const float* __restrict__ sinks, const bf16_t* __restrict__ gate,
+    long g_stride) {
   // pages hold 16 tokens; scores live in the base-2 domain (scale * log2 e folded in) so that every
   // exponential is one v_exp_f32
   const float sc2 = scale * 1.44269504088896341f;
@@ -379,7 +399,13 @@ __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
   // per 16 dims - no LDS, no barrier.
   const bf16_t* kbase = k_cache + (long)g * DK + 8 * quad;
   const bf16_t* vbase = v_cache + ((long)g * DV + c16) * 16 + 4 * quad;
-  const int jfirst = lo_t & ~15;
+  // key tiles: those that hold kept keys (up to kend), then the window's from wfirst on
+  const int kend = (min(keep, hi) + 15) & ~15, wfirst = max(kend, lo_t & ~15);
+  const int jfirst = kend > 0 ? 0 : wfirst;
+  auto next_tile = [&](int j) {
+    j += 16;
+    return j >= kend && j < wfirst ? wfirst : j;
+  };
   int pg_n = bt[jfirst >> 4];
   bf16x8 kf_n[DK / 32];
   s16x4 vf_n[DV / 16];
@@ -392,22 +418,23 @@ __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
     for (int dt = 0; dt < DV / 16; ++dt) vf_n[dt] = *reinterpret_cast<const s16x4*>(vpg + dt * 256);
   };
   issue(jfirst);
-  pg_n = bt[min(jfirst + 16, hi - 1) >> 4];
-  for (int j0 = jfirst; j0 < hi; j0 += 16) {
+  int j1 = next_tile(jfirst);
+  pg_n = bt[min(j1, hi - 1) >> 4];
+  for (int j0 = jfirst; j0 < hi; j0 = j1, j1 = next_tile(j1)) {
     bf16x8 kf[DK / 32];
     s16x4 vf[DV / 16];
 #pragma unroll
     for (int ks = 0; ks < DK / 32; ++ks) kf[ks] = kf_n[ks];
 #pragma unroll
     for (int dt = 0; dt < DV / 16; ++dt) vf[dt] = vf_n[dt];
-    if (j0 + 16 < hi) {
-      issue(j0 + 16);
-      pg_n = bt[min(j0 + 32, hi - 1) >> 4];
+    if (j1 < hi) {
+      issue(j1);
+      pg_n = bt[min(next_tile(j1), hi - 1) >> 4];
     }
     s16x4 pb[QT];
     float alpha[QT];
     bool rescale[QT];
-    const bool inner = j0 >= lo_max && j0 + 15 <= p0;
+    const bool inner = (j0 >= lo_max || j0 + 15 < keep) && j0 + 15 <= p0;  // wave-uniform: every row sees every key
 #pragma unroll
     for (int t = 0; t < QT; ++t) {
       f32x4 sacc = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -422,7 +449,7 @@ __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
             const int j = j0 + 4 * quad + i;
-            if (j < my_lo[t] || j > my_p[t]) pv[i] = 0.f;
+            if ((j < my_lo[t] && j >= keep) || j > my_p[t]) pv[i] = 0.f;
           }
         }
         l[t] += (pv[0] + pv[1]) + (pv[2] + pv[3]);
@@ -430,20 +457,24 @@ __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
         for (int i = 0; i < 4; ++i) pb[t][i] = (short)f2bf(pv[i]);
         continue;
       }
-      float sv[4], tmax = -INFINITY;
+      float sv[4];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {  // sacc[i]: key j0 + 4 quad + i, query 16 t + c16
-        const int j = j0 + 4 * quad + i;
-        sv[i] = (q_live[t] && j >= my_lo[t] && j <= my_p[t]) ? (CAP ? cap2 * tanh_exp2(sacc[i] * icap) : sacc[i] * sc2) : -INFINITY;
-        tmax = fmaxf(tmax, sv[i]);
+      for (int i = 0; i < 4; ++i) sv[i] = CAP ? cap2 * tanh_exp2(sacc[i] * icap) : sacc[i] * sc2;
+      if (!inner) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {  // sacc[i]: key j0 + 4 quad + i, query 16 t + c16
+          const int j = j0 + 4 * quad + i;
+          if ((j < my_lo[t] && j >= keep) || j > my_p[t]) sv[i] = -INFINITY;
+        }
       }
-      tmax = xor32_max_f(xor16_max(tmax));
+      const float tmax = xor32_max_f(xor16_max(fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3]))));
       const float mn = fmaxf(m[t], tmax);
-      alpha[t] = m[t] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m[t] - mn);
+      const float mb = mn == -INFINITY ? 0.f : mn;  // no live key yet: exp2(-inf - 0) = 0
+      alpha[t] = __builtin_amdgcn_exp2f(m[t] - mb);
       float ps = 0.f;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const float pv = sv[i] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(sv[i] - mn);
+        const float pv = __builtin_amdgcn_exp2f(sv[i] - mb);
         ps += pv;
         pb[t][i] = (short)f2bf(pv);
       }
@@ -474,7 +505,8 @@ __global__ __launch_bounds__(64) void window_prefill_mfma_kernel(
   for (int t = 0; t < QT; ++t) {
     if (CAP == 2) l[t] = xor32_sum_f(xor16_sum(l[t]));
     if (!q_live[t]) continue;  // oacc[t][dt][i] = O[q = 16 t + c16][d = 16 dt + 4 quad + i]
-    const float inv = l[t] > 0.f ? 1.f / l[t] : 0.f;
+    float inv = l[t] > 0.f ? 1.f / l[t] : 0.f;
+    if (gate != nullptr) inv *= sigmoid_f(bf2f(gate[(long)(row0 + 16 * t + c16) * g_stride + h]));
     bf16_t* orow = out + (long)(row0 + 16 * t + c16) * Hq * DV + (long)h * DV;
 #pragma unroll
     for (int dt = 0; dt < DV / 16; ++dt) {
@@ -506,9 +538,11 @@ int k8sllm_hy_qk_norm_cache(void* qkv, long stride, const float* qw, const float
 
 int k8sllm_hy_window_prefill(void* out, const void* qkv, long q_stride, const void* k_cache, const void* v_cache,
                              const int* cu, const int* ctx, const int* block_tables, int bt_stride, int S, long T,
-                             int Hq, int G, int dk, int dv, int bs, float scale, int window, int chunked, float cap,
-                             int sink, const float* sinks, int f32, int mfma, hipStream_t s) {
+                             int Hq, int G, int dk, int dv, int bs, float scale, int window, int chunked, int keep,
+                             float cap, int sink, const float* sinks, const void* gate, long g_stride, int f32, int mfma,
+                             hipStream_t s) {
   if (T <= 0 || S <= 0) return 0;
+  if (keep < 0 || (keep > 0 && (chunked || window <= 0))) return -1;
   if (dk > kGenDK || dv > 64 * kGenVC || G < 1 || Hq % G) return -1;
   // bf16 with matrix-core head sizes and 16-byte aligned rows: the MFMA kernel
   if (!f32 && mfma && bs == 16 && q_stride % 8 == 0 && (dk == 64 || dk == 128) && (dv == 64 || dv == 128)) {
@@ -519,7 +553,7 @@ int k8sllm_hy_window_prefill(void* out, const void* qkv, long q_stride, const vo
 #define K8SLLM_WPC(DK, DV, QT, CAP)                                                                                    \
   hipLaunchKernelGGL((window_prefill_mfma_kernel<DK, DV, QT, CAP>), grid, dim3(64), 0, s, (bf16_t*)out,                 \
                      (const bf16_t*)qkv, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, cu, ctx,             \
-                     block_tables, bt_stride, S, Hq, G, scale, window, chunked, cap, sink, sinks)
+                     block_tables, bt_stride, S, Hq, G, scale, window, chunked, keep, cap, sink, sinks, (const bf16_t*)gate, g_stride)
 #define K8SLLM_WP(DK, DV, QT) \
   if (cap > 0.f && cap <= kMaxCapPlain && !sink) K8SLLM_WPC(DK, DV, QT, 2); \
   else if (cap > 0.f) K8SLLM_WPC(DK, DV, QT, 1); \
@@ -541,19 +575,20 @@ int k8sllm_hy_window_prefill(void* out, const void* qkv, long q_stride, const vo
   if (f32)
     hipLaunchKernelGGL(window_prefill_kernel<float>, dim3(T, Hq), dim3(64), 0, s, (float*)out, (const float*)qkv,
                        q_stride, (const float*)k_cache, (const float*)v_cache, cu, ctx, block_tables, bt_stride, S, Hq,
-                       G, dk, dv, bs, scale, window, chunked, cap, sink, sinks);
+                       G, dk, dv, bs, scale, window, chunked, keep, cap, sink, sinks, (const float*)gate, g_stride);
   else
     hipLaunchKernelGGL(window_prefill_kernel<bf16_t>, dim3(T, Hq), dim3(64), 0, s, (bf16_t*)out, (const bf16_t*)qkv,
                        q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, cu, ctx, block_tables, bt_stride, S,
-                       Hq, G, dk, dv, bs, scale, window, chunked, cap, sink, sinks);
+                       Hq, G, dk, dv, bs, scale, window, chunked, keep, cap, sink, sinks, (const bf16_t*)gate, g_stride);
   return (int)hipGetLastError();
 }
 
 int k8sllm_hy_window_decode(void* out, const void* qkv, long q_stride, const void* k_cache, const void* v_cache,
                             const int* block_tables, int bt_stride, const int* seq_lens, int B, int Hq, int G, int dk,
-                            int dv, int bs, float scale, int window, int chunked, float cap, int sink,
-                            const float* sinks, int f32, int vec, hipStream_t s) {
+                            int dv, int bs, float scale, int window, int chunked, int keep, float cap, int sink,
+                            const float* sinks, const void* gate, long g_stride, int f32, int vec, hipStream_t s) {
   if (B <= 0) return 0;
+  if (keep < 0 || (keep > 0 && (chunked || window <= 0))) return -1;
   if (dk > kGenDK || dv > 64 * kGenVC || G < 1 || Hq % G) return -1;
   const int R = Hq / G;
   if (!f32 && vec && bs == 16 && dk % 8 == 0 && q_stride % 8 == 0 && dk <= kMaxDK && dv <= 64 * kMaxVC &&
@@ -562,7 +597,7 @@ int k8sllm_hy_window_decode(void* out, const void* qkv, long q_stride, const voi
   hipLaunchKernelGGL((window_decode_vec_kernel<RR, (RR == 8 ? 4 : 8)>), dim3(B, G), dim3(RR == 8 ? 256 : 512), 0, s,     \
                      (bf16_t*)out, (const bf16_t*)qkv,                                                                  \
                      q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, bt_stride, seq_lens, Hq, G, \
-                     dk, dv, scale, window, chunked, cap, sink, sinks)
+                     dk, dv, scale, window, chunked, keep, cap, sink, sinks, (const bf16_t*)gate, g_stride)
     if (R == 1) K8SLLM_WD(1);
     else if (R == 2) K8SLLM_WD(2);
     else if (R == 4) K8SLLM_WD(4);
@@ -573,11 +608,11 @@ int k8sllm_hy_window_decode(void* out, const void* qkv, long q_stride, const voi
   if (f32)
     hipLaunchKernelGGL(window_decode_kernel<float>, dim3(B, Hq), dim3(64), 0, s, (float*)out, (const float*)qkv,
                        q_stride, (const float*)k_cache, (const float*)v_cache, block_tables, bt_stride, seq_lens, Hq, G,
-                       dk, dv, bs, scale, window, chunked, cap, sink, sinks);
+                       dk, dv, bs, scale, window, chunked, keep, cap, sink, sinks, (const float*)gate, g_stride);
   else
     hipLaunchKernelGGL(window_decode_kernel<bf16_t>, dim3(B, Hq), dim3(64), 0, s, (bf16_t*)out, (const bf16_t*)qkv,
                        q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, bt_stride, seq_lens, Hq,
-                       G, dk, dv, bs, scale, window, chunked, cap, sink, sinks);
+                       G, dk, dv, bs, scale, window, chunked, keep, cap, sink, sinks, (const bf16_t*)gate, g_stride);
   return (int)hipGetLastError();
 }
 }

@@ -8,7 +8,9 @@ per-head sinks, and ungated experts with a softmax-over-all router; and the gate
 rotary grouped-query attention with per-head temperatures, the fixed-decay linear-attention
 recurrence, gated linear units and the logit soft cap; and layer norms before and after a sublayer,
 token-shift mixes, attention within position chunks with capped scores, the selective scan (a decay per
-channel and state), linear attention with a current-token bonus and the delta rule with a decay per head.
+channel and state), linear attention with a current-token bonus and the delta rule with a decay per head;
+and several residual streams with learned read / mix / write weights, windows that keep the first tokens
+visible, per-head output gates, and routers with a choice correction and identity experts.
 
 GPU tensors run the gfx950 kernels of ``_k8sllm_hybrid`` (``ops/csrc/hybrid``; built by
 ``python -m k8s_llm_monitor_amd.ops.build --only hybrid``) for bfloat16 and float32 activations
@@ -165,6 +167,33 @@ def join_norm(residual: torch.Tensor, branch: tuple, post: Optional[tuple], pre:
     nw, nb = pre if pre is not None else (None, None)
     native().join_norm(out, residual, y[0], y[1], w0, w1, float(mix), pw, pb, nw, nb, float(eps))
     return out
+
+
+def stream_norm(src: torch.Tensor, y: Optional[torch.Tensor], write: Optional[tuple], read: Optional[torch.Tensor],
+                w: torch.Tensor, eps: float, out_dtype: torch.dtype, S: int) -> tuple:
+    """Several residual streams per token.  ``src`` [T, S, d] fp32, or [T, 1, d] for S equal streams (the
+    model's start).  ``y`` [T, d] (any float dtype; None: nothing is written) with ``write`` = (mix [S, S],
+    out [S]) fp32: every stream t becomes ``sum_s mix[s, t] x_s + out[t] y``, all at once from the old ones.
+    Then with ``read`` [S] fp32 (None: all ones) ``u = sum_t read[t] x_t``.  Returns (the RMSNorm of u times
+    ``w`` in ``out_dtype`` [T, d], the new streams [T, S, d] - ``src`` itself, updated in place, where it holds
+    all of them).  Sums and norm are fp32."""
+    T, n, d = src.shape
+    if not src.is_cuda:
+        x = src
+        if y is not None:
+            x = torch.einsum("nsd,st->ntd", src.expand(T, S, d), write[0].float()) + write[1].float().view(1, S, 1) * y.float().unsqueeze(1)
+            if n == S:
+                src.copy_(x)
+                x = src
+        u = x.expand(T, S, d).sum(1) if read is None else torch.einsum("nsd,s->nd", x.expand(T, S, d), read.float())
+        return (u * torch.rsqrt(u.pow(2).mean(-1, keepdim=True) + eps) * w.float()).to(out_dtype), x
+    out = torch.empty(T, d, dtype=out_dtype, device=src.device)
+    dst = None
+    if y is not None:
+        dst = src if n == S else torch.empty(T, S, d, dtype=torch.float32, device=src.device)
+    mix, wo = write if y is not None else (None, None)
+    native().stream_norm(out, dst, src, int(S), y, mix, wo, read, w, float(eps))
+    return out, (dst if dst is not None else src)
 
 
 def token_mix(h: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, seg_cu: torch.Tensor, seg_ctx: torch.Tensor,
@@ -470,15 +499,28 @@ def _first_key(p: int, window: int, chunked: bool) -> int:
     return p - p % window if chunked else max(0, p - window + 1)
 
 
+def _visible(p: int, window: int, chunked: bool, keep: int) -> list:
+    """The positions that a row at position ``p`` sees."""
+    lo = _first_key(p, window, chunked)
+    return list(range(min(keep, lo))) + list(range(lo, p + 1))
+
+
+def _head_gate(o: torch.Tensor, gate: Optional[torch.Tensor], g_col: int) -> torch.Tensor:
+    """o [H, dv] (one row's heads) times sigmoid of that row's gate logits."""
+    return o if gate is None else o * torch.sigmoid(gate[g_col:g_col + o.shape[0]].float()).unsqueeze(-1)
+
+
 def window_attention_prefill(qkv: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, cu: torch.Tensor,
                              ctx: torch.Tensor, block_tables: torch.Tensor, Hq: int, Hkv: int, dk: int, dv: int,
                              scale: float, window: int, sink: bool, mfma: int = 1,
-                             sinks: Optional[torch.Tensor] = None, chunked: bool = False,
-                             cap: float = 0.0) -> torch.Tensor:
+                             sinks: Optional[torch.Tensor] = None, chunked: bool = False, cap: float = 0.0, keep: int = 0,
+                             gate: Optional[torch.Tensor] = None, g_col: int = 0) -> torch.Tensor:
     """Attention of the step's prompt chunks over the paged cache (which already holds their own
     keys): row r of segment s at position p = ctx[s] + r sees positions max(0, p - window + 1) .. p
     (``window`` 0: all of 0 .. p), or with ``chunked`` those of its own chunk of ``window`` positions,
-    p - p % window .. p (chunks count from position 0).  ``cap`` > 0: a score s (after ``scale``) becomes
+    p - p % window .. p (chunks count from position 0).  ``keep``: with a sliding window, the first ``keep``
+    positions of the sequence stay visible too.  ``gate``: rows of a projection [T, *]; head h of a row is
+    multiplied by sigmoid(gate[row, g_col + h]) before it is rounded.  ``cap`` > 0: a score s (after ``scale``) becomes
     ``cap * tanh(s / cap)``.  ``sink``: the softmax denominator has one more term that carries
     no value - exp(0), or exp(sinks[h]) for head h where ``sinks`` [Hq] fp32 is given (a learned,
     unscaled logit).  Scores and weights are fp32.  Returns [T, Hq*dv].  GPU, bf16, head sizes
@@ -496,23 +538,25 @@ def window_attention_prefill(qkv: torch.Tensor, k_cache: torch.Tensor, v_cache: 
             vs = v_cache[bt].permute(0, 3, 1, 2).reshape(-1, Hkv, dv)[:n_all].float()
             for r in range(cul[s], cul[s + 1]):
                 p = ctxl[s] + r - cul[s]
-                lo = _first_key(p, window, chunked)
-                o = _attend(qkv[r, : Hq * dk].float().view(Hq, dk), ks[lo:p + 1], vs[lo:p + 1], scale, sink, sinks, cap)
-                out[r] = o.reshape(-1).to(qkv.dtype)
+                js = _visible(p, window, chunked, keep)
+                o = _attend(qkv[r, : Hq * dk].float().view(Hq, dk), ks[js], vs[js], scale, sink, sinks, cap)
+                out[r] = _head_gate(o, gate[r] if gate is not None else None, g_col).reshape(-1).to(qkv.dtype)
         return out
     out = torch.empty(T, Hq * dv, dtype=qkv.dtype, device=qkv.device)
     native().window_attention_prefill(out, qkv, k_cache, v_cache, cu, ctx, block_tables, Hq, Hkv, dk, dv, float(scale),
-                                      int(window), bool(sink), sinks, int(mfma), bool(chunked), float(cap))
+                                      int(window), bool(sink), sinks, int(mfma), bool(chunked), float(cap), int(keep), gate,
+                                      int(g_col))
     return out
 
 
 def window_attention_decode(qkv: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                             block_tables: torch.Tensor, seq_lens: torch.Tensor, Hq: int, Hkv: int, dk: int, dv: int,
                             scale: float, window: int, sink: bool, vec: bool = True,
-                            sinks: Optional[torch.Tensor] = None, chunked: bool = False,
-                            cap: float = 0.0) -> torch.Tensor:
+                            sinks: Optional[torch.Tensor] = None, chunked: bool = False, cap: float = 0.0, keep: int = 0,
+                            gate: Optional[torch.Tensor] = None, g_col: int = 0) -> torch.Tensor:
     """One query per sequence (its newest token, already in the cache) over the last ``window``
-    cached positions (``chunked``: those of its own chunk; ``cap``: as in window_attention_prefill);
+    cached positions (``chunked``: those of its own chunk; ``cap``, ``keep``, ``gate``: as in
+    window_attention_prefill);
     ``seq_lens`` count that token (0: a padding row, output zero)."""
     B = qkv.shape[0]
     if not qkv.is_cuda:
@@ -521,16 +565,17 @@ def window_attention_decode(qkv: torch.Tensor, k_cache: torch.Tensor, v_cache: t
         for b, n in enumerate(seq_lens.tolist()):
             if n <= 0:
                 continue
-            lo = _first_key(n - 1, window, chunked)
+            js = _visible(n - 1, window, chunked, keep)
             bt = block_tables[b, : (n + bs - 1) // bs].long()
-            ks = k_cache[bt].reshape(-1, Hkv, dk)[lo:n].float()
-            vs = v_cache[bt].permute(0, 3, 1, 2).reshape(-1, Hkv, dv)[lo:n].float()
-            out[b] = _attend(qkv[b, : Hq * dk].float().view(Hq, dk), ks, vs, scale, sink,
-                             sinks, cap).reshape(-1).to(qkv.dtype)
+            ks = k_cache[bt].reshape(-1, Hkv, dk)[js].float()
+            vs = v_cache[bt].permute(0, 3, 1, 2).reshape(-1, Hkv, dv)[js].float()
+            o = _attend(qkv[b, : Hq * dk].float().view(Hq, dk), ks, vs, scale, sink, sinks, cap)
+            out[b] = _head_gate(o, gate[b] if gate is not None else None, g_col).reshape(-1).to(qkv.dtype)
         return out
     out = torch.empty(B, Hq * dv, dtype=qkv.dtype, device=qkv.device)
     native().window_attention_decode(out, qkv, k_cache, v_cache, block_tables, seq_lens, Hq, Hkv, dk, dv, float(scale),
-                                     int(window), bool(sink), sinks, bool(vec), bool(chunked), float(cap))
+                                     int(window), bool(sink), sinks, bool(vec), bool(chunked), float(cap), int(keep), gate,
+                                     int(g_col))
     return out
 
 
@@ -641,11 +686,12 @@ def _no_sink(H: int, device) -> torch.Tensor:
 def latent_attention(qa: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor,
                      H: int, scale: float, window: int, sinks: Optional[torch.Tensor], cu: Optional[torch.Tensor] = None,
                      ctx: Optional[torch.Tensor] = None, seq_lens: Optional[torch.Tensor] = None, fast: int = 1,
-                     split: int = 0, sink: bool = True) -> torch.Tensor:
+                     split: int = 0, sink: bool = True, gate: Optional[torch.Tensor] = None, g_col: int = 0) -> torch.Tensor:
     """Attention of ``qa`` [T, H * pitch] (latent_queries) over the latent pages: every head reads
     the one key stream ``k_cache`` [blocks, bs, pitch] and the one value stream ``v_cache`` [blocks, 1,
     kv_rank, bs]; sliding window and learned sinks as in window_attention_* (``sink`` False: an
-    ordinary softmax, nothing but the keys in the denominator).  ``cu`` / ``ctx``: prompt
+    ordinary softmax, nothing but the keys in the denominator).  ``gate``: a sigmoid gate per row and head, as in
+    window_attention_prefill.  ``cu`` / ``ctx``: prompt
     chunks (rows of segment s at positions ctx[s] ..); else ``seq_lens``: one row per sequence, at its
     newest token.  Returns [T, H * kv_rank].  GPU, bf16, pitch a multiple of 32 up to 320 and kv_rank a
     multiple of 16 up to 256 (``fast``): the matrix-core kernel, 16 heads of one token per tile
@@ -662,12 +708,13 @@ def latent_attention(qa: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
         # so low that its weight exp(logit - max) is exactly zero in fp32
         sk = sinks if sink else _no_sink(H, qa.device)
         if native().latent_attention(out, qa, k_cache, v_cache, cu, ctx, seq_lens, block_tables, int(H), float(scale),
-                                     int(window), sk, int(split)):
+                                     int(window), sk, int(split), gate, int(g_col)):
             return out
     args = (H, 1, pitch, dv, scale, window, bool(sink))
+    kw = dict(sinks=sinks, gate=gate, g_col=g_col)
     if cu is not None:
-        return window_attention_prefill(qa, k_cache, v_cache, cu, ctx, block_tables, *args, mfma=fast, sinks=sinks)
-    return window_attention_decode(qa, k_cache, v_cache, block_tables, seq_lens, *args, vec=bool(fast), sinks=sinks)
+        return window_attention_prefill(qa, k_cache, v_cache, cu, ctx, block_tables, *args, mfma=fast, **kw)
+    return window_attention_decode(qa, k_cache, v_cache, block_tables, seq_lens, *args, vec=bool(fast), **kw)
 
 
 # ---------------------------------------------------------------- Mamba-2
@@ -955,29 +1002,34 @@ def moe_router(h: torch.Tensor, wr: torch.Tensor, bias: Optional[torch.Tensor], 
     return ids, wts, gate
 
 
-def moe_router_grouped(h: torch.Tensor, wr: torch.Tensor, E: int, K: int, groups: int, keep: int,
-                       scale: float) -> tuple:
-    """fp32 router with sigmoid scores and a choice restricted to groups: ``s = sigmoid(wr h)``; the E
-    experts form ``groups`` equal groups of neighbours, a group's score is the sum of its two largest
-    scores (its one score where a group is one expert), and only experts of the ``keep`` best groups
-    can be chosen; the ``K`` largest scores among those are taken (lowest index wins a tie) and
-    weighted ``s / (sum of the chosen s + 1e-20) * scale``.  Returns (ids [T, K] int32, weights [T, K] fp32)."""
+def moe_router_grouped(h: torch.Tensor, wr: torch.Tensor, E: int, K: int, groups: int, keep: int, scale: float,
+                       soft: bool = False, corr: Optional[torch.Tensor] = None, best2: bool = True,
+                       renorm: bool = True) -> tuple:
+    """fp32 router whose choice is restricted to groups.  Scores ``s = sigmoid(wr h)``, or with ``soft`` the
+    softmax over all E logits; choice scores ``s + corr`` (``corr`` [E] fp32, None: zeros - they may be
+    negative).  The E experts form ``groups`` equal groups of neighbours; a group counts as the sum of its two
+    largest choice scores (its one where a group is one expert), or without ``best2`` as its largest; only
+    experts of the ``keep`` best groups can be chosen.  The ``K`` largest choice scores among those are taken
+    (lowest index wins a tie) and weighted ``s / (sum of the chosen s + 1e-20) * scale``, or without
+    ``renorm`` ``s * scale``.  Returns (ids [T, K] int32, weights [T, K] fp32)."""
     T = h.shape[0]
     if not h.is_cuda:
-        sc = torch.sigmoid(h.float() @ wr.float().t())
-        masked = sc
+        lg = h.float() @ wr.float().t()
+        sc = torch.softmax(lg, -1) if soft else torch.sigmoid(lg)
+        choice = sc if corr is None else sc + corr.float()
         if groups > 1:
             per = E // groups
-            gs = sc.view(T, groups, per).topk(min(2, per), dim=-1).values.sum(-1)
+            gs = choice.view(T, groups, per).topk(min(2, per) if best2 else 1, dim=-1).values.sum(-1)
             best = gs.topk(keep, dim=-1).indices
             ok = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, best, True)
-            masked = torch.where(ok.repeat_interleave(per, dim=1), sc, torch.full_like(sc, -1.0))
-        idx = masked.topk(K, dim=-1).indices
+            choice = torch.where(ok.repeat_interleave(per, dim=1), choice, torch.full_like(sc, -math.inf))
+        idx = choice.topk(K, dim=-1).indices
         w = sc.gather(1, idx)
-        return idx.to(torch.int32), w / (w.sum(-1, keepdim=True) + 1e-20) * scale
+        return idx.to(torch.int32), (w / (w.sum(-1, keepdim=True) + 1e-20) if renorm else w) * scale
     ids = torch.empty(T, K, dtype=torch.int32, device=h.device)
     wts = torch.empty(T, K, dtype=torch.float32, device=h.device)
-    native().moe_router_grouped(ids, wts, h, wr, int(E), int(K), int(groups), int(keep), float(scale))
+    native().moe_router_grouped(ids, wts, h, wr, corr, int(E), int(K), int(groups), int(keep), float(scale), bool(soft), bool(best2),
+                                bool(renorm))
     return ids, wts
 
 
@@ -988,12 +1040,14 @@ TILE_MIN_ROWS = 1024
 
 def moe_experts(h: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor,
                 shared: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None, il: bool = False,
-                mfma: bool = True, act: str = "swiglu", limit: float = 0.0, tile: bool = False) -> torch.Tensor:
+                mfma: bool = True, act: str = "swiglu", limit: float = 0.0, tile: bool = False,
+                identity: int = 0) -> torch.Tensor:
     """Sum over each token's chosen experts of ``wts * down_e(silu(gate_e h) * up_e h)`` with
     ``w13`` [E, 2*ff, d] (gate rows then up rows; ``il``: interleaved per 128 rows as [64 gate |
     64 up], ops.interleave_gate_up) and ``w2`` [E, d, ff], plus ``gate * shared`` (the shared
     expert's output [T, d] and its per-token gate; ``gate`` None: 1).  ``act`` "gelu": ungated
-    experts ``down_e(gelu(up_e h))`` with ``w13`` [E, ff, d].  ``act`` "clamped_swish": gated experts whose
+    experts ``down_e(gelu(up_e h))`` with ``w13`` [E, ff, d]; "relu_sq": the same with the squared ReLU.
+    ``identity``: ids E .. E + identity - 1 are experts whose output is h itself.  ``act`` "clamped_swish": gated experts whose
     unit is ``g * sigmoid(1.702 g) * (u + 1)`` with g = min(gate_e h, limit), u = clamp(up_e h, -limit,
     limit).  fp32 [T, d].
 
@@ -1016,28 +1070,32 @@ def moe_experts(h: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w13: torc
                 if il:
                     we = we.view(ff // 64, 2, 64, d).permute(1, 0, 2, 3).reshape(2 * ff, d)
                 gu = (hf[rows] @ we.t()).to(h.dtype).float()
-                if act == "gelu":
-                    a = F.gelu(gu).to(h.dtype).float()
+                if act in ("gelu", "relu_sq"):
+                    a = _act_torch(gu, act).to(h.dtype).float()
                 elif act == "clamped_swish":
                     a = _clamped_unit(gu[:, :ff], gu[:, ff:], limit).to(h.dtype).float()
                 else:
                     a = (_silu(gu[:, :ff]) * gu[:, ff:]).to(h.dtype).float()
                 out.index_add_(0, rows, (a @ w2[e].float().t()).to(h.dtype).float() * wts[rows, slot].unsqueeze(-1))
+        if identity:
+            out += hf * (wts * (ids >= E)).sum(-1, keepdim=True)
         if shared is not None:
             out += shared.float() * gate.unsqueeze(-1) if gate is not None else shared.float()
         return out
     ext = native()
     n = T * K
-    offsets = torch.empty(E + 1, dtype=torch.int32, device=h.device)
+    # identity experts sort behind the others: the GEMMs run over the first E experts' rows only
+    offsets = torch.empty(E + identity + 1, dtype=torch.int32, device=h.device)
     sorted_idx = torch.empty(n, dtype=torch.int32, device=h.device)
     inv_idx = torch.empty(n, dtype=torch.int32, device=h.device)
-    ext.moe_align(ids, E, offsets, sorted_idx, inv_idx)
-    code = {"swiglu": 1, "gelu": 2, "clamped_swish": 3}[act]
-    if act == "gelu" and n >= TILE_MIN_ROWS and h.dtype == torch.bfloat16 and ff % 256 == 0 and d % 256 == 0:
-        from .. import ops  # large steps of plain experts: the prefill tile GEMM twice, GELU between
+    ext.moe_align(ids, E + identity, offsets, sorted_idx, inv_idx)
+    offsets = offsets[:E + 1]
+    code = {"swiglu": 1, "gelu": 2, "clamped_swish": 3, "relu_sq": 4}[act]
+    if act in ("gelu", "relu_sq") and n >= TILE_MIN_ROWS and h.dtype == torch.bfloat16 and ff % 256 == 0 and d % 256 == 0:
+        from .. import ops  # large steps of plain experts: the prefill tile GEMM twice, the activation between
 
         xs = ops.gather_rows(h, sorted_idx, K)
-        a = activation(ops.moe_grouped_gemm(xs, w13, offsets, zero_fill=False), "gelu")
+        a = activation(ops.moe_grouped_gemm(xs, w13, offsets, zero_fill=False), act)
         ys = ops.moe_grouped_gemm(a, w2, offsets, zero_fill=False)
     elif act == "clamped_swish" and tile and n >= TILE_MIN_ROWS and h.dtype == torch.bfloat16:
         from .. import ops  # large steps: the prefill tile GEMM twice, the clamped unit as a launch between
@@ -1057,7 +1115,7 @@ def moe_experts(h: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor, w13: torc
         ys = torch.empty(n, d, dtype=h.dtype, device=h.device)
         ext.grouped_gemm(ys, a, w2, offsets, None, 1, 0, False, mfma, 0.0)
     out = torch.empty(T, d, dtype=torch.float32, device=h.device)
-    ext.moe_combine(out, ys, inv_idx, wts, shared, gate)
+    ext.moe_combine(out, ys, inv_idx, wts, shared, gate, ids if identity else None, h if identity else None, E)
     return out
 
 

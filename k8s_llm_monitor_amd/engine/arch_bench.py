@@ -10,7 +10,10 @@ or the gated delta rule in every layer, routed clamped experts) beside a Dunesun
 attention layer with the same experts and one Mamba-2 layer of equal state size for every Levovik
 layer; Dopivik (selective scan, wkv, and attention beside the delta rule, in turn, norms on both sides of
 every sublayer) beside a Dunesun model with a Mamba-2 layer of equal state size for every recurrence and
-an attention layer with the same heads and window size for every attention.  Both models run through the same
+an attention layer with the same heads and window size for every attention; Zifisun (latent attention and
+windowed attention in turn, several residual streams, experts beside identity experts) beside a
+Kisutar model of the same two kinds of attention with the same heads, head sizes, windows and
+experts in every layer.  Both models run through the same
 ModelRunner step functions the engine uses: one prefill step of ``seqs`` whole prompts, then decode
 steps of ``batch`` sequences (hipGraph replay where the model's decode is captured)."""
 from __future__ import annotations
@@ -212,8 +215,39 @@ def _dopivik_pair(size: str, window: int) -> tuple:
     return new, ref
 
 
+# Zifisun: (name, width, heads, kv heads, head dim, latent unrotated dim, rotated dim, value dim, q rank, kv rank,
+#           experts, identity experts, top, expert ff, shared ff, streams, kept first tokens, layers)
+ZIFISUN_SIZES = {
+    "s": ("d1024", 1024, 8, 2, 128, 96, 32, 128, 384, 128, 8, 4, 2, 1024, 1024, 4, 4, 4),
+    "m": ("d2048", 2048, 16, 4, 128, 96, 32, 128, 768, 256, 8, 4, 2, 2048, 2048, 4, 4, 4),
+    "l": ("d4096", 4096, 32, 8, 128, 96, 32, 128, 1536, 256, 8, 4, 2, 3584, 3584, 4, 4, 2),
+}
+
+
+def _zifisun_pair(size: str, window: int) -> tuple:
+    """Zifisun (latent attention and first-token-keeping windowed attention in turn, routed feed-forwards with a
+    shared expert) and a Kisutar model with the same two kinds of attention, heads, windows and experts
+    (one residual stream with token shift and depth average, no identity experts)."""
+    name, d, H, G, D, dn, dr, dv, Q, R, E, ident, K, ff, fs, streams, keep, L = ZIFISUN_SIZES[size]
+    flat = lambda m: tuple(sorted(m.items()))
+    lat = {"heads": H, "dim": dn, "rot_dim": dr, "vdim": dv, "q_rank": Q, "kv_rank": R, "mask.size": window,
+           "scale": (dn + dr) ** -0.5, "rot.base": 10000.0, "rot.dims": dr}
+    att = {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "mask.size": window, "scale": D ** -0.5}
+
+    def layers(extra, mlp):
+        return tuple(LayerSpec("latent_attention", flat(lat), mlp) if i % 2 == 0 else
+                     LayerSpec("attention", flat(dict(att, **extra)), mlp) for i in range(L))
+
+    new = HybridConfig(name=f"zifisun-{name}", arch="zifisun", vocab_size=32000, d_model=d,
+                       layers=layers({"mask.keep_first": keep}, MoESpec(E, K, ff, fs, groups=2, keep_groups=1, identity=ident)),
+                       max_position=8192, norm_eps=1e-6, streams=streams)
+    ref = HybridConfig(name=f"kisutar-mixed-{name}", arch="kisutar", vocab_size=32000, d_model=d,
+                       layers=layers({}, MoESpec(E, K, ff, fs)), max_position=8192, norm_eps=1e-6)
+    return new, ref
+
+
 PAIRS = {"dunesun": _pair, "kisutar": _kisutar_pair, "bitonex": _bitonex_pair, "levovik": _levovik_pair,
-         "dopivik": _dopivik_pair}
+         "dopivik": _dopivik_pair, "zifisun": _zifisun_pair}
 
 
 def _measure(cfg, seqs: int, prompt: int, batch: int, steps: int, warmup: int, graphs: bool) -> dict:

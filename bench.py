@@ -22,7 +22,7 @@ Modes (``--mode``):
   Mixtral-style model, ``kisutar``: beside an all-attention Dunesun model, ``bitonex``: beside a Dunesun
   model of attention and Mamba-2 layers, ``levovik``: beside a Dunesun model with an attention and a Mamba-2
   layer for each of its layers, ``dopivik``: beside a Dunesun model with a Mamba-2 layer per recurrence
-  and an attention layer per attention), one GPU, random weights.
+  and an attention layer per attention, ``zifisun``: beside a Kisutar model of the same kinds of attention), one GPU, random weights.
 ``--production``: the server runs with the reference's timeouts (15 s write, 30 s llm.timeout)
 instead of the bench's 600 s; answers that reach the deadline come back truncated
 (finish_reason "deadline") and overload as 503 - both are counted in the JSON line.
@@ -73,7 +73,7 @@ def parse(argv=None):
     ap.add_argument("--arch-seqs", type=int, default=4, help="arch: prompts in the prefill step")
     ap.add_argument("--arch-window", type=int, default=1024, help="arch: the Dunesun attention layers' window")
     ap.add_argument("--arch-which", choices=["both", "new", "ref"], default="both")
-    ap.add_argument("--arch-design", choices=["dunesun", "kisutar", "bitonex", "levovik", "dopivik"], default="dunesun",
+    ap.add_argument("--arch-design", choices=["dunesun", "kisutar", "bitonex", "levovik", "dopivik", "zifisun"], default="dunesun",
                     help="arch: the layer-list design to measure beside its closest existing model")
     ap.add_argument("--rate", type=float, default=16.0, help="poisson: arrivals per second per replica")
     ap.add_argument("--production", action="store_true",

@@ -240,6 +240,113 @@ __global__ __launch_bounds__(256) void hy_router_grouped_kernel(int* __restrict_
   }
 }
 
+// The same for large steps with few experts (E <= NACC <= 16, d a multiple of 8): a workgroup takes TT = 4 tokens, so
+// that every weight row is read once for four of them, and wave w finishes token w on its own (lane = expert
+// or group; a wave's LDS instructions execute in issue order).
+template <typename T, int NACC>
+__global__ __launch_bounds__(256) void hy_router_grouped4_kernel(int* __restrict__ ids, float* __restrict__ wts,
+                                                                 const T* __restrict__ h, long rows, int d,
+                                                                 const float* __restrict__ wr,
+                                                                 const float* __restrict__ corr, int E, int K,
+                                                                 int groups, int keep, float scale, int soft, int best2,
+                                                                 int renorm) {
+  constexpr int TT = 4;
+  __shared__ float part[4][TT][NACC];
+  __shared__ float sc[TT][NACC], ch[TT][NACC], gsc[TT][NACC];
+  __shared__ int gok[TT][NACC], sel[TT][NACC];
+  const long t0 = (long)blockIdx.x * TT;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  float acc[TT][NACC];
+#pragma unroll
+  for (int q = 0; q < TT; ++q)
+#pragma unroll
+    for (int e = 0; e < NACC; ++e) acc[q][e] = 0.f;
+  for (int c = tid * 8; c < d; c += 2048) {
+    float xv[TT][8];
+#pragma unroll
+    for (int q = 0; q < TT; ++q) load8(h + min(t0 + q, rows - 1) * d + c, xv[q]);
+#pragma unroll
+    for (int e = 0; e < NACC; ++e)
+      if (e < E) {
+        float w[8];
+        load8(wr + (long)e * d + c, w);
+#pragma unroll
+        for (int q = 0; q < TT; ++q)
+#pragma unroll
+          for (int i = 0; i < 8; ++i) acc[q][e] += xv[q][i] * w[i];
+      }
+  }
+#pragma unroll
+  for (int q = 0; q < TT; ++q)
+#pragma unroll
+    for (int e = 0; e < NACC; ++e) {
+      const float v = wave_sum_dpp(acc[q][e]);
+      if (lane == 0) part[wave][q][e] = v;
+    }
+  __syncthreads();
+  const long t = t0 + wave;
+  const int ec = min(lane, NACC - 1), per = E / groups;
+  const bool live = lane < E;
+  const float z = part[0][wave][ec] + part[1][wave][ec] + part[2][wave][ec] + part[3][wave][ec];
+  float s;
+  if (soft) {
+    const float mx = wave_max_dpp(live ? z : -INFINITY);
+    const float p = live ? expf(z - mx) : 0.f;
+    s = p / wave_sum_dpp(p);
+  } else {
+    s = 1.f / (1.f + expf(-z));
+  }
+  float c = corr != nullptr && live ? s + corr[ec] : s;
+  c = c == c ? c : -INFINITY;  // a strict order whatever the input
+  if (live) {
+    sc[wave][lane] = s;
+    ch[wave][lane] = c;
+  }
+  __builtin_amdgcn_wave_barrier();
+  bool able = live;
+  if (keep < groups) {
+    float gv = -INFINITY;
+    if (lane < groups) {
+      float m1 = -INFINITY, m2 = -INFINITY;
+      for (int e = lane * per; e < (lane + 1) * per; ++e) {
+        const float v = ch[wave][e];
+        if (v > m1) {
+          m2 = m1;
+          m1 = v;
+        } else if (v > m2) {
+          m2 = v;
+        }
+      }
+      gv = best2 && per > 1 ? m1 + m2 : m1;
+      gsc[wave][lane] = gv;
+    }
+    __builtin_amdgcn_wave_barrier();
+    if (lane < groups) {
+      int rank = 0;
+      for (int g = 0; g < groups; ++g) rank += (gsc[wave][g] > gv || (gsc[wave][g] == gv && g < lane)) ? 1 : 0;
+      gok[wave][lane] = rank < keep;
+    }
+    __builtin_amdgcn_wave_barrier();
+    able = live && gok[wave][ec / per];
+  }
+  if (able) {
+    int rank = 0;
+    for (int e = 0; e < E; ++e)
+      if (keep == groups || gok[wave][e / per]) rank += (ch[wave][e] > c || (ch[wave][e] == c && e < lane)) ? 1 : 0;
+    if (rank < K) sel[wave][rank] = lane;
+  }
+  __builtin_amdgcn_wave_barrier();
+  if (lane < K && t < rows) {
+    float n = 1.f;
+    if (renorm) {
+      n = 1e-20f;
+      for (int k = 0; k < K; ++k) n += sc[wave][sel[wave][k]];
+    }
+    ids[t * K + lane] = sel[wave][lane];
+    wts[t * K + lane] = sc[wave][sel[wave][lane]] / n * scale;
+  }
+}
+
 constexpr int TM = 64, TN = 64, TK = 16;
 
 __device__ __forceinline__ float gelu_erf_f(float z) { return 0.5f * z * (1.f + erff(z * 0.70710678118654752f)); }
@@ -481,13 +588,25 @@ int k8sllm_hy_router_grouped(int* ids, float* wts, const void* h, long T, int d,
   if (E > kMaxE || K > kMaxK || K < 1 || groups < 1 || E % groups || keep < 1 || keep > groups ||
       K > keep * (E / groups))
     return -1;
+  if (T >= 1024 && E <= 16 && d % 8 == 0) {
+#define K8SLLM_R4(T_, NACC)                                                                                        \
+  hipLaunchKernelGGL((hy_router_grouped4_kernel<T_, NACC>), dim3((unsigned)((T + 3) / 4)), dim3(256), 0, s, ids, wts, \
+                     (const T_*)h, T, d, wr, corr, E, K, groups, keep, scale, soft, best2, renorm)
+    if (f32) {
+      if (E <= 8) K8SLLM_R4(float, 8); else if (E <= 12) K8SLLM_R4(float, 12); else K8SLLM_R4(float, 16);
+    } else {
+      if (E <= 8) K8SLLM_R4(bf16_t, 8); else if (E <= 12) K8SLLM_R4(bf16_t, 12); else K8SLLM_R4(bf16_t, 16);
+    }
+#undef K8SLLM_R4
+    return (int)hipGetLastError();
+  }
 #define K8SLLM_RG(T_, NACC)                                                                                        \
   hipLaunchKernelGGL((hy_router_grouped_kernel<T_, NACC>), dim3(T), dim3(256), 0, s, ids, wts, (const T_*)h, d, wr, corr, \
                      E, K, groups, keep, scale, soft, best2, renorm)
   if (f32) {
-    if (E <= 8) K8SLLM_RG(float, 8); else if (E <= 16) K8SLLM_RG(float, 16); else K8SLLM_RG(float, 0);
+    if (E <= 8) K8SLLM_RG(float, 8); else if (E <= 12) K8SLLM_RG(float, 12); else if (E <= 16) K8SLLM_RG(float, 16); else K8SLLM_RG(float, 0);
   } else {
-    if (E <= 8) K8SLLM_RG(bf16_t, 8); else if (E <= 16) K8SLLM_RG(bf16_t, 16); else K8SLLM_RG(bf16_t, 0);
+    if (E <= 8) K8SLLM_RG(bf16_t, 8); else if (E <= 12) K8SLLM_RG(bf16_t, 12); else if (E <= 16) K8SLLM_RG(bf16_t, 16); else K8SLLM_RG(bf16_t, 0);
   }
 #undef K8SLLM_RG
   return (int)hipGetLastError();

@@ -146,10 +146,19 @@ __global__ __launch_bounds__(NT) void moe_align_kernel(const int* __restrict__ i
   __shared__ int cnt[ME][NT];
   __shared__ int wsum[NT / 64];
   const int t = threadIdx.x;
-  const long C = (n + NT - 1) / NT;
-  const long b0 = t * C, b1 = min(n, b0 + C);
+  // a thread's items: a multiple of 4, so that ids are read (and inv_idx written) 16 bytes at a time
+  const long C = ((n + NT - 1) / NT + 3) & ~3L;
+  const long b0 = min(n, t * C), b1 = min(n, b0 + C), b4 = b0 + ((b1 - b0) & ~3L);
   for (int e = 0; e < E; ++e) cnt[e][t] = 0;
-  for (long i = b0; i < b1; ++i) cnt[ids[i]][t] += 1;
+#pragma unroll 4
+  for (long i = b0; i < b4; i += 4) {
+    const int4 e = *reinterpret_cast<const int4*>(ids + i);
+    cnt[e.x][t] += 1;
+    cnt[e.y][t] += 1;
+    cnt[e.z][t] += 1;
+    cnt[e.w][t] += 1;
+  }
+  for (long i = b4; i < b1; ++i) cnt[ids[i]][t] += 1;
   __syncthreads();
   int base = 0;
   for (int e = 0; e < E; ++e) {
@@ -160,9 +169,22 @@ __global__ __launch_bounds__(NT) void moe_align_kernel(const int* __restrict__ i
     base += tot;
   }
   if (t == 0) offsets[E] = base;
-  for (long i = b0; i < b1; ++i) {
-    const int e = ids[i];
-    const int pos = cnt[e][t]++;
+#pragma unroll 4
+  for (long i = b0; i < b4; i += 4) {
+    const int4 e = *reinterpret_cast<const int4*>(ids + i);
+    int4 pos;
+    pos.x = cnt[e.x][t]++;
+    pos.y = cnt[e.y][t]++;
+    pos.z = cnt[e.z][t]++;
+    pos.w = cnt[e.w][t]++;
+    sorted_idx[pos.x] = (int)i;
+    sorted_idx[pos.y] = (int)i + 1;
+    sorted_idx[pos.z] = (int)i + 2;
+    sorted_idx[pos.w] = (int)i + 3;
+    *reinterpret_cast<int4*>(inv_idx + i) = pos;
+  }
+  for (long i = b4; i < b1; ++i) {
+    const int pos = cnt[ids[i]][t]++;
     sorted_idx[pos] = (int)i;
     inv_idx[i] = pos;
   }

@@ -319,6 +319,15 @@ def test_moe_route_align_combine():
     _close(y, ref.moe_combine(xs.cpu(), inv.cpu(), w.cpu(), T).to(DEV), atol=2e-2, rtol=1e-2, what="combine")
 
 
+@pytest.mark.parametrize("T,E,K", [(1, 1, 1), (3, 8, 1), (301, 8, 2), (1023, 16, 3), (1366, 12, 3), (5003, 5, 1), (777, 40, 3), (517, 200, 3)])
+def test_moe_align_sizes(T, E, K):
+    """Item counts that are multiples of nothing, fewer items than threads, every counter layout."""
+    ids = torch.randint(0, E, (T, K), generator=torch.Generator().manual_seed(T), dtype=torch.int32)
+    got = ops.moe_align(ids.to(DEV), E)
+    for a, b in zip(got, ref.moe_align(ids, E)):
+        assert torch.equal(a.cpu(), b)
+
+
 @pytest.mark.parametrize("splits", [1, 4, 7])
 @pytest.mark.parametrize("M,N,K", [(1, 256, 512), (7, 4096, 4096), (16, 128, 1024), (33, 640, 14336),
                                    (64, 4096, 4096), (50, 6144, 4096)])

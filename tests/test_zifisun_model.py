@@ -710,11 +710,32 @@ def test_gpu_router_choice(E, K, groups, keep, shift):
 
 
 @pytest.mark.gpu
+@pytest.mark.parametrize("E,K,groups,keep", [r for r in ROUTES if r[0] <= 16])
+def test_gpu_router_choice_in_large_steps(E, K, groups, keep):
+    """From 1024 rows on a workgroup takes four tokens (here also a last, partly filled one)."""
+    h, wr, corr = _route_case(E, 72, 1027, E, -1.0)
+    for dtype in (torch.float32, torch.bfloat16):
+        hd = h.to(dtype)
+        got = [hops.moe_router_grouped(hd[:n].cuda(), wr.cuda(), E, K, groups, keep, 1.3, soft=True, corr=corr.cuda(), best2=False, renorm=False)
+               for n in (1027, 1000)]
+        assert torch.equal(got[0][0][:1000], got[1][0])  # against the one-token workgroups
+        close(got[0][1][:1000].cpu(), got[1][1].double().cpu(), tol=2e-5)
+        wi, ww = _route_want(hd[1000:].float(), wr, corr, K, groups, keep)
+        assert torch.equal(got[0][0][1000:].cpu(), wi)
+        close(got[0][1][1000:].cpu(), ww * 1.3, tol=2e-5)
+        a = hops.moe_router_grouped(hd.cuda(), wr.cuda(), E, K, groups, keep, 0.7)
+        b = hops.moe_router_grouped(hd[:1000].cuda(), wr.cuda(), E, K, groups, keep, 0.7)
+        assert torch.equal(a[0][:1000], b[0])
+        close(a[1][:1000].cpu(), b[1].double().cpu(), tol=2e-5)
+
+
+@pytest.mark.gpu
 def test_gpu_router_gives_valid_experts_for_any_input():
     """Not-a-number rows still get K different experts of the list (nothing indexes by an undefined id)."""
     h = torch.randn(6, 16)
     h[2], h[4, 3] = float("nan"), float("inf")
-    for E, K, groups, keep in ((12, 3, 4, 2), (5, 5, 1, 1)):
+    for E, K, groups, keep, rep in ((12, 3, 4, 2, 1), (5, 5, 1, 1, 1), (12, 3, 4, 2, 200), (5, 5, 1, 1, 200)):
+        h = h.repeat(rep, 1)
         ids, _ = hops.moe_router_grouped(h.cuda(), torch.randn(E, 16).cuda(), E, K, groups, keep, 1.0, soft=True, corr=torch.randn(E).cuda(),
                                          best2=False, renorm=False)
         ids = ids.cpu()

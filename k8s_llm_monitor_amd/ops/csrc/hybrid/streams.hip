@@ -1,5 +1,5 @@
 // Several residual streams per token, mixed around every sublayer with learned weights.
-//   stream_norm   x_t <- sum_s mix[s][t] x_s + out[t] * y  (all streams at once, from the old ones), then
+//   stream_norm   x_t <- sum_s mix[s][t] x_s + out[t] * y  (the right-hand side reads the streams before the step), then
 //                 u = sum_t in[t] x_t  and  h = u / rms(u) * w: what the sublayer just run leaves and what the
 //                 next one reads, in one launch
 // src: the streams [rows][S][d] fp32 (contiguous per token), or one row per token that stands for all S equal

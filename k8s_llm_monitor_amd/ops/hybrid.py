@@ -173,7 +173,7 @@ def stream_norm(src: torch.Tensor, y: Optional[torch.Tensor], write: Optional[tu
                 w: torch.Tensor, eps: float, out_dtype: torch.dtype, S: int) -> tuple:
     """Several residual streams per token.  ``src`` [T, S, d] fp32, or [T, 1, d] for S equal streams (the
     model's start).  ``y`` [T, d] (any float dtype; None: nothing is written) with ``write`` = (mix [S, S],
-    out [S]) fp32: every stream t becomes ``sum_s mix[s, t] x_s + out[t] y``, all at once from the old ones.
+    out [S]) fp32: every stream t becomes ``sum_s mix[s, t] x_s + out[t] y`` of the streams before.
     Then with ``read`` [S] fp32 (None: all ones) ``u = sum_t read[t] x_t``.  Returns (the RMSNorm of u times
     ``w`` in ``out_dtype`` [T, d], the new streams [T, S, d] - ``src`` itself, updated in place, where it holds
     all of them).  Sums and norm are fp32."""
